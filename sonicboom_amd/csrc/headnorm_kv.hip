@@ -1,9 +1,12 @@
-// Queries and keys normed per head, values mixed with an earlier layer's, keys and values stored.
+// Queries and keys rotated and normed per head, values mixed with an earlier layer's, keys and values stored.
 //
 // From the float32 rows of a stacked product [q: heads_q x dk | k: heads_kv x dk | v: heads_kv x dv]
 // (whole, or in K slices that are added here in ascending order):
-//   every head of q and k is divided by its root mean square (eps inside the root) and multiplied by
-//   a weight of the head's size that the heads share (NULL: the head passes as it is);
+//   with inv_freq the pairs (i, i + rot_dims / 2) of the first rot_dims numbers of every head of q and k
+//   turn by position * inv_freq[i];
+//   every head of q and k is then divided by its root mean square (eps inside the root) and multiplied by
+//   a weight of the head's size that the heads share (NULL: the head passes as it is, or, with `unit`, is
+//   divided without a weight);
 //   v <- (1 - lam) v + lam v_first when v_first is given (lam one number in memory), and the v of
 //   before the mixing is written to v_out when that is given (the first mixing layer's);
 //   q goes out in the activation type, k and v into the page of the row's position.
@@ -22,7 +25,30 @@ struct Args {
   const int32_t *row_pos, *row_seq, *page_table; int max_pages, n_pages;
   void *k_cache, *v_cache;
   int heads_q, heads_kv, dk, dv, store;
+  const float *inv_freq; int rot_dims; int unit;
 };
+
+// cosines and sines of the row's position, once per block
+__device__ __forceinline__ void row_angles(const Args &a, int row, float *cs, float *sn) {
+  const int half = a.rot_dims / 2;
+  const float pos = float(a.row_pos[row]);
+  for (int j = threadIdx.x; j < 2 * half; j += blockDim.x) {
+    const int i = j < half ? j : j - half;
+    const float theta = pos * a.inv_freq[i];
+    if (j < half) cs[i] = cosf(theta);
+    else sn[i] = sinf(theta);
+  }
+  __syncthreads();
+}
+
+// number d of a head after its pair has turned; other: the pair's other number
+__device__ __forceinline__ float turned(float v, float other, int d, int half, const float *cs, const float *sn) {
+  const int i = d < half ? d : d - half;
+  float y0, y1;
+  if (d < half) rotate_pair(v, other, cs[i], sn[i], y0, y1);
+  else rotate_pair(other, v, cs[i], sn[i], y0, y1);
+  return d < half ? y0 : y1;
+}
 
 constexpr int kMaxSlices = 8;      // slices whose loads the unrolled loops ask for together (more: the plain loop)
 
@@ -48,6 +74,9 @@ template <typename TQ, typename TC, int THREADS>
 __global__ void __launch_bounds__(THREADS) headnorm_kv_store_kernel(Args a) {
   const int row = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const float *src = a.qkv + size_t(row) * a.row_stride;
+  __shared__ float cs[kMaxHead / 2], sn[kMaxHead / 2];
+  if (a.inv_freq) row_angles(a, row, cs, sn);
+  const int half = a.inv_freq ? a.rot_dims / 2 : 0;
   int page = -1, slot = 0;
   if (a.store) {
     const int pos = a.row_pos[row], c = pos / SB_PAGE;
@@ -66,18 +95,21 @@ __global__ void __launch_bounds__(THREADS) headnorm_kv_store_kernel(Args a) {
       v[i] = 0.0f;
       if (d < a.dk) {
         v[i] = sum_slices(src + col + d, a.n_slices, a.slice_stride);
+        if (d < 2 * half)
+          v[i] = turned(v[i], sum_slices(src + col + (d < half ? d + half : d - half), a.n_slices, a.slice_stride), d, half, cs, sn);
         sq += double(v[i] * v[i]);
       }
     }
     const bool is_q = u < a.heads_q;
     const void *w = is_q ? a.q_w : a.k_w;
+    const bool norm = w || a.unit;
     float inv = 1.0f;
-    if (w) inv = 1.0f / sqrtf(float(wave_sum(sq) / double(a.dk)) + a.eps);
+    if (norm) inv = 1.0f / sqrtf(float(wave_sum(sq) / double(a.dk)) + a.eps);
 #pragma unroll
     for (int i = 0; i < kMaxHead / 64; ++i) {
       const int d = lane + 64 * i;
       if (d >= a.dk) continue;
-      const float o = w ? (v[i] * inv) * ld_dyn(w, a.w_dtype, d) : v[i];
+      const float o = w ? (v[i] * inv) * ld_dyn(w, a.w_dtype, d) : norm ? v[i] * inv : v[i];
       if (is_q) st_f((TQ *)a.q_out, size_t(row) * a.heads_q * a.dk + col + d, o);
       else if (page >= 0)
         st_f((TC *)a.k_cache, (size_t(page) * a.heads_kv + (u - a.heads_q)) * SB_PAGE * a.dk + sb_key_index(slot, d, a.dk), o);
@@ -104,6 +136,9 @@ __global__ void __launch_bounds__(256) headnorm_kv_store_wide_kernel(Args a) {
   constexpr int HEADS_PER_BLOCK = 256 / LANES;
   const int row = blockIdx.x, tid = threadIdx.x, sub = tid % LANES, slot_in_block = tid / LANES;
   const float *src = a.qkv + size_t(row) * a.row_stride;
+  __shared__ float cs[kMaxHead / 2], sn[kMaxHead / 2];
+  if (a.inv_freq) row_angles(a, row, cs, sn);
+  const int half = a.inv_freq ? a.rot_dims / 2 : 0;
   int page = -1, slot = 0;
   if (a.store) {
     const int pos = a.row_pos[row], c = pos / SB_PAGE;
@@ -119,6 +154,13 @@ __global__ void __launch_bounds__(256) headnorm_kv_store_wide_kernel(Args a) {
     if (live) {
       const float4 lo = *reinterpret_cast<const float4 *>(src + u * a.dk + d), hi = *reinterpret_cast<const float4 *>(src + u * a.dk + d + 4);
       v[0] = lo.x; v[1] = lo.y; v[2] = lo.z; v[3] = lo.w; v[4] = hi.x; v[5] = hi.y; v[6] = hi.z; v[7] = hi.w;
+      if (d < 2 * half) {       // (half is a multiple of 8: the other numbers of the eight pairs are neighbours too)
+        const float *op = src + u * a.dk + (d < half ? d + half : d - half);
+        const float4 ol = *reinterpret_cast<const float4 *>(op), oh = *reinterpret_cast<const float4 *>(op + 4);
+        const float o[8] = {ol.x, ol.y, ol.z, ol.w, oh.x, oh.y, oh.z, oh.w};
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[i] = turned(v[i], o[i], d + i, half, cs, sn);
+      }
     }
     double sq = 0.0;
 #pragma unroll
@@ -128,12 +170,12 @@ __global__ void __launch_bounds__(256) headnorm_kv_store_wide_kernel(Args a) {
     if (!live) continue;
     const bool is_q = u < a.heads_q;
     const void *w = is_q ? a.q_w : a.k_w;
-    const float inv = w ? 1.0f / sqrtf(float(sq / double(a.dk)) + a.eps) : 1.0f;
+    const float inv = (w || a.unit) ? 1.0f / sqrtf(float(sq / double(a.dk)) + a.eps) : 1.0f;
     uint32_t packed[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const float o0 = w ? (v[2 * i] * inv) * ld_dyn(w, a.w_dtype, d + 2 * i) : v[2 * i];
-      const float o1 = w ? (v[2 * i + 1] * inv) * ld_dyn(w, a.w_dtype, d + 2 * i + 1) : v[2 * i + 1];
+      const float o0 = w ? (v[2 * i] * inv) * ld_dyn(w, a.w_dtype, d + 2 * i) : v[2 * i] * inv;
+      const float o1 = w ? (v[2 * i + 1] * inv) * ld_dyn(w, a.w_dtype, d + 2 * i + 1) : v[2 * i + 1] * inv;
       packed[i] = uint32_t(f32_to_bf16(o0)) | uint32_t(f32_to_bf16(o1)) << 16;
     }
     const uint4 out = make_uint4(packed[0], packed[1], packed[2], packed[3]);
@@ -161,7 +203,10 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
                                     const void *lam, int lam_dtype, float *v_out, const int32_t *row_pos,
                                     const int32_t *row_seq, void *k_cache, void *v_cache, int cache_dtype,
                                     const int32_t *page_table, int max_pages, int n_pages, int n_rows, int heads_q,
-                                    int heads_kv, int dk, int dv, int store, void *stream) {
+                                    int heads_kv, int dk, int dv, int store, const float *inv_freq, int rot_dims, int unit,
+                                    void *stream) {
+  SB_REQUIRE(!inv_freq || (row_pos && rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= dk),
+             "sb_headnorm_kv_store: rotary width %d must be even and at most the head's %d", rot_dims, dk);
   SB_REQUIRE(q_out && qkv, "sb_headnorm_kv_store: null pointer");
   SB_REQUIRE(n_rows >= 0 && heads_q > 0 && heads_kv >= 0 && dk > 0 && dv > 0 && n_slices > 0,
              "sb_headnorm_kv_store: bad sizes rows=%d heads=%d/%d dk=%d dv=%d", n_rows, heads_q, heads_kv, dk, dv);
@@ -174,7 +219,8 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
   SB_SUPPORT(dk <= kMaxHead, "sb_headnorm_kv_store: head size %d is above the limit of %d", dk, kMaxHead);
   if (n_rows == 0) return SB_OK;
   const Args a{q_out, qkv, row_stride, n_slices, size_t(n_rows) * row_stride, q_w, k_w, w_dtype, eps, v_first, lam, lam_dtype, v_out,
-               row_pos, row_seq, page_table, max_pages, n_pages, k_cache, v_cache, heads_q, heads_kv, dk, dv, store ? 1 : 0};
+               row_pos, row_seq, page_table, max_pages, n_pages, k_cache, v_cache, heads_q, heads_kv, dk, dv, store ? 1 : 0,
+               inv_freq, inv_freq ? rot_dims : 0, unit};
   hipStream_t s = (hipStream_t)stream;
   const bool qf = q_dtype == SB_F32, cf = !store || cache_dtype == SB_F32;
   // (a wave a head: the sums do not depend on the block's size, so few rows may take more waves a row)
@@ -182,7 +228,7 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
   else if (qf) headnorm_kv_store_kernel<float, bf16_t, 256><<<n_rows, 256, 0, s>>>(a);
   else if (cf && store) headnorm_kv_store_kernel<bf16_t, float, 256><<<n_rows, 256, 0, s>>>(a);
   else if (n_rows <= 64) headnorm_kv_store_kernel<bf16_t, bf16_t, 1024><<<n_rows, 1024, 0, s>>>(a);
-  else if (n_rows >= 512 && n_slices == 1 && dk % 8 == 0 && row_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(qkv) & 15) == 0 &&
+  else if (n_rows >= 512 && n_slices == 1 && dk % 8 == 0 && (!inv_freq || rot_dims % 16 == 0) && row_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(qkv) & 15) == 0 &&
            (reinterpret_cast<uintptr_t>(q_out) & 15) == 0 && (!store || (reinterpret_cast<uintptr_t>(k_cache) & 15) == 0)) {
     if (dk <= 64) headnorm_kv_store_wide_kernel<8><<<n_rows, 256, 0, s>>>(a);
     else if (dk <= 128) headnorm_kv_store_wide_kernel<16><<<n_rows, 256, 0, s>>>(a);

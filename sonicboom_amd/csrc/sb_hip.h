@@ -254,15 +254,16 @@ int sb_scale(float *x, float scale, size_t n, void *stream);
 
 /* ---- head norms, value mixing and store (csrc/headnorm_kv.hip) ---------------------------------
  * qkv f32 [n_slices][n_rows][row_stride] = [q: heads_q x dk | k: heads_kv x dk | v: heads_kv x dv], slices
- * added in ascending order; every head of q and k divided by its root mean square (eps inside the root)
- * times q_w / k_w [dk] (NULL: as it is); v <- (1 - lam) v + lam v_first when v_first is given; the v of
+ * added in ascending order; with inv_freq the pairs (i, i + rot_dims / 2) of every head of q and k turn by
+ * position * inv_freq[i]; every head of q and k is then divided by its root mean square (eps inside the root)
+ * times q_w / k_w [dk] (NULL: as it is, or with `unit` divided without a weight); v <- (1 - lam) v + lam v_first when v_first is given; the v of
  * before the mixing to v_out when that is given; q out in q_dtype, k and v (store != 0) into the pages. */
 int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, int row_stride, int n_slices,
                          const void *q_w, const void *k_w, int w_dtype, float eps, const float *v_first,
                          const void *lam, int lam_dtype, float *v_out, const int32_t *row_pos,
                          const int32_t *row_seq, void *k_cache, void *v_cache, int cache_dtype,
                          const int32_t *page_table, int max_pages, int n_pages, int n_rows, int heads_q,
-                         int heads_kv, int dk, int dv, int store, void *stream);
+                         int heads_kv, int dk, int dv, int store, const float *inv_freq, int rot_dims, int unit, void *stream);
 
 /* sb_attention with values of v_dim numbers a head (cache values [page][kv head][v_dim][position], out
  * [rows, heads_q * v_dim]), scores capped as softcap * tanh(s / softcap) when softcap > 0, and with `sink`
@@ -487,7 +488,8 @@ int sb_random_normal(void *out, int out_kind, uint64_t n, uint64_t first, uint64
  * sb_sigmoid_mul: x[t, i] *= sigmoid(gate[t * gate_stride + i]).  sb_softcap: x <- cap tanh(x / cap).
  * sb_rope_kv_store_sized: value heads of v_dim numbers; every cosine and sine times `magnitude`.
  * sb_attention_sink: the sink's score a number of the query head's own (sink_scores f32 [heads_q]); an output
- *   gate, the result times sigmoid(gate[row * gate_stride + i]).
+ *   gate, the result times sigmoid(gate[row * gate_stride + i]), or with gate_per_head all of head h times
+ *   sigmoid(gate[row * gate_stride + h]).
  * sb_latent_prepare_split: the latent's part read from rows of its own; `magnitude` as above.
  * sb_head_product_gated(_bf16): gate_per_head, one gate number a head.
  * sb_moe_route_grouped / sb_moe_router_grouped: score_kind 0 softmax over the chosen, 1 sigmoid, 2 softmax
@@ -507,7 +509,7 @@ int sb_attention_sink(void *out, const void *q, int act_dtype, int q_stride, con
                       int cache_dtype, const int32_t *page_table, int max_pages, int n_pages_total,
                       const int32_t *row_pos, const int32_t *row_seq, int n_rows, int heads_q, int heads_kv, int head_dim,
                       int v_dim, float scale, int window, float softcap, int sink, const float *sink_scores,
-                      const float *gate, int gate_stride, void *stream);
+                      const float *gate, int gate_stride, int gate_per_head, void *stream);
 int sb_latent_prepare_split(void *q_plain, void *q_latent, int act_dtype, const float *p, int row_stride, int q_off,
                             const float *kv_rows, int kv_stride, int kv_off, const void *c_weight, int c_w_dtype, float eps,
                             const float *inv_freq, int rot_dims, int interleaved, float magnitude, const int32_t *row_pos,
@@ -524,6 +526,34 @@ int sb_moe_route_grouped(int32_t *ids, float *weights, const float *z, int n_row
 int sb_moe_router_grouped(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows, int n_in,
                           int n_experts, int top, int has_gate, int score_kind, float score_scale, int n_groups,
                           int keep_groups, void *stream);
+
+/* ---- the pass that ends a block of branches, and the layer norm (csrc/join.hip) -------------------
+ * sb_join: out[r,:] = base[r,:] + sum_b scale_b N_b(sum of branch b's slices) + vec, for up to three branches
+ *   (term_ptrs: {part f32, norm weight or NULL} each; term_ints: {slices, weight dtype, 1: divided by its root mean
+ *   square, term_eps inside the root} each; slice_strides in numbers); then h = what the next block reads:
+ *   0 nothing, 1 RMS norm, 2 layer norm, 3 out itself in h_dtype.  base may be out.
+ * sb_layernorm: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w of the rows named by `rows` (NULL: all).
+ * few != 0: up to 64 rows take blocks of 1024 threads (a row's sums are then ordered otherwise). */
+int sb_join(float *out, const float *base, const void *const *term_ptrs, const int *term_ints, const float *term_scales,
+            const size_t *slice_strides, int n_terms, float term_eps, const void *vec, int vec_dtype, void *h, int h_dtype,
+            int then, const void *h_weight, int h_w_dtype, float h_eps, int n_rows, int width, int few, void *stream);
+int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dtype, const int32_t *rows, int n_rows,
+                 int width, float eps, int few, void *stream);
+
+/* ---- linear attention with decays (csrc/decay_scan.hip) ------------------------------------------
+ * sb_decay_scan: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t per head (S f32 D x E in
+ *   state[slots[s]]), out_t = o_t / rms(o_t) (* w) * silu(g_t); alpha from log_decay f32 [rows, heads * D], or one
+ *   number a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
+ *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart.
+ * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width]. */
+int sb_decay_scan_max_side(void);
+int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
+                  int row_stride, const float *log_decay, int ld_stride, const float *decay, const float *inv_freq,
+                  int rot_dims, const int32_t *row_pos, float q_scale, float k_scale, const void *w, int w_dtype, float eps,
+                  float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E,
+                  void *stream);
+int sb_log_decay(float *out, int out_stride, const float *a, int a_stride, const float *w, const float *bias, int n_rows,
+                 int rank, int width, float rate, void *stream);
 
 #ifdef __cplusplus
 }

@@ -122,6 +122,7 @@ class DecodeLoop:
         # a part that steers its work from the host (Python control flow over the step's
         # sequences) cannot be replayed from a recording; parts say so with graph_safe
         parts = [p for b in engine.model.blocks for p in (getattr(b, "mixer", None), getattr(b, "ffn", None))]
+        parts += engine.model.junctions
         self.use_graph = use_graph and all(getattr(p, "graph_safe", False) for p in parts if p is not None)
         # added rows would run a mixer's per-sequence state of some live slot: no padding then
         self.pad_batches = not engine.cache.state

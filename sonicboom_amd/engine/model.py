@@ -45,6 +45,11 @@ class DecoderModel:
         self.final_norm = build_part(spec.final_norm, tensors, rt)
         shared = {t.name for t in spec.embedding.all_tensors() + spec.head.all_tensors()
                   + spec.final_norm.all_tensors()}
+        self.junctions = [build_part(j, tensors, rt) for j in spec.junctions]
+        for j in spec.junctions:
+            for t in j.all_tensors():
+                if t.name not in shared:
+                    tensors.pop(t.name, None)
         self.blocks = []
         for b in spec.blocks:
             self.blocks.append(build_part(b, tensors, rt))

@@ -315,9 +315,17 @@ class Engine:
         if tracer is not None:
             tracer("embedding", x)
         h = None
+        for junction in model.junctions:
+            h = junction.begin(x, ctx)
+        if not model.order or model.order[0].junction is None:
+            h = None                           # (a block reads its own norm of x)
         for i, e in enumerate(model.order):
-            nxt = model.order[i + 1].block if i + 1 < len(model.order) else None
-            next_norm = getattr(model.blocks[nxt], "first_norm", None) if nxt is not None else None
+            if e.junction is not None:
+                h = model.junctions[e.junction].forward(x, ctx, e.turn, h=h,
+                                                        next_norm=getattr(model.blocks[e.block], "first_norm", None))
+            nxt = model.order[i + 1] if i + 1 < len(model.order) else None
+            then = None if nxt is None else model.blocks[nxt.block] if nxt.junction is None else model.junctions[nxt.junction]
+            next_norm = getattr(then, "first_norm", None)
             # a block reports what it has computed through ctx.trace, if it cares to
             ctx.trace = (lambda what, t, _i=i: tracer(f"entry{_i}.{what}", t)) if tracer is not None else None
             h = model.blocks[e.block].forward(x, ctx, self.bindings[i], h=h, next_norm=next_norm)

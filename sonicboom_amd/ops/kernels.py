@@ -10,6 +10,7 @@ a missing library or a refused size raises
 from __future__ import annotations
 
 import contextlib
+import ctypes
 import math
 import threading
 
@@ -1231,20 +1232,28 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
                       k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], page_table: Optional[torch.Tensor],
                       heads_q: int, heads_kv: int, head_dim: int, v_dim: int, store: bool = True,
                       v_first: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None,
-                      v_out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      v_out: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
+                      unit: bool = False) -> torch.Tensor:
     """From float32 rows [n, heads_q*head_dim + heads_kv*(head_dim + v_dim)] of a stacked product (or
-    [slices, n, ...], added here): every head of q and k divided by its root mean square and
-    multiplied by a weight [head_dim] that the heads share (None: as it is), the values mixed as
+    [slices, n, ...], added here): with ``inv_freq`` the pairs (i, i + rot_dims/2) of every head of q and k
+    turned by position * inv_freq[i]; then every head of q and k divided by its root mean square and
+    multiplied by a weight [head_dim] that the heads share (None: as it is, or with ``unit`` divided without a
+    weight), the values mixed as
     (1 - lam) v + lam v_first when ``v_first`` (float32 [n, heads_kv*v_dim]) is given, the values of
     before the mixing written to ``v_out``; returns q [n, heads_q*head_dim] in ``q_dtype`` and, with
     ``store``, puts keys and values into the pages of the rows' positions."""
-    _dev(qkv, q_weight, k_weight, row_pos, row_seq, k_cache, v_cache, page_table, v_first, lam, v_out)
+    _dev(q_weight, k_weight, row_pos, row_seq, k_cache, v_cache, page_table, v_first, lam, v_out)
     if qkv.dtype != torch.float32:
         raise KernelLibraryError("the stacked product must be float32")
     n_slices = 1
     if qkv.dim() == 3:
+        _dev(qkv)
         n_slices = qkv.shape[0]
         qkv = qkv.view(-1, qkv.shape[2])
+    _on_gpu(qkv)
+    if qkv.dim() != 2 or qkv.stride(1) != 1:            # (a column range of wider rows is fine)
+        raise KernelLibraryError("rows of the stacked product must be contiguous")
+    row_stride = qkv.stride(0) if qkv.shape[0] > 1 else qkv.shape[1]
     n = qkv.shape[0] // n_slices
     need = heads_q * head_dim + (heads_kv * (head_dim + v_dim) if store else 0)
     if qkv.dim() != 2 or qkv.shape[1] < need:
@@ -1266,12 +1275,19 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
             raise KernelLibraryError(f"the {what} must be float32 [rows, {nv}]")
     if v_first is not None and (lam is None or lam.numel() != 1):
         raise KernelLibraryError("mixing values takes one number")
+    if inv_freq is not None:
+        _dev(inv_freq)
+        if inv_freq.dtype != torch.float32 or inv_freq.numel() != rot_dims // 2:
+            raise KernelLibraryError(f"a rotation of {rot_dims} numbers takes {rot_dims // 2} float32 frequencies")
+        if not store:
+            _i32(row_pos, n, "row positions")
     q = torch.empty((n, heads_q * head_dim), dtype=q_dtype, device=qkv.device)
     check(library.core().sb_headnorm_kv_store(
-        _p(q), _dt(q), _p(qkv), qkv.shape[1], n_slices, _p(q_weight), _p(k_weight), _dt(wt) if wt is not None else 0,
+        _p(q), _dt(q), _p(qkv), row_stride, n_slices, _p(q_weight), _p(k_weight), _dt(wt) if wt is not None else 0,
         float(eps), _p(v_first), _p(lam) if v_first is not None else None, _dt(lam) if lam is not None else 0, _p(v_out),
         _p(row_pos), _p(row_seq), _p(k_cache), _p(v_cache), _dt(k_cache) if store else 0, _p(page_table), max_pages,
-        n_pages, n, heads_q, heads_kv, head_dim, v_dim, 1 if store else 0, _stream()))
+        n_pages, n, heads_q, heads_kv, head_dim, v_dim, 1 if store else 0, _p(inv_freq), int(rot_dims), 1 if unit else 0,
+        _stream()))
     return q
 
 
@@ -1282,10 +1298,11 @@ def attention_capped_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
     """Attention of rows ``q`` [n, hq*hd] over the cache by the plain kernel, values of ``v_dim``,
     scores capped as softcap tanh(s / softcap) (0: not), with ``sink`` one more key of score 0
     without a value in every softmax (``sink_scores`` float32 [hq]: of the head's own score instead); [n, hq*v_dim].
-    ``gate`` float32 [n, hq*v_dim] (a view of wider rows is fine): the result times sigmoid(gate)."""
+    ``gate`` float32 [n, hq*v_dim] (a view of wider rows is fine): the result times sigmoid(gate); [n, hq]: every
+    number of a head times the head's one."""
     _dev(q, k_cache, v_cache, page_table, row_pos, row_seq, sink_scores)
     _check_sink(sink, sink_scores, heads_q)
-    g_stride = _check_gate(gate, q.shape[0], heads_q * v_dim)
+    g_stride, per_head = _check_gate(gate, q.shape[0], heads_q, v_dim)
     n = q.shape[0]
     if q.dim() != 2 or q.shape[1] != heads_q * head_dim:
         raise KernelLibraryError(f"queries must be [rows, {heads_q * head_dim}]")
@@ -1295,18 +1312,22 @@ def attention_capped_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
     check(library.core().sb_attention_sink(
         _p(out), _p(q), _dt(q), q.shape[1], _p(k_cache), _p(v_cache), _dt(k_cache), _p(page_table),
         page_table.shape[1], k_cache.shape[0], _p(row_pos), _p(row_seq), n, heads_q, heads_kv, head_dim, v_dim,
-        float(scale), int(window), float(softcap), 1 if sink else 0, _p(sink_scores), _p(gate), g_stride, _stream()))
+        float(scale), int(window), float(softcap), 1 if sink else 0, _p(sink_scores), _p(gate), g_stride, per_head,
+        _stream()))
     return out
 
 
-def _check_gate(gate, rows, width) -> int:
-    """The distance between the rows of an output gate (0 without one)."""
+def _check_gate(gate, rows, heads, v_dim):
+    """(distance between the rows of an output gate, 1 when it holds a number a head): (0, 0) without one."""
     if gate is None:
-        return 0
+        return 0, 0
     _on_gpu(gate)
-    if gate.dtype != torch.float32 or gate.dim() != 2 or tuple(gate.shape) != (rows, width) or gate.stride(1) != 1:
-        raise KernelLibraryError(f"an output gate must be float32 [{rows}, {width}], dense along a row")
-    return gate.stride(0) if rows > 1 else width
+    width = heads * v_dim
+    if gate.dtype != torch.float32 or gate.dim() != 2 or gate.shape[0] != rows or gate.shape[1] not in (width, heads) \
+            or gate.stride(1) != 1:
+        raise KernelLibraryError(f"an output gate must be float32 [{rows}, {width}] or [{rows}, {heads}], dense along a row")
+    per_head = 1 if gate.shape[1] == heads else 0       # (values of one number: the two forms are the same)
+    return (gate.stride(0) if rows > 1 else gate.shape[1]), per_head
 
 
 def _check_sink(sink, sink_scores, heads_q):
@@ -1440,7 +1461,7 @@ def attention_capped_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch
     _dev(q, k_cache, v_cache, page_table, row_pos, tiles, sink_scores)
     _check_sink(sink, sink_scores, heads_q)
     n = q.shape[0]
-    g_stride = _check_gate(gate, n, heads_q * v_dim)
+    g_stride, per_head = _check_gate(gate, n, heads_q, v_dim)
     if q.dim() != 2 or q.shape[1] != heads_q * head_dim or q.dtype != torch.bfloat16:
         raise KernelLibraryError(f"queries must be bfloat16 [rows, {heads_q * head_dim}]")
     _check_cache_kv(k_cache, v_cache, heads_kv, head_dim, v_dim)
@@ -1467,7 +1488,7 @@ def attention_capped_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch
     check(lib.sb_cattn_sink_bf16(_p(out), _p(q), _p(k_cache), _p(v_cache), _p(page_table), max_pages, k_cache.shape[0],
                                  _p(row_pos), _p(tiles), n_tiles, n, heads_q, heads_kv, float(scale), int(window),
                                  float(softcap), 1 if sink else 0, chunks, chunk_pages, _p(part_o), _p(part_ml), None, None, 0,
-                                 _p(sink_scores), _p(gate), g_stride, _stream()),
+                                 _p(sink_scores), _p(gate), g_stride, per_head, _stream()),
           lib, "sb_cattn_last_error")
     return out
 
@@ -1827,3 +1848,136 @@ def attention_shared(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         o = attention_shared_plain(q, k_cache, v_cache, page_table, ctx.row_pos, ctx.row_seq, heads_q, heads_kv, head_dim,
                                    v_dim, scale, r1, r2)
     return head_mix(o, mix, out_dtype)
+
+
+# --------------------------------------------------------------------------
+# Branches of one block joining the stream; layer norm; linear attention with decays.
+
+JOIN_THEN = {None: 0, "rms": 1, "layer": 2, "copy": 3}
+JOIN_MAX_TERMS = 3
+
+
+def layernorm(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, out_dtype: torch.dtype,
+              rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * weight of float32 rows ``x`` [n, width]; ``rows`` (int32)
+    picks and orders source rows."""
+    _dev(x, weight, rows)
+    if x.dtype != torch.float32 or x.dim() != 2:
+        raise KernelLibraryError("layernorm input must be float32 [rows, width]")
+    width = x.shape[1]
+    if weight is not None and weight.numel() != width:
+        raise KernelLibraryError(f"layernorm weight has {weight.numel()} elements, the rows have {width}")
+    n = x.shape[0] if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows, n, "row index")
+    y = torch.empty((n, width), dtype=out_dtype, device=x.device)
+    check(library.core().sb_layernorm(_p(y), _dt(y), _p(x), _p(weight), _dt(weight) if weight is not None else 0, _p(rows), n,
+                                      width, float(eps), 1 if out_dtype == torch.bfloat16 else 0, _stream()))
+    return y
+
+
+def join(out: torch.Tensor, base: torch.Tensor, terms, act_dtype: torch.dtype, term_eps: float = 0.0,
+         vec: Optional[torch.Tensor] = None, then: Optional[str] = None, then_weight: Optional[torch.Tensor] = None,
+         then_eps: float = 0.0, out_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
+    """out = base + the sum of ``terms`` + ``vec`` [width] in float32, in one pass over the row; ``base`` may be ``out``.
+
+    A term is (part, scale, normed, weight): ``part`` float32 [rows, width] or slices of it [slices, rows, width]
+    that are added first; ``normed``: the sum is divided by its root mean square (``term_eps`` inside the root) and
+    multiplied by ``weight`` [width] (None: not).  ``then`` is what is returned, in ``out_dtype``: "rms" or "layer",
+    that norm of ``out`` with ``then_weight`` and ``then_eps``; "copy", ``out`` itself; None: nothing.
+    ``act_dtype`` bfloat16: few rows may take another block shape than many."""
+    _dev(out, base, vec, then_weight)
+    if out.dtype != torch.float32 or base.dtype != torch.float32 or out.dim() != 2 or out.shape != base.shape:
+        raise KernelLibraryError("the stream must be float32 [rows, width]")
+    n, width = out.shape
+    if len(terms) > JOIN_MAX_TERMS:
+        raise KernelLibraryError(f"{len(terms)} branches, at most {JOIN_MAX_TERMS} join in one pass")
+    ptrs, ints, scales, strides = [], [], [], []
+    for part, scale, normed, weight in terms:
+        _dev(part, weight)
+        if part.dtype != torch.float32 or part.dim() not in (2, 3) or tuple(part.shape[-2:]) != (n, width):
+            raise KernelLibraryError(f"a branch's result {tuple(part.shape)} does not fit the stream {tuple(out.shape)}")
+        if weight is not None and weight.numel() != width:
+            raise KernelLibraryError(f"a branch's norm has {weight.numel()} weights, the rows have {width}")
+        slices = part.shape[0] if part.dim() == 3 else 1
+        ptrs += [_p(part), _p(weight)]
+        ints += [slices, _dt(weight) if weight is not None else 0, 1 if normed else 0]
+        scales.append(float(scale))
+        strides.append(n * width)
+    for t, what in ((vec, "vector"), (then_weight, "norm's weight")):
+        if t is not None and t.numel() != width:
+            raise KernelLibraryError(f"the {what} has {t.numel()} elements, the rows have {width}")
+    h = None
+    code = JOIN_THEN[then]
+    if code:
+        h = torch.empty((n, width), dtype=out_dtype, device=out.device)
+    nt = len(terms)
+    check(library.core().sb_join(
+        _p(out), _p(base), (ctypes.c_void_p * max(1, 2 * nt))(*ptrs), (ctypes.c_int * max(1, 3 * nt))(*ints),
+        (ctypes.c_float * max(1, nt))(*scales), (ctypes.c_size_t * max(1, nt))(*strides), nt, float(term_eps), _p(vec),
+        _dt(vec) if vec is not None else 0, _p(h), _dt(h) if h is not None else 0, code, _p(then_weight),
+        _dt(then_weight) if then_weight is not None else 0, float(then_eps), n, width,
+        1 if act_dtype == torch.bfloat16 else 0, _stream()))
+    return h
+
+
+def decay_scan_max_side() -> int:
+    """Rows and columns of a head's matrix that the decaying scans take at most (256 each)."""
+    return int(library.core().sb_decay_scan_max_side())
+
+
+def log_decay(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], rate: float) -> torch.Tensor:
+    """rate * log(sigmoid(a w + bias)) in float32: ``a`` float32 [n, rank] (a view of wider rows is fine), ``w`` float32
+    [rank, width], ``bias`` float32 [width]; [n, width]."""
+    _dev(w, bias)
+    rank, width = w.shape
+    _f32_rows(a, a.shape[0], rank, "a decay's inner numbers")
+    if w.dtype != torch.float32 or (bias is not None and (bias.dtype != torch.float32 or bias.numel() != width)):
+        raise KernelLibraryError("a decay's matrix and bias must be float32 [rank, width] and [width]")
+    out = torch.empty((a.shape[0], width), dtype=torch.float32, device=a.device)
+    check(library.core().sb_log_decay(_p(out), width, _p(a), a.stride(0), _p(w), _p(bias), a.shape[0], rank, width, float(rate),
+                                      _stream()))
+    return out
+
+
+def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, state: torch.Tensor, ctx, heads: int,
+               dim: int, v_dim: int, eps: float, out_dtype: torch.dtype, log_decay: Optional[torch.Tensor] = None,
+               decay: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, q_scale: float = 1.0,
+               k_scale: float = 1.0, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0) -> torch.Tensor:
+    """S = alpha S + k v^T, o = S^T q per head over every sequence's rows of the step, from ``state`` float32
+    [slots, heads, dim, v_dim], which moves on; returns o / rms(o) (* weight) * silu(g) [n, heads*v_dim] in ``out_dtype``.
+
+    ``q``, ``k`` [n, heads*dim], ``v``, ``g`` [n, heads*v_dim]: float32 parts of the same wider rows.  alpha: the
+    exponential of ``log_decay`` float32 [n, heads*dim], or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
+    pairs (i, i + rot_dims/2) of every head of q and k turn by position * inv_freq[i]; then q and k are multiplied by
+    their scales."""
+    n = q.shape[0]
+    _on_gpu(q, k, v, g)
+    for t, width, what in ((q, heads * dim, "queries"), (k, heads * dim, "keys"), (v, heads * v_dim, "values"),
+                           (g, heads * v_dim, "gates")):
+        _f32_rows(t, n, width, what)
+        if n > 1 and t.stride(0) != q.stride(0):
+            raise KernelLibraryError("queries, keys, values and gates must be parts of the same rows")
+    _dev(state, log_decay, decay, weight, inv_freq, ctx.cu_rows, ctx.slots, ctx.row_pos)
+    if state.dtype != torch.float32 or tuple(state.shape[1:]) != (heads, dim, v_dim):
+        raise KernelLibraryError(f"the state must be float32 [slots, {heads}, {dim}, {v_dim}]")
+    if (log_decay is None) == (decay is None):
+        raise KernelLibraryError("a decaying scan takes the logarithms of its decays, or one decay a head")
+    if log_decay is not None:
+        _f32_rows(log_decay, n, heads * dim, "logarithms of decays")
+    else:
+        _f32_vec(decay, heads, "decays")
+    if weight is not None and weight.numel() != v_dim:
+        raise KernelLibraryError(f"the heads' norm has {weight.numel()} weights, a head has {v_dim}")
+    if inv_freq is not None:
+        _f32_vec(inv_freq, rot_dims // 2, "frequencies")
+        _i32(ctx.row_pos, n, "row positions")
+    _i32(ctx.cu_rows, ctx.n_seqs + 1, "first rows")
+    _i32(ctx.slots, ctx.n_seqs, "slots")
+    out = torch.empty((n, heads * v_dim), dtype=out_dtype, device=q.device)
+    check(library.core().sb_decay_scan(
+        _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
+        log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
+        float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
+        _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _stream()))
+    return out

@@ -57,7 +57,7 @@ _CORE_SIGNATURES = {
     "sb_scale": [_P, _F, _Z, _P],
     "sb_embed_pos_norm": [_P, _P, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P, _I, _I, _F, _F, _I, _P],
     "sb_headnorm_kv_store": [_P, _I, _P, _I, _I, _P, _P, _I, _F, _P, _P, _I, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I,
-                             _I, _I, _I, _I, _I, _P],
+                             _I, _I, _I, _I, _I, _P, _I, _I, _P],
     "sb_attention_capped": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P],
     "sb_moe_max_top": [],
     "sb_moe_route": [_P, _P, _P, _I, _I, _I, _I, _I, _P],
@@ -89,13 +89,19 @@ _CORE_SIGNATURES = {
     "sb_softcap": [_P, _F, _Z, _P],
     "sb_rope_kv_store_sized": [_P, _I, _P, _I, _I, _I, _P, _P, _P, _I, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F,
                                _P],
-    "sb_attention_sink": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _P, _I, _P],
+    "sb_attention_sink": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _P, _I, _I, _P],
     "sb_latent_prepare_split": [_P, _P, _I, _P, _I, _I, _P, _I, _I, _P, _I, _F, _P, _I, _I, _F, _P, _P, _P, _I, _P, _I, _I,
                                 _I, _I, _I, _I, _I, _P],
     "sb_head_product_gated": [_P, _I, _I, _I, _P, _I, _I, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "sb_head_product_gated_bf16": [_P, _I, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "sb_moe_route_grouped": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
     "sb_moe_router_grouped": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],
+    "sb_join": [_P, _P, _P, _P, _P, _P, _I, _F, _P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P],
+    "sb_layernorm": [_P, _I, _P, _P, _I, _P, _I, _I, _F, _I, _P],
+    "sb_decay_scan_max_side": [],
+    "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
+                      _P],
+    "sb_log_decay": [_P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P],
 }
 # Entry points of later kernels; declared when the library has them.
 _OPTIONAL_SIGNATURES = {
@@ -135,9 +141,9 @@ _CAPPED_ATTN_SIGNATURES = {
     "sb_cattn_bf16": [_P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _I, _I, _I, _P, _P, _P],
     # the same, then dist_r1, dist_r2, all_values, stream
     "sb_cattn_shared_bf16": [_P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P],
-    # the same, then sink_scores, gate, gate_stride, stream
+    # the same, then sink_scores, gate, gate_stride, gate_per_head, stream
     "sb_cattn_sink_bf16": [_P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
-                           _P, _I, _P],
+                           _P, _I, _I, _P],
     "sb_cattn_tile_rows": [],
     "sb_cattn_key_dim": [],
     "sb_cattn_value_dim": [],

@@ -17,8 +17,10 @@ Every size and switch is a parameter of the spec:
     for later layers under ``value_mix_key``; "mix": v <- (1 - lam) v + lam v_first with the layer's
     own number lam; what is mixed is what the cache keeps), sink_scores (the sink's score is a number of
     the query head's own, a tensor of heads_q numbers, as it is: weights exp(s_j) / (exp(sink_a) + sum
-    exp(s_j))), out_gate (the heads' results side by side times sigmoid(W_g h), number by number, before
-    the output product; W_g is stacked under q, k and v)
+    exp(s_j))), out_gate (True: the heads' results side by side times sigmoid(W_g h), number by number, before
+    the output product; "head": head a's result times sigmoid((W_g h)_a), one number a head; W_g is
+    stacked under q, k and v), qk_norm_weight (False: the head norms have no weight), given_input (the
+    mixer's stacked input matrix is part of a larger one: see ``input_weight`` below)
 
 and the position encoding is a nested part.  The three input projections are
 packed into one matrix when the mixer is built, so a step runs one product
@@ -43,6 +45,8 @@ NAMES = {"q_weight": "q_proj.weight", "k_weight": "k_proj.weight", "v_weight": "
          "o_bias": "o_proj.bias", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "value_mix": "value_mix",
          "sink": "sink", "g_weight": "g"}
 
+HEAD_GATE = "head"           # an output gate of one number a head
+
 
 def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_dim: int,
                    position: PartSpec, window: int = 0, scale: Optional[float] = None,
@@ -50,7 +54,7 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
                    v_dim: Optional[int] = None, qk_norm: bool = False, qk_norm_eps: float = 0.0,
                    softcap: float = 0.0, sink: bool = False, value_mix: Optional[str] = None,
                    value_mix_key: str = "values", names: Optional[dict] = None, sink_scores: bool = False,
-                   out_gate: bool = False) -> PartSpec:
+                   out_gate=False, qk_norm_weight: bool = True, given_input: bool = False) -> PartSpec:
     """``names``: what the file calls a role's tensor after ``prefix``, where that is not what
     ``NAMES`` says."""
     nm = dict(NAMES, **(names or {}))
@@ -68,7 +72,7 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
         tensors["v_bias"] = TensorSpec(prefix + nm["v_bias"], (vw,))
     if out_bias:
         tensors["o_bias"] = TensorSpec(prefix + nm["o_bias"], (width,))
-    if qk_norm:
+    if qk_norm and qk_norm_weight:
         tensors["q_norm"] = TensorSpec(prefix + nm["q_norm"], (head_dim,), init=(1.0, 0.02))
         tensors["k_norm"] = TensorSpec(prefix + nm["k_norm"], (head_dim,), init=(1.0, 0.02))
     if sink_scores:
@@ -76,7 +80,7 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
             raise ValueError("scores of a sink belong to a mixer that has one")
         tensors["sink"] = TensorSpec(prefix + nm["sink"], (heads_q,), init=(0.0, 0.5))
     if out_gate:
-        tensors["g_weight"] = TensorSpec(prefix + nm["g_weight"], (heads_q * v_dim, width))
+        tensors["g_weight"] = TensorSpec(prefix + nm["g_weight"], (heads_q * (1 if out_gate == HEAD_GATE else v_dim), width))
     if value_mix not in (None, "first", "mix"):
         raise ValueError(f"value_mix is None, 'first' or 'mix', not {value_mix!r}")
     if value_mix is not None:
@@ -87,7 +91,8 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
         "window": int(window), "scale": scale, "qkv_bias": qkv_bias, "out_bias": out_bias,
         "out_scale": float(out_scale), "v_dim": v_dim, "qk_norm": bool(qk_norm), "qk_norm_eps": float(qk_norm_eps),
         "softcap": float(softcap), "sink": bool(sink), "value_mix": value_mix, "value_mix_key": value_mix_key,
-        "sink_scores": bool(sink_scores), "out_gate": bool(out_gate),
+        "sink_scores": bool(sink_scores), "out_gate": HEAD_GATE if out_gate == HEAD_GATE else bool(out_gate),
+        "given_input": bool(given_input),
     }, tensors, {"position": position})
 
 
@@ -122,15 +127,18 @@ class Attention(Mixer):
         self.lam = tensors.get("value_mix") if self.value_mix == "mix" else None
         self.sink_scores = tensors["sink"].float().contiguous() if p.get("sink_scores") else None
         self.out_gate = bool(p.get("out_gate", False))
+        self.gate_width = self.heads_q * (1 if p.get("out_gate") == HEAD_GATE else self.v_dim)
         # head norms, capped scores, a sink, values of their own size or mixed values, an output gate: the path
-        # whose kernels take them.  Head norms and mixed values go with mixers that do not rotate (one kernel
-        # norms, mixes and stores); the others rotate and store with the kernel of the plain path.
+        # whose kernels take them.  With head norms or mixed values one kernel rotates, then norms, mixes and
+        # stores; the others rotate and store with the kernel of the plain path.
         self.extended = bool(self.qk_norm or self.softcap or self.sink or self.value_mix or self.v_dim != self.head_dim
-                             or self.out_gate)
+                             or self.out_gate or p.get("given_input"))
         self.head_norm_path = bool(self.qk_norm or self.value_mix)
         if self.extended:
-            if self.head_norm_path and self.position.rotary_tables() != (None, None, 0):
-                raise ValueError("head norms and mixed values are built for mixers without a rotation")
+            tables = self.position.rotary_tables()
+            if self.head_norm_path and (tables is None or tables[1] is not None or self.position.interleaved
+                                        or getattr(self.position, "magnitude", 1.0) != 1.0):
+                raise ValueError("head norms and mixed values take no rotation, or the rotate-half one by plain frequencies")
             if self.position.rotary_tables() is None:
                 raise ValueError("capped scores, sinks, gates and values of their own size take a rotary position "
                                  "encoding, or none")
@@ -152,7 +160,14 @@ class Attention(Mixer):
             b_qkv = torch.cat([b.float() for b in bs], dim=0)
             if self.out_gate:
                 b_qkv = torch.cat([b_qkv, torch.zeros(tensors["g_weight"].shape[0], dtype=torch.float32, device=b_qkv.device)])
-        self.qkv = Linear(w_qkv, b_qkv, rt.fast_kernels)
+        self.input_weight = None
+        if p.get("given_input"):
+            # the part around the mixer makes one product for several mixers: it takes the stacked matrix from
+            # here while the model is built, and hands the product's rows to from_rows()
+            if b_qkv is not None:
+                raise ValueError("a mixer whose input product is given has no biases on q, k and v")
+            self.input_weight = w_qkv
+        self.qkv = None if p.get("given_input") else Linear(w_qkv, b_qkv, rt.fast_kernels)
         # an order entry that reads another entry's cache projects queries only: the model asks for
         # that projection (query_only) before finish_build() drops the separate query weight
         self._q_parts = (tensors["q_weight"], None if b_qkv is None else b_qkv[: self.q_width])
@@ -169,6 +184,7 @@ class Attention(Mixer):
 
     def finish_build(self) -> None:
         self._q_parts = None
+        self.input_weight = None
 
     def cache_spec(self) -> KVSpec:
         return KVSpec(self.heads_kv, self.head_dim, self.window, self.v_dim)
@@ -183,6 +199,13 @@ class Attention(Mixer):
         a = self._attend(h, ctx, binding)
         return self.out.add_into(a, x, then_norm, self.rt.act_dtype, scale=self.out_scale)
 
+    def from_rows(self, rows, ctx, binding):
+        """The heads' results (what the output product reads) from the stacked input product's float32 rows
+        [rows, q | k | v (| gate)], whole, or a column range of wider rows."""
+        if not self.head_norm_path:
+            return self._attend_rotating(None, ctx, binding, rows)
+        return self._attend_extended(None, ctx, binding, rows)
+
     def produce(self, h, ctx, binding):
         """attention(h) in float32 (whole, or in K slices of the output product), for a block that
         adds it up itself."""
@@ -190,59 +213,70 @@ class Attention(Mixer):
             raise ValueError("a mixer that hands its result over has no multiplier of its own")
         return self.out.raw(self._attend(h, ctx, binding))
 
-    def _attend_rotating(self, h, ctx, binding):
+    def _attend_rotating(self, h, ctx, binding, rows=None):
         """The extended path of mixers that rotate (or have no position encoding and no head norms): the plain path's
         rotate-and-store kernel with the values' own size, attention with the sink's scores, the output gate."""
         rt = self.rt
         if not binding.writes_cache:
             raise RuntimeError("this mixer stores the keys and values it reads")
         # (with a gate the product is taken whole: the gate's columns are read where they lie)
-        qkv = None if self.out_gate else self.qkv.partial(h)
         bias = None
-        if qkv is not None:
-            bias = self.qkv.bias
+        if rows is not None:
+            qkv = rows.contiguous()
         else:
-            qkv = self.qkv(h, torch.float32)
+            qkv = None if self.out_gate else self.qkv.partial(h)
+            if qkv is not None:
+                bias = self.qkv.bias
+            else:
+                qkv = self.qkv(h, torch.float32)
         inv_freq, freq_factors, rot_dims = self.position.rotary_tables()
         page_table = ctx.page_table(binding.group)
         q = ops.rope_kv_store(qkv, rt.act_dtype, inv_freq, freq_factors, rot_dims, ctx.row_pos, ctx.row_seq,
                               binding.k_cache, binding.v_cache, page_table, self.heads_q, self.heads_kv, self.head_dim,
                               bias=bias, v_dim=self.v_dim, magnitude=float(getattr(self.position, "magnitude", 1.0)))
         # the gate rides in the attention kernel's last pass (or, when a row's pages are shared out, in the merge)
-        gate = qkv[:, self.g_off:self.g_off + self.heads_q * self.v_dim] if self.out_gate else None
+        gate = qkv[:, self.g_off:self.g_off + self.gate_width] if self.out_gate else None
         a = ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
                                  self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
                                  fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate)
         return a
 
-    def _attend_extended(self, h, ctx, binding):
+    def _attend_extended(self, h, ctx, binding, rows=None):
         if not self.head_norm_path:
-            return self._attend_rotating(h, ctx, binding)
+            return self._attend_rotating(h, ctx, binding, rows)
         rt = self.rt
         writes = binding.writes_cache
+        if not writes and (rows is not None or self.out_gate):
+            raise RuntimeError("this mixer stores the keys and values it reads")
         if not writes:
             self.query_only()
-        proj = self.qkv if writes else self._q_only
-        qkv = proj.partial(h)
-        if qkv is None:
-            qkv = proj(h, torch.float32)
+        qkv = rows
+        if rows is None:
+            proj = self.qkv if writes else self._q_only
+            qkv = None if self.out_gate else proj.partial(h)
+            if qkv is None:
+                qkv = proj(h, torch.float32)
         v_first = v_out = None
         if writes and self.value_mix is not None:
             shared = ctx.shared
             if self.value_mix == "first":
-                v_out = torch.empty((ctx.n_rows, self.heads_kv * self.v_dim), dtype=torch.float32, device=h.device)
+                v_out = torch.empty((ctx.n_rows, self.heads_kv * self.v_dim), dtype=torch.float32, device=rt.device)
                 shared[self.value_mix_key] = v_out
             else:
                 v_first = shared.get(self.value_mix_key)
                 if v_first is None:
                     raise RuntimeError(f"no earlier layer of this step has left its values under {self.value_mix_key!r}")
         page_table = ctx.page_table(binding.group)
+        inv_freq, _, rot_dims = self.position.rotary_tables()
         q = ops.headnorm_kv_store(qkv, rt.act_dtype, self.q_norm, self.k_norm, self.qk_norm_eps, ctx.row_pos, ctx.row_seq,
                                   binding.k_cache, binding.v_cache, page_table, self.heads_q, self.heads_kv,
-                                  self.head_dim, self.v_dim, store=writes, v_first=v_first, lam=self.lam, v_out=v_out)
+                                  self.head_dim, self.v_dim, store=writes, v_first=v_first, lam=self.lam, v_out=v_out,
+                                  inv_freq=inv_freq, rot_dims=rot_dims if inv_freq is not None else 0,
+                                  unit=self.qk_norm and self.q_norm is None)
+        gate = qkv[:, self.g_off:self.g_off + self.gate_width] if self.out_gate else None
         return ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
                                     self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
-                                    fast=rt.fast_kernels, sink_scores=self.sink_scores)
+                                    fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate)
 
     def _attend(self, h, ctx, binding):
         """The heads' results [rows, heads_q * v_dim] in the activation type; keys and values of the

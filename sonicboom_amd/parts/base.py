@@ -23,8 +23,9 @@ copy in the activation type, ``ctx`` the step's
                 (their launches depend on device buffers only, so a decode step may be
                 recorded once and replayed).
                 Mixers and feed-forwards may also offer ``produce(h, ctx[, binding])``, which returns the
-                result (a float32 tensor, K slices of it, or a :class:`Branch`) instead of adding it:
-                blocks that norm a sublayer's output need it.
+                result (a float32 tensor, K slices of it, a :class:`Branch`, or a list of :class:`Joined`)
+                instead of adding it: blocks that norm a sublayer's output, or join their branches in one
+                pass, need it.
 * **block**     ``mixer`` attribute and ``forward(x, ctx, binding, h=None, next_norm=None)``;
                 optionally ``first_norm``, the norm the block starts with (the block before
                 may then hand over ``h`` = first_norm(x) from its last pass), ``state_specs() ->
@@ -32,6 +33,10 @@ copy in the activation type, ``ctx`` the step's
                 ``binding.states["block.<name>"]``), and calls of
                 ``ctx.trace(name, x)`` after its mixer and feed-forward when that is set.
 * **embedding** ``forward(ids, ctx) -> x`` (``ctx.row_pos`` for embeddings that add a position's row)
+* **junction**  what stands between two blocks of the run order: ``begin(x0, ctx)`` once a step with the
+                embedding's output, ``forward(x, ctx, turn, next_norm=, h=)`` where the order says so, which
+                overwrites x (``turn``: the number of the pass) and returns next_norm(x) when its last
+                pass could make it; ``first_norm`` as a block has it
 * **head**      ``forward(h) -> float32 logits [rows, vocab]``
 """
 from __future__ import annotations
@@ -43,7 +48,7 @@ import torch
 
 from .spec import PartSpec
 
-CATEGORIES = ("norm", "position", "mixer", "ffn", "block", "embedding", "head")
+CATEGORIES = ("norm", "position", "mixer", "ffn", "block", "embedding", "junction", "head")
 
 
 @dataclass(frozen=True)
@@ -107,6 +112,20 @@ class Branch:
     part_weights: Optional[torch.Tensor] = None
     extra: Optional[torch.Tensor] = None
     extra_weights: Optional[torch.Tensor] = None
+
+
+@dataclass
+class Joined:
+    """What a sublayer hands to a block that joins several branches in one pass: ``scale`` times the sum of
+    ``part``'s slices (float32 [rows, width], or [slices, rows, width]), divided by its root mean square and
+    multiplied by ``norm_weight`` first when that is given (``eps`` inside the root)."""
+    part: torch.Tensor
+    scale: float = 1.0
+    norm_weight: Optional[torch.Tensor] = None
+    eps: float = 0.0
+
+    def term(self):
+        return (self.part, self.scale, self.norm_weight is not None, self.norm_weight)
 
 
 class Part:

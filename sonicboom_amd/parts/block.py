@@ -18,14 +18,16 @@ stream in the activation type for the sublayer that reads it next.
 ``parallel``: both sublayers read the same stream, each through a norm of its own, and their results
 join it together: x += mixer(norm1(x)) + ffn(norm2(x)).  One pass norms the stream for both (the root
 mean square is the same, the weights differ); the mixer and the feed-forward then add into the stream
-one after the other.
+one after the other.  Without a second norm both sublayers read the first one's result, x += mixer(h) + ffn(h)
+with h = norm1(x): they hand their results over (``produce``) and one pass adds the slices of all of
+them, norms those that are normed, adds the sum into the stream and leaves what the next block reads.
 """
 from __future__ import annotations
 
 import torch
 
 from .. import ops
-from .base import Branch, Part, StateSpec, register_part
+from .base import Branch, Joined, Part, StateSpec, register_part
 from .spec import PartSpec, TensorSpec
 
 
@@ -117,7 +119,9 @@ class StreamAsItIs:
     in the activation type.  A block before it that cannot produce that in its last pass is simply
     followed by the conversion."""
     fusable = False
+    join_kind = "copy"
     weight = None
+    eps = 0.0
 
     def forward(self, x, out_dtype, rows=None):
         if rows is not None:
@@ -173,12 +177,45 @@ class OutNormBlock(Part):
 
 
 def parallel_block_spec(mixer_norm: PartSpec, mixer: PartSpec, ffn_norm: PartSpec = None, ffn: PartSpec = None) -> PartSpec:
+    """``ffn_norm`` None: the feed-forward reads the mixer's norm."""
     parts = {"mixer_norm": mixer_norm, "mixer": mixer}
     if ffn is not None:
-        if ffn_norm is None:
-            raise ValueError("a block with a feed-forward needs the norm before it")
-        parts.update(ffn_norm=ffn_norm, ffn=ffn)
+        parts["ffn"] = ffn
+        if ffn_norm is not None:
+            parts["ffn_norm"] = ffn_norm
     return PartSpec("block", "parallel", {}, {}, parts)
+
+
+def _terms(y):
+    """A sublayer's result as terms of the joining pass."""
+    if isinstance(y, Joined):
+        return [y]
+    if isinstance(y, (list, tuple)):
+        return [t for one in y for t in _terms(one)]
+    return [Joined(y)]
+
+
+def join_branches(x, results, act_dtype, next_norm=None):
+    """x += the sublayers' ``results`` in one pass over the row; next_norm(x) in ``act_dtype`` when that pass can make
+    it, else None."""
+    terms = []
+    for y in results:
+        if isinstance(y, Branch):       # slices with a multiplier a row each: a pass of their own, after which they are in x
+            ops.norm_add(x, y.part, None, 0.0, 0.0, None, part_weights=y.part_weights, extra=y.extra,
+                         extra_weights=y.extra_weights, by_row=y.by_row, norm=False)
+        else:
+            terms += _terms(y)
+    kind = getattr(next_norm, "join_kind", None)
+    epses = {t.eps for t in terms if t.norm_weight is not None}
+    if len(epses) > 1:
+        raise ValueError("the branches of a block are normed with one eps")
+    # (the pass takes a few branches; what is more goes first)
+    while len(terms) > ops.JOIN_MAX_TERMS:
+        ops.join(x, x, [t.term() for t in terms[:ops.JOIN_MAX_TERMS]], act_dtype, max(epses, default=0.0))
+        terms = terms[ops.JOIN_MAX_TERMS:]
+    return ops.join(x, x, [t.term() for t in terms], act_dtype, max(epses, default=0.0), then=kind,
+                    then_weight=next_norm.weight if kind else None, then_eps=next_norm.eps if kind else 0.0,
+                    out_dtype=act_dtype)
 
 
 @register_part("block", "parallel")
@@ -191,9 +228,13 @@ class ParallelBlock(Part):
         self.mixer = parts["mixer"]
         self.ffn_norm = parts.get("ffn_norm")
         self.ffn = parts.get("ffn")              # None: the block is its mixer's branch alone
+        # both branches read one norm's result: where both hand their results over, one pass joins them
+        self.one_norm = self.ffn is not None and self.ffn_norm is None
+        self.joins = all(hasattr(p, "produce") for p in (self.mixer, self.ffn) if p is not None) \
+            and (self.one_norm or not hasattr(self.mixer, "fuses_norm"))
         # with two branches the block norms for both in one pass of its own; alone, the mixer's norm is what
         # the block before may apply in its last pass
-        self.first_norm = self.mixer_norm if self.ffn is None else None
+        self.first_norm = self.mixer_norm if self.ffn is None or self.one_norm else None
         a, b = self.mixer_norm, self.ffn_norm
         # one pass for both norms when they are RMS norms over whole rows with the same eps and plain weights
         self.one_pass = b is not None and all(
@@ -207,6 +248,22 @@ class ParallelBlock(Part):
         Both branches are normed before either result joins the stream."""
         act = self.rt.act_dtype
         f = None
+        trace = getattr(ctx, "trace", None)
+        if self.one_norm or (self.ffn is None and self.joins):
+            if h is None:
+                h = self.mixer_norm.forward(x, act)
+            out = None
+            if self.joins:
+                results = [self.mixer.produce(h, ctx, binding)]
+                if self.ffn is not None:
+                    results.append(self.ffn.produce(h, ctx))
+                out = join_branches(x, results, act, next_norm)
+            else:
+                self.mixer.forward(h, x, ctx, binding)
+                self.ffn.forward(h, x, ctx)
+            if trace is not None:
+                trace("after_mixer" if self.ffn is None else "after_ffn", x)
+            return out
         if self.ffn is not None:
             if h is None and self.one_pass:
                 h, f = ops.rmsnorm_pair(x, self.mixer_norm.weight, self.ffn_norm.weight, self.mixer_norm.eps, act)
@@ -219,7 +276,6 @@ class ParallelBlock(Part):
             out = self.mixer.forward(h, x, ctx, binding, then_norm=next_norm if last else None)
         else:
             out = self.mixer.forward(h, x, ctx, binding)
-        trace = getattr(ctx, "trace", None)
         if trace is not None:
             trace("after_mixer", x)
         if last:

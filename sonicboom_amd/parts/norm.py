@@ -1,4 +1,4 @@
-"""RMS norm (/root/reference/core/src/nn/norm.cpp:25-42), whole rows or in groups."""
+"""RMS norm (/root/reference/core/src/nn/norm.cpp:25-42), whole rows or in groups, and the layer norm."""
 from __future__ import annotations
 
 from .. import ops
@@ -34,9 +34,33 @@ class RMSNorm(Part):
         # a projection's last pass may apply this norm (it exposes weight, eps and groups); the fused
         # passes multiply by the weight as it is
         self.fusable = self.offset == 0.0
+        # the pass that joins a block's branches may apply it (ops.join)
+        self.join_kind = "rms" if self.fusable and self.groups == 1 else None
         self.weight = tensors.get("weight")
 
     def forward(self, x, out_dtype, rows=None):
         if self.offset:
             return ops.offset_norm(x, self.weight, self.eps, self.offset, out_dtype, rows)
         return ops.rmsnorm(x, self.weight, self.eps, out_dtype, rows, groups=self.groups)
+
+
+def layernorm_spec(weight_name: str, width: int, eps: float) -> PartSpec:
+    return PartSpec("norm", "layernorm", {"width": width, "eps": float(eps)},
+                    {"weight": TensorSpec(weight_name, (width,), init=(1.0, 0.02))})
+
+
+@register_part("norm", "layernorm")
+class LayerNorm(Part):
+    """y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w over the whole row, without a bias."""
+    category = "norm"
+    fusable = False            # the products' last passes apply RMS norms
+    join_kind = "layer"
+
+    def __init__(self, spec, tensors, parts, rt):
+        super().__init__(spec, tensors, parts, rt)
+        self.width = int(spec.params["width"])
+        self.eps = float(spec.params["eps"])
+        self.weight = tensors.get("weight")
+
+    def forward(self, x, out_dtype, rows=None):
+        return ops.layernorm(x, self.weight, self.eps, out_dtype, rows)

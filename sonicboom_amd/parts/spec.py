@@ -35,7 +35,7 @@ class TensorSpec:
 @dataclass
 class PartSpec:
     """A part: its category ("mixer", "ffn", "norm", "position", "block",
-    "embedding", "head"), its kind within the category, its constants, the
+    "embedding", "junction", "head"), its kind within the category, its constants, the
     tensors it owns by role, and the parts nested in it by role."""
     category: str
     kind: str
@@ -59,10 +59,14 @@ class OrderEntry:
     with the same number share keys and values; the one with ``writes_cache``
     stores them, the others only read.  ``None`` means the mixer keeps nothing
     per token.  Per-sequence state of fixed size belongs to the entry itself.
+    ``junction`` indexes ``ModelSpec.junctions``: that part acts on the stream
+    right before the block, as the number ``turn`` of its turns.
     """
     block: int
     cache: Optional[int] = None
     writes_cache: bool = True
+    junction: Optional[int] = None
+    turn: int = 0
 
 
 @dataclass
@@ -79,10 +83,11 @@ class ModelSpec:
     stop_tokens: Tuple[int, ...] = ()
     # Names that may be in the file without being used (a tied head's copy).
     ignorable_tensors: Tuple[str, ...] = ()
+    junctions: List[PartSpec] = field(default_factory=list)     # what order entries name as their junction
 
     def all_tensors(self) -> List[TensorSpec]:
         seen, out = set(), []
-        parts = [self.embedding, *self.blocks, self.final_norm, self.head]
+        parts = [self.embedding, *self.junctions, *self.blocks, self.final_norm, self.head]
         for p in parts:
             for t in p.all_tensors():
                 if t.name not in seen:
@@ -95,6 +100,8 @@ class ModelSpec:
         for i, e in enumerate(self.order):
             if not 0 <= e.block < len(self.blocks):
                 raise ValueError(f"order entry {i} names block {e.block}, the model has {len(self.blocks)}")
+            if e.junction is not None and not 0 <= e.junction < len(self.junctions):
+                raise ValueError(f"order entry {i} names junction {e.junction}, the model has {len(self.junctions)}")
             if e.cache is not None and e.writes_cache:
                 if e.cache in caches_written:
                     raise ValueError(
