@@ -265,9 +265,9 @@ def main() -> int:
     ap.add_argument("--prompt", type=int, default=PROMPT, help="cached prompt tokens per sequence")
     ap.add_argument("--context", type=int, default=CONTEXT, help="cache size per sequence")
     ap.add_argument("--workload", choices=("steady", "mixed", "forms", "designs"), default="steady")
-    ap.add_argument("--design", choices=("rasizen", "tatelorn", "nalasun", "fitatar"), default="rasizen",
+    ap.add_argument("--design", choices=("rasizen", "tatelorn", "nalasun", "fitatar", "dudatar"), default="rasizen",
                     help="--workload designs: the design that runs beside the Qwen2.5 design")
-    ap.add_argument("--beside", choices=("qwen2", "rasizen", "tatelorn", "nalasun", "fitatar"), default="qwen2",
+    ap.add_argument("--beside", choices=("qwen2", "rasizen", "tatelorn", "nalasun", "fitatar", "dudatar"), default="qwen2",
                     help="--workload designs: the design at the same sizes that the first one runs beside")
     ap.add_argument("--design-sizes", default="2048,4096",
                     help="--workload designs: the widths of the layer sizes to run, comma separated")
@@ -742,6 +742,25 @@ def fitatar_sizes(width, vocab=32768, experts=8, top=2):
             "norm": {"eps": 1e-6}, "layers": layers}
 
 
+def dudatar_sizes(width, vocab=32768):
+    """Layer sizes in the manner of a real model of this width: four layers of which the middle two run three times
+    (eight layer runs): attention with heads of 128 (a quarter of them kv heads) beside retention with heads of 128 x 128
+    (half as many), and gated linear attention with as many heads of 128 x 128 as the Qwen2.5 layer has; a gated
+    feed-forward of the Qwen2.5 layer's weights in every layer."""
+    heads = width // 128
+    inner = (8 * width // 3 + 255) // 256 * 256
+    right = max(1, heads // 2)
+    both = {"type": "parallel", "mlp": {"kind": "dense", "ff": inner}, "mixer": {
+        "left": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                 "rot": {"base": 1e6, "dims": 64}},
+        "right": {"heads": right, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-5 - 5.0 * i / right) for i in range(right)],
+                  "rot": {"base": 1e6, "dims": 128}}}}
+    linear = {"type": "gla", "mlp": {"kind": "dense", "ff": inner},
+              "mixer": {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "rank": 16}}
+    return {"architecture": "Dudatar", "vocab": vocab, "width": width, "logit_softcap": 30.0, "norm": {"eps": 1e-6},
+            "loop": {"start": 1, "stop": 3, "times": 3}, "layers": [both, both, linear, both]}
+
+
 VECTOR_F32_FLOPS = 157.3e12      # the vector units' float32 peak, against which the recurrences' scans are priced
 
 
@@ -753,7 +772,7 @@ class AllOpsTimer:
             "attention_tall_ok", "attention_mfma_ok", "attention_decode_rope_ok", "gate_code", "reduce_resid_norm_ok",
             "attention_decode_pages_per_wave", "gemm_tile_shape", "gemm_few_rows_kernel", "mingru_chunk_rows",
             "loaded_paths", "check", "latent_attention_mfma_ok", "capped_attention_mfma_ok", "moe_max_top", "moe_plan",
-            "time_conv_max_taps", "state_scan_limits", "state_scan_chunk_rows", "shared_attention_mfma_ok")
+            "time_conv_max_taps", "state_scan_limits", "state_scan_chunk_rows", "shared_attention_mfma_ok", "decay_scan_max_side", "decay_chunk_rows")
     INNER = ("attention_plain", "attention_decode_mfma", "attention_prefill_mfma", "latent_attention_plain",
              "latent_attention_mfma", "attention_capped_plain", "attention_capped_mfma",
              "moe_product_plain", "attention_shared_plain", "attention_shared_mfma",
@@ -786,6 +805,10 @@ class AllOpsTimer:
                         label = f"{_name} {n}x{k}"
                     elif _name == "head_product":
                         label = f"{_name} {tuple(args[1].shape)}"
+                    elif _name == "join":
+                        label = f"{_name} {len(args[2])} branches"
+                    elif _name == "decay_scan":
+                        label = f"{_name} {'channel' if kw.get('log_decay') is not None else 'head'} {args[6]}x{args[7]}x{args[8]}"
                     elif _name == "time_conv":
                         label = f"{_name} {args[1].shape[0]}"
                     elif _name in ("activate", "sigmoid_mul_", "rmsnorm_pair"):
@@ -884,6 +907,17 @@ def design_roofline(label, us, calls, rows, depth, batch, width, cfgs):
         h, d, e = cfgs["delta"]
         nbytes = rows * (4 * (2 * h * d + 3 * h * e) + 2 * h * e) + (2 * batch * 4 * h * d * e if decode else 0)
         flops, peak_f = rows * h * d * e * 7, VECTOR_F32_FLOPS
+    elif label.startswith("decay_scan"):
+        h, d, e = (int(v) for v in label.split()[-1].split("x"))
+        own = 1 if "channel" in label else 0
+        nbytes = rows * (4 * h * ((2 + own) * d + 2 * e) + 2 * h * e) + (2 * batch * 4 * h * d * e if decode else 0)
+        flops, peak_f = rows * h * d * e * 4, VECTOR_F32_FLOPS
+    elif label == "log_decay":
+        nbytes = rows * H * 128 * 4
+    elif label == "layernorm":
+        nbytes = (rows if calls > 1 or decode else 1) * width * (4 + 2)
+    elif label.startswith("join"):
+        nbytes = rows * width * (4 * int(label.split()[1]) + 8 + 2)      # one slice of every branch at least
     elif label == "qk_rownorm_store":
         nbytes = rows * (H * 128 + cfgs["kvw"]) * (4 + 2) + rows * cfgs["kvw"] * 2
     elif label == "attention_shared":
@@ -907,7 +941,7 @@ def design_comparison(a) -> int:
     out, table = {}, []
     for width in (int(v) for v in a.design_sizes.split(",")):
         sizes = {"rasizen": rasizen_sizes, "tatelorn": tatelorn_sizes, "nalasun": nalasun_sizes, "fitatar": fitatar_sizes,
-                 "qwen2": qwen_sizes}
+                 "dudatar": dudatar_sizes, "qwen2": qwen_sizes}
         for design, cfg in ((a.design, sizes[a.design](width)), (a.beside, sizes[a.beside](width))):
             model = DecoderModel.from_random(cfg, seed=0, dtype="bfloat16", device="cuda:0")
             heads = width // 128

@@ -183,6 +183,8 @@ class PagedCache:
         return len(self._free_slots)
 
     def held_pages(self, group: int = 0) -> int:
+        if not self.pools:            # a model whose mixers keep no keys: states alone
+            return 0
         return self.pools[group].n_pages - self.pools[group].free_count
 
     # ---- a step ------------------------------------------------------------

@@ -43,7 +43,7 @@ CORE_SOURCES = [
     "attention_plain.hip", "sampling.hip", "gemm_skinny.hip", "gemm_stream.hip", "gemm_mfma.hip",
     "random_fill.hip", "recurrent.hip", "attention_latent.hip", "attention_latent_mfma.hip",
     "outnorm.hip", "headnorm_kv.hip", "moe.hip", "moe_mfma.hip", "timeconv.hip", "state_space.hip",
-    "attention_mixed.hip", "join.hip", "decay_scan.hip",
+    "attention_mixed.hip", "join.hip", "decay_scan.hip", "decay_chunks.hip",
 ]
 HEADERS = ["common.h", "sb_hip.h", "mfma.h"]
 ATTN_SOURCES = ["attention_mfma.hip"]

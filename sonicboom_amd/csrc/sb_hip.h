@@ -540,18 +540,29 @@ int sb_join(float *out, const float *base, const void *const *term_ptrs, const i
 int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dtype, const int32_t *rows, int n_rows,
                  int width, float eps, int few, void *stream);
 
-/* ---- linear attention with decays (csrc/decay_scan.hip) ------------------------------------------
+/* ---- linear attention with decays (csrc/decay_scan.hip, csrc/decay_chunks.hip) --------------------
  * sb_decay_scan: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t per head (S f32 D x E in
  *   state[slots[s]]), out_t = o_t / rms(o_t) (* w) * silu(g_t); alpha from log_decay f32 [rows, heads * D], or one
  *   number a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
  *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart.
- * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width]. */
+ * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width].
+ * sb_decay_chunks: the same scan over runs of sb_decay_chunk_rows(D) rows (chunks int32 [n_chunks, 4], sequence after
+ *   sequence, each sequence's runs full but its last) on the matrix cores in float32; q and k turn by `angles` f32
+ *   [n_rows, half, 2] (sb_angle_table; NULL: not); part f32 [n_chunks, heads, D, E] and, with log_decay, part_decay f32
+ *   [n_chunks, heads, D] are scratch. */
 int sb_decay_scan_max_side(void);
 int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
                   int row_stride, const float *log_decay, int ld_stride, const float *decay, const float *inv_freq,
                   int rot_dims, const int32_t *row_pos, float q_scale, float k_scale, const void *w, int w_dtype, float eps,
                   float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E,
                   void *stream);
+int sb_decay_chunk_rows(int D);
+int sb_angle_table(float *out, const int32_t *row_pos, const float *inv_freq, int n_rows, int half, void *stream);
+int sb_decay_chunks(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
+                    int row_stride, const float *log_decay, int ld_stride, const float *decay, const float *angles, int half,
+                    float q_scale, float k_scale, const void *w, int w_dtype, float eps, float *state,
+                    const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E, const int32_t *chunks,
+                    int n_chunks, int chunk_rows, float *part, float *part_decay, void *stream);
 int sb_log_decay(float *out, int out_stride, const float *a, int a_stride, const float *w, const float *bias, int n_rows,
                  int rank, int width, float rate, void *stream);
 

@@ -1926,6 +1926,22 @@ def decay_scan_max_side() -> int:
     return int(library.core().sb_decay_scan_max_side())
 
 
+def decay_chunk_rows(dim: int) -> int:
+    """The rows of a chunk of the chunked form of :func:`decay_scan` for heads of ``dim`` key channels."""
+    return int(library.core().sb_decay_chunk_rows(int(dim)))
+
+
+def angle_table(row_pos: torch.Tensor, inv_freq: torch.Tensor, n_rows: int) -> torch.Tensor:
+    """Cosine and sine of row_pos[r] * inv_freq[i], float32 [n_rows, pairs, 2]."""
+    _dev(row_pos, inv_freq)
+    _i32(row_pos, n_rows, "row positions")
+    half = inv_freq.numel()
+    _f32_vec(inv_freq, half, "frequencies")
+    out = torch.empty((n_rows, half, 2), dtype=torch.float32, device=inv_freq.device)
+    check(library.core().sb_angle_table(_p(out), _p(row_pos), _p(inv_freq), n_rows, half, _stream()))
+    return out
+
+
 def log_decay(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], rate: float) -> torch.Tensor:
     """rate * log(sigmoid(a w + bias)) in float32: ``a`` float32 [n, rank] (a view of wider rows is fine), ``w`` float32
     [rank, width], ``bias`` float32 [width]; [n, width]."""
@@ -1943,14 +1959,19 @@ def log_decay(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], ra
 def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, state: torch.Tensor, ctx, heads: int,
                dim: int, v_dim: int, eps: float, out_dtype: torch.dtype, log_decay: Optional[torch.Tensor] = None,
                decay: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, q_scale: float = 1.0,
-               k_scale: float = 1.0, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0) -> torch.Tensor:
+               k_scale: float = 1.0, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
+               chunks: Optional[torch.Tensor] = None, angles: Optional[torch.Tensor] = None) -> torch.Tensor:
     """S = alpha S + k v^T, o = S^T q per head over every sequence's rows of the step, from ``state`` float32
     [slots, heads, dim, v_dim], which moves on; returns o / rms(o) (* weight) * silu(g) [n, heads*v_dim] in ``out_dtype``.
 
     ``q``, ``k`` [n, heads*dim], ``v``, ``g`` [n, heads*v_dim]: float32 parts of the same wider rows.  alpha: the
     exponential of ``log_decay`` float32 [n, heads*dim], or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
     pairs (i, i + rot_dims/2) of every head of q and k turn by position * inv_freq[i]; then q and k are multiplied by
-    their scales."""
+    their scales.
+
+    ``chunks`` int32 [n, 4]: the step's rows in runs of :func:`decay_chunk_rows` rows; the scan then takes its chunked form
+    (float32 throughout; it orders its sums otherwise than the walk, from which it differs by rounding), and turns by
+    ``angles``, the step's :func:`angle_table`."""
     n = q.shape[0]
     _on_gpu(q, k, v, g)
     for t, width, what in ((q, heads * dim, "queries"), (k, heads * dim, "keys"), (v, heads * v_dim, "values"),
@@ -1975,6 +1996,25 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     _i32(ctx.cu_rows, ctx.n_seqs + 1, "first rows")
     _i32(ctx.slots, ctx.n_seqs, "slots")
     out = torch.empty((n, heads * v_dim), dtype=out_dtype, device=q.device)
+    n_chunks = _scan_chunks(chunks)
+    if n_chunks:
+        if inv_freq is None:
+            angles = None
+        else:
+            _dev(angles)
+            if angles is None or angles.dtype != torch.float32 or tuple(angles.shape) != (n, rot_dims // 2, 2):
+                raise KernelLibraryError(f"the chunked scan turns by a table of angles, float32 [{n}, {rot_dims // 2}, 2]")
+        part = torch.empty((n_chunks, heads, dim, v_dim), dtype=torch.float32, device=q.device)
+        part_decay = None
+        if log_decay is not None:
+            part_decay = torch.empty((n_chunks, heads, dim), dtype=torch.float32, device=q.device)
+        check(library.core().sb_decay_chunks(
+            _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
+            log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(angles), rot_dims // 2 if angles is not None else 0,
+            float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
+            _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _p(chunks), n_chunks, decay_chunk_rows(dim), _p(part),
+            _p(part_decay), _stream()))
+        return out
     check(library.core().sb_decay_scan(
         _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
         log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),

@@ -101,6 +101,10 @@ _CORE_SIGNATURES = {
     "sb_decay_scan_max_side": [],
     "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
                       _P],
+    "sb_decay_chunk_rows": [_I],
+    "sb_angle_table": [_P, _P, _P, _I, _I, _P],
+    "sb_decay_chunks": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I, _P,
+                        _I, _I, _P, _P, _P],
     "sb_log_decay": [_P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P],
 }
 # Entry points of later kernels; declared when the library has them.

@@ -13,7 +13,9 @@ The input projections are stacked into one matrix, so a step runs one product; i
 everything that follows up to the output product's operand is float32: rotation, the decays' second product, their
 logarithms and exponentials, the state, the read-out, the norm and the gate.  The state is per-sequence state of the
 cache (a row per slot, zeroed when the slot is handed out, moved on by every step), so prompts cut into steps,
-batches and decoding all run the same recurrence, to the bit in the 32-bit path.
+batches and decoding all run the same recurrence, to the bit in the 32-bit path.  With bfloat16 activations a step
+that brings a sequence more rows than a chunk takes the scan's chunked form on the matrix cores (float32 throughout;
+it differs from the walk by rounding); the 32-bit path always walks.
 
 ``side_by_side``: two mixers that read the same input and meet as weight * (n(left) + n(right)), n the RMS norm over
 the model's width with a weight of its own.  Their input matrices are stacked into one product; the pass that joins
@@ -90,6 +92,12 @@ class _DecayMixer(Mixer):
         self.input_weight = stacked if p.get("given_input") else None
         self.inp = None if p.get("given_input") else Linear(stacked, None, rt.fast_kernels)
         self.out = Linear(tensors["out"], None, rt.fast_kernels)
+        # the chunked form takes a step's rows in runs of this many (the context lists them)
+        self.chunk = ops.decay_chunk_rows(self.head_dim) if rt.act_dtype != torch.float32 and stacked.is_cuda else 0
+        self.row_tile = self.chunk or None
+
+    def _chunks(self, ctx):
+        return ctx.row_tiles(self.chunk) if self.chunk and ctx.max_new > self.chunk else None
 
     def further_inputs(self, tensors):
         return []
@@ -132,12 +140,23 @@ class Retention(_DecayMixer):
             raise ValueError("retention takes no rotation, or the rotate-half one by plain frequencies")
         self.inv_freq, _, rot_dims = tables
         self.rot_dims = rot_dims if self.inv_freq is not None else 0
+        self.turns = None if self.inv_freq is None else ("angles", tuple(self.inv_freq.tolist()))
+
+    def _angles(self, ctx):
+        """The step's cosines and sines: one table for all mixers that turn alike."""
+        shared = ctx.shared if ctx.shared is not None else {}
+        if self.turns not in shared:
+            shared[self.turns] = ops.angle_table(ctx.row_pos, self.inv_freq, ctx.n_rows)
+        return shared[self.turns]
 
     def from_rows(self, rows, ctx, binding):
         """What the output product reads, from the stacked product's float32 rows (a column range of wider rows is fine)."""
         q, k, v, g = self._cut(rows)
+        chunks = self._chunks(ctx)
+        angles = self._angles(ctx) if chunks is not None and self.turns is not None else None
         return ops.decay_scan(q, k, v, g, binding.state, ctx, self.heads, self.head_dim, self.v_dim, self.eps, self.rt.act_dtype,
-                              decay=self.decay, k_scale=self.head_dim ** -0.5, inv_freq=self.inv_freq, rot_dims=self.rot_dims)
+                              decay=self.decay, k_scale=self.head_dim ** -0.5, inv_freq=self.inv_freq, rot_dims=self.rot_dims,
+                              chunks=chunks, angles=angles)
 
 
 @register_part("mixer", "gated_linear_attention")
@@ -165,7 +184,7 @@ class GatedLinearAttention(_DecayMixer):
         first = 2 * (self.qk_width + self.v_width)
         log_decay = ops.log_decay(rows[:, first:first + self.rank], self.decay_up, self.decay_bias, self.rate)
         return ops.decay_scan(q, k, v, g, binding.state, ctx, self.heads, self.head_dim, self.v_dim, self.eps, self.rt.act_dtype,
-                              log_decay=log_decay, weight=self.norm, q_scale=self.head_dim ** -0.5)
+                              log_decay=log_decay, weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
 
 
 def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float, left_norm: str, right_norm: str,

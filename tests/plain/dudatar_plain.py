@@ -197,3 +197,13 @@ def forward(cfg, w, tokens, layers_out=None):
     z = linear(layer_norm(x, w["final.norm"], cfg["norm"]["eps"]), w["head"])
     cap = float(cfg.get("logit_softcap") or 0.0)
     return cap * np.tanh(z / cap) if cap else z
+
+
+def greedy(cfg, w, prompt, n: int):
+    """``n`` tokens after ``prompt``, each the first largest logit of the whole sequence so far."""
+    tokens, out = list(prompt), []
+    for _ in range(n):
+        t = int(np.argmax(forward(cfg, w, tokens)[-1]))
+        out.append(t)
+        tokens.append(t)
+    return out
