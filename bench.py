@@ -38,6 +38,8 @@ error, one JSON line to standard output.  ``--design tatelorn`` puts the Tatelor
 norm what their sublayers give back, attention with head norms, capped scores and a sink, routed
 experts) in the Rasizen design's place (``--design fitatar``: the Fitatar design, layers of two parallel branches with
 latent attention through a query latent, gated attention with a sink score a head and experts chosen within groups;
+``--design dudatar``: the Dudatar design, attention beside retention and gated linear attention, layers of one norm and
+a run of layers that is repeated;
 ``--design nalasun``: the Nalasun design, state-space and delta-rule
 recurrences, attention with shared head weights and routed experts behind short convolutions): eight layers, the first with a dense gated feed-forward, the
 others with eight experts of which a row takes two plus a shared one, so that a row passes as many
@@ -808,7 +810,7 @@ class AllOpsTimer:
                     elif _name == "join":
                         label = f"{_name} {len(args[2])} branches"
                     elif _name == "decay_scan":
-                        label = f"{_name} {'channel' if kw.get('log_decay') is not None else 'head'} {args[6]}x{args[7]}x{args[8]}"
+                        label = f"{_name} {'head' if kw.get('decay') is not None else 'channel'} {args[6]}x{args[7]}x{args[8]}"
                     elif _name == "time_conv":
                         label = f"{_name} {args[1].shape[0]}"
                     elif _name in ("activate", "sigmoid_mul_", "rmsnorm_pair"):

@@ -46,44 +46,106 @@ struct ChunkArgs {
   int vec4;                                  // rows can be read four numbers at a time
 };
 
-// Four numbers d .. d + 3 of a head's row `src`, turned and scaled; numbers past the head's last are zeros.
-__device__ __forceinline__ float4 load_head4(const ChunkArgs &a, const float *src, int row, int d, float scale) {
-  float x[4] = {0.f, 0.f, 0.f, 0.f};
-  if (d < a.D) {
-    if (a.vec4) {
-      const float4 v = *(const float4 *)(src + d);
-      x[0] = v.x; x[1] = v.y; x[2] = v.z; x[3] = v.w;
-      if (d < 2 * a.half) {            // (half is a multiple of 4 here: the four turn together)
-        const bool lo = d < a.half;
-        const int i = lo ? d : d - a.half;
-        const float4 o = *(const float4 *)(src + (lo ? d + a.half : d - a.half));
-        const float4 t0 = *(const float4 *)(a.angles + size_t(row) * a.half + i), t1 = *(const float4 *)(a.angles + size_t(row) * a.half + i + 2);
-        const float ov[4] = {o.x, o.y, o.z, o.w}, c[4] = {t0.x, t0.z, t1.x, t1.z}, s[4] = {t0.y, t0.w, t1.y, t1.w};
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          float y0, y1;
-          rotate_pair(lo ? x[e] : ov[e], lo ? ov[e] : x[e], c[e], s[e], y0, y1);
-          x[e] = lo ? y0 : y1;
-        }
-      }
-    } else {
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        if (d + e >= a.D) continue;
-        x[e] = src[d + e];
-        if (d + e < 2 * a.half) {
-          const bool lo = d + e < a.half;
-          const int i = lo ? d + e : d + e - a.half;
-          const float ov = src[lo ? d + e + a.half : d + e - a.half];
-          const float2 t = a.angles[size_t(row) * a.half + i];
-          float y0, y1;
-          rotate_pair(lo ? x[e] : ov, lo ? ov : x[e], t.x, t.y, y0, y1);
-          x[e] = lo ? y0 : y1;
-        }
-      }
+// What a thread needs for four numbers of a head's row: themselves, what they turn with, cosines and sines.
+struct Four { float4 x, o, t0, t1; };
+
+// The loads for numbers d .. d + 3 of row `row`; no branch stands between them (numbers past the head's last read its
+// last again, heads that do not turn skip the rest).  turning: 2 with their angles, 1 without (asked for before), 0 not.
+__device__ __forceinline__ void fetch_four(Four &f, const ChunkArgs &a, const float *head, int row, int d, int turning) {
+  const float *src = head + size_t(row) * a.row_stride;
+  const int at = min(d, a.D - 4);
+  f.x = *(const float4 *)(src + at);
+  if (turning) {            // (half is a multiple of 4: the four turn together, or none does)
+    const bool lo = at < a.half, on = at < 2 * a.half;
+    f.o = *(const float4 *)(src + (on ? (lo ? at + a.half : at - a.half) : at));
+    if (turning == 2) {
+      const float2 *t = a.angles + size_t(row) * a.half + (on ? (lo ? at : at - a.half) : 0);
+      f.t0 = *(const float4 *)t;
+      f.t1 = *(const float4 *)(t + 2);
     }
   }
+}
+
+__device__ __forceinline__ float4 finish_four(const Four &f, const ChunkArgs &a, int d, bool live, float scale, bool turning) {
+  float x[4] = {f.x.x, f.x.y, f.x.z, f.x.w};
+  if (turning) {
+    const bool lo = d < a.half, on = d < 2 * a.half;
+    const float o[4] = {f.o.x, f.o.y, f.o.z, f.o.w}, c[4] = {f.t0.x, f.t0.z, f.t1.x, f.t1.z}, s[4] = {f.t0.y, f.t0.w, f.t1.y, f.t1.w};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float y0, y1;
+      rotate_pair(lo ? x[e] : o[e], lo ? o[e] : x[e], c[e], s[e], y0, y1);
+      x[e] = on ? (lo ? y0 : y1) : x[e];
+    }
+  }
+  if (!live || d >= a.D) return make_float4(0.f, 0.f, 0.f, 0.f);
   return make_float4(x[0] * scale, x[1] * scale, x[2] * scale, x[3] * scale);
+}
+
+// The same for rows that cannot be read four numbers at a time.
+__device__ __forceinline__ float4 load_single(const ChunkArgs &a, const float *head, int row, int d, float scale) {
+  const float *src = head + size_t(row) * a.row_stride;
+  float x[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    if (d + e >= a.D) continue;
+    x[e] = src[d + e];
+    if (d + e < 2 * a.half) {
+      const bool lo = d + e < a.half;
+      const int i = lo ? d + e : d + e - a.half;
+      const float ov = src[lo ? d + e + a.half : d + e - a.half];
+      const float2 t = a.angles[size_t(row) * a.half + i];
+      float y0, y1;
+      rotate_pair(lo ? x[e] : ov, lo ? ov : x[e], t.x, t.y, y0, y1);
+      x[e] = lo ? y0 : y1;
+    }
+    x[e] *= scale;
+  }
+  return make_float4(x[0], x[1], x[2], x[3]);
+}
+
+// The chunk's queries (or NULL) and keys into LDS, rows of STRIDE numbers; rows past the chunk's last are zeros.
+template <int DP, int CR, int STRIDE>
+__device__ __forceinline__ void stage_heads(const ChunkArgs &a, const float *qp, const float *kp, int r0, int nr, float *qs, float *ks) {
+  constexpr int N = CR * (DP / 4) / THREADS;         // fours a thread
+  if (a.vec4) {
+    const bool turning = a.half > 0;
+    Four q[N], k[N];
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      const int idx = threadIdx.x + u * THREADS, row = r0 + min(idx / (DP / 4), nr - 1), d = (idx % (DP / 4)) * 4;
+      fetch_four(k[u], a, kp, row, d, turning ? 2 : 0);
+      if (qp) fetch_four(q[u], a, qp, row, d, turning ? 1 : 0);
+    }
+#pragma unroll
+    for (int u = 0; u < N; ++u) {
+      const int idx = threadIdx.x + u * THREADS, i = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
+      *(float4 *)&ks[i * STRIDE + d] = finish_four(k[u], a, d, i < nr, a.k_scale, turning);
+      if (qp) {
+        q[u].t0 = k[u].t0; q[u].t1 = k[u].t1;
+        *(float4 *)&qs[i * STRIDE + d] = finish_four(q[u], a, d, i < nr, a.q_scale, turning);
+      }
+    }
+  } else {
+    for (int idx = threadIdx.x; idx < CR * (DP / 4); idx += THREADS) {
+      const int i = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
+      float4 x = make_float4(0.f, 0.f, 0.f, 0.f), y = x;
+      if (i < nr) {
+        y = load_single(a, kp, r0 + i, d, a.k_scale);
+        if (qp) x = load_single(a, qp, r0 + i, d, a.q_scale);
+      }
+      *(float4 *)&ks[i * STRIDE + d] = y;
+      if (qp) *(float4 *)&qs[i * STRIDE + d] = x;
+    }
+  }
+}
+
+// The logarithms of a thread's channel over its part of the chunk's rows (rows past the last read the last again).
+template <int PR>
+__device__ __forceinline__ void fetch_logs(const ChunkArgs &a, float *l, int head, int r0, int nr, int d, int part) {
+  const float *src = a.log_decay + head * a.D + min(d, a.D - 1);
+#pragma unroll
+  for (int i = 0; i < PR; ++i) l[i] = src[size_t(r0 + min(part * PR + i, nr - 1)) * a.ld_stride];
 }
 
 // powers of the head's decay, 0 .. n
@@ -102,36 +164,39 @@ __global__ void __launch_bounds__(THREADS) chunk_local_kernel(ChunkArgs a) {
   const int r0 = c[0], nr = c[1];
   const float *kp = a.k + size_t(head) * a.D, *vp = a.v + size_t(head) * a.E;
   if (!CHANNEL) decay_powers(pw, a.decay[head], CR);
-  for (int idx = tid; idx < CR * (DP / 4); idx += THREADS) {
-    const int i = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
-    float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-    if (i < nr) x = load_head4(a, kp + size_t(r0 + i) * a.row_stride, r0 + i, d, a.k_scale);
-    *(float4 *)&ks[i][d] = x;
-  }
-  for (int idx = tid; idx < CR * (EP / 4); idx += THREADS) {
-    const int i = idx / (EP / 4), e = (idx % (EP / 4)) * 4;
-    float4 x = make_float4(0.f, 0.f, 0.f, 0.f);
-    const float *src = vp + size_t(r0 + i) * a.row_stride + e;
-    if (i < nr && e < a.E) {
-      if (a.vec4) x = *(const float4 *)src;
-      else {
-        x.x = src[0];
-        if (e + 1 < a.E) x.y = src[1];
-        if (e + 2 < a.E) x.z = src[2];
-        if (e + 3 < a.E) x.w = src[3];
-      }
+  // the logarithms are asked for first, then the values, then the keys
+  float l[CHANNEL ? PR : 1];
+  const int ch = tid % DP, part = tid / DP;
+  if (CHANNEL) fetch_logs<PR>(a, l, head, r0, nr, ch, part);
+  constexpr int NV = CR * (EP / 4) / THREADS;
+  if (a.vec4) {
+    float4 x[NV];
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int idx = tid + u * THREADS, row = r0 + min(idx / (EP / 4), nr - 1), e = (idx % (EP / 4)) * 4;
+      x[u] = *(const float4 *)(vp + size_t(row) * a.row_stride + min(e, a.E - 4));
     }
-    *(float4 *)&vs[i][e] = x;
+    stage_heads<DP, CR, KS>(a, nullptr, kp, r0, nr, nullptr, &ks[0][0]);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int idx = tid + u * THREADS, i = idx / (EP / 4), e = (idx % (EP / 4)) * 4;
+      *(float4 *)&vs[i][e] = (i < nr && e < a.E) ? x[u] : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+  } else {
+    stage_heads<DP, CR, KS>(a, nullptr, kp, r0, nr, nullptr, &ks[0][0]);
+    for (int idx = tid; idx < CR * EP; idx += THREADS) {
+      const int i = idx / EP, e = idx % EP;
+      vs[i][e] = (i < nr && e < a.E) ? vp[size_t(r0 + i) * a.row_stride + e] : 0.0f;
+    }
   }
   __syncthreads();
   if (CHANNEL) {
     // a thread a (channel, part of the rows): the sum of the logarithms of the rows after a row, backwards
-    const int d = tid % DP, part = tid / DP;
-    float l[PR], total = 0.0f;
+    const int d = ch;
+    float total = 0.0f;
 #pragma unroll
     for (int i = 0; i < PR; ++i) {
-      const int row = part * PR + i;
-      l[i] = (d < a.D && row < nr) ? fmaxf(a.log_decay[size_t(r0 + row) * a.ld_stride + head * a.D + d], kLeastLog) * kLog2e : 0.0f;
+      l[i] = (d < a.D && part * PR + i < nr) ? fmaxf(l[i], kLeastLog) * kLog2e : 0.0f;
       total += l[i];
     }
     sums[part][d] = total;
@@ -232,34 +297,40 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
   const int r0 = c[0], nr = c[1];
   const float *qp = a.q + size_t(head) * a.D, *kp = a.k + size_t(head) * a.D, *vp = a.v + size_t(head) * a.E;
   if (!CHANNEL) decay_powers(pw, a.decay[head], CR);
-  for (int idx = tid; idx < CR * (DP / 4); idx += THREADS) {
-    const int i = idx / (DP / 4), d = (idx % (DP / 4)) * 4;
-    float4 x = make_float4(0.f, 0.f, 0.f, 0.f), y = x;
-    if (i < nr) {
-      x = load_head4(a, qp + size_t(r0 + i) * a.row_stride, r0 + i, d, a.q_scale);
-      y = load_head4(a, kp + size_t(r0 + i) * a.row_stride, r0 + i, d, a.k_scale);
-    }
-    *(float4 *)&qs[i * QS + d] = x;
-    *(float4 *)&kps[i * QS + d] = y;
+  float l[CHANNEL ? PR : 1];
+  const int ch = tid % DP, part = tid / DP;
+  if (CHANNEL) fetch_logs<PR>(a, l, head, r0, nr, ch, part);
+  stage_heads<DP, CR, QS>(a, qp, kp, r0, nr, qs, kps);
+  // What the second half of the kernel reads from memory is asked for now and arrives while P is made: the wave's
+  // columns of S_in, of the chunk's values and of the gate.
+  const int rsub = RSPLIT > 1 ? wave / (WAVES / RSPLIT) : 0, ew = RSPLIT > 1 ? wave % (WAVES / RSPLIT) : wave;
+  const int t0 = rsub * RT;                                // the wave's first row tile
+  const float *S = a.part + (size_t(blockIdx.y) * a.heads + head) * a.D * a.E;
+  float sv[ET][DP / 4], vv[ET][CR / 4];
+#pragma unroll
+  for (int x = 0; x < ET; ++x) {
+    const int e = min((ew + x * (WAVES / RSPLIT)) * 16 + col, a.E - 1);
+#pragma unroll
+    for (int u = 0; u < DP / 4; ++u) sv[x][u] = S[size_t(min(4 * u + grp, a.D - 1)) * a.E + e];
+#pragma unroll
+    for (int u = 0; u < CR / 4; ++u) vv[x][u] = vp[size_t(r0 + min(4 * u + grp, nr - 1)) * a.row_stride + e];
   }
   if (CHANNEL) {
     // L, times log2(e): a thread a (channel, part of the rows)
-    const int d = tid % DP, part = tid / DP;
-    float l[PR], total = 0.0f;
+    float total = 0.0f;
 #pragma unroll
     for (int i = 0; i < PR; ++i) {
-      const int row = part * PR + i;
-      l[i] = (d < a.D && row < nr) ? fmaxf(a.log_decay[size_t(r0 + row) * a.ld_stride + head * a.D + d], kLeastLog) * kLog2e : 0.0f;
+      l[i] = (ch < a.D && part * PR + i < nr) ? fmaxf(l[i], kLeastLog) * kLog2e : 0.0f;
       total += l[i];
     }
-    sums[part][d] = total;
+    sums[part][ch] = total;
     __syncthreads();
     float before = 0.0f;
-    for (int p = 0; p < part; ++p) before += sums[p][d];
+    for (int p = 0; p < part; ++p) before += sums[p][ch];
 #pragma unroll
     for (int i = 0; i < PR; ++i) {
       before += l[i];
-      ls[(part * PR + i) * QS + d] = before;
+      ls[(part * PR + i) * QS + ch] = before;
     }
   }
   __syncthreads();
@@ -351,36 +422,19 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
   }
   __syncthreads();
   // ---- o = q S_in (scaled) + P v
-  const int rsub = RSPLIT > 1 ? wave / (WAVES / RSPLIT) : 0, ew = RSPLIT > 1 ? wave % (WAVES / RSPLIT) : wave;
-  const int t0 = rsub * RT;                                // the wave's first row tile
-  const float *S = a.part + (size_t(blockIdx.y) * a.heads + head) * a.D * a.E;
   f32x4_t acc[ET][RT];
   bool live[ET];
 #pragma unroll
   for (int x = 0; x < ET; ++x) {
-    const int e0 = (ew + x * (WAVES / RSPLIT)) * 16;
-    live[x] = e0 < a.E;
+    live[x] = (ew + x * (WAVES / RSPLIT)) * 16 < a.E;
 #pragma unroll
     for (int t = 0; t < RT; ++t) acc[x][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     if (!live[x]) continue;
-    const int e = min(e0 + col, a.E - 1);
-    constexpr int AHEAD = 8;
-    float cur[AHEAD];
 #pragma unroll
-    for (int u = 0; u < AHEAD; ++u) cur[u] = S[size_t(min(4 * u + grp, a.D - 1)) * a.E + e];
-    for (int s = 0; s < ksteps; s += AHEAD) {
-      float next[AHEAD];
+    for (int u = 0; u < DP / 4; ++u) {
+      if (u < ksteps)                     // (numbers past the head's last are zeros in the queries)
 #pragma unroll
-      for (int u = 0; u < AHEAD; ++u) next[u] = S[size_t(min(4 * (s + AHEAD + u) + grp, a.D - 1)) * a.E + e];
-#pragma unroll
-      for (int u = 0; u < AHEAD; ++u) {
-        if (s + u >= ksteps) break;
-#pragma unroll
-        for (int t = 0; t < RT; ++t)      // (numbers past the head's last are zeros in the queries)
-          acc[x][t] = mfma_f32(qs[(16 * (t0 + t) + col) * QS + 4 * (s + u) + grp], cur[u], acc[x][t]);
-      }
-#pragma unroll
-      for (int u = 0; u < AHEAD; ++u) cur[u] = next[u];
+        for (int t = 0; t < RT; ++t) acc[x][t] = mfma_f32(qs[(16 * (t0 + t) + col) * QS + 4 * u + grp], sv[x][u], acc[x][t]);
     }
     if (!CHANNEL) {
 #pragma unroll
@@ -390,18 +444,25 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
     }
     // the chunk's own rows: column tile J of P meets rows 16 J .. of v; row tiles before J have none of it
 #pragma unroll
-    for (int J = 0; J < NT; ++J) {
-      float vv[4];
-#pragma unroll
-      for (int s = 0; s < 4; ++s) vv[s] = vp[size_t(r0 + min(16 * J + 4 * s + grp, nr - 1)) * a.row_stride + e];
+    for (int J = 0; J < NT; ++J)
 #pragma unroll
       for (int t = 0; t < RT; ++t) {
         if (t0 + t < J) continue;         // uniform over the wave
 #pragma unroll
         for (int s = 0; s < 4; ++s)
-          acc[x][t] = mfma_f32(ps[(16 * (t0 + t) + col) * PS + 16 * J + 4 * s + grp], vv[s], acc[x][t]);
+          acc[x][t] = mfma_f32(ps[(16 * (t0 + t) + col) * PS + 16 * J + 4 * s + grp], vv[x][4 * J + s], acc[x][t]);
       }
-    }
+  }
+  // the gate's numbers arrive while the norms are worked out
+  float gate[ET][RT][4];
+#pragma unroll
+  for (int x = 0; x < ET; ++x) {
+    const int e = min((ew + x * (WAVES / RSPLIT)) * 16 + col, a.E - 1);
+#pragma unroll
+    for (int t = 0; t < RT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        gate[x][t][r] = a.g[size_t(r0 + min(16 * (t0 + t) + 4 * grp + r, nr - 1)) * a.row_stride + head * a.E + e];
   }
   // ---- the head's norm: a row's squares over the sixteen lanes, then over the waves that share it
 #pragma unroll
@@ -433,10 +494,10 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
       for (int x = 0; x < ET; ++x) {
         const int e = (ew + x * (WAVES / RSPLIT)) * 16 + col;
         if (!live[x] || e >= a.E) continue;
-        const float gate = a.g[size_t(r0 + i) * a.row_stride + head * a.E + e];
+        const float gt = gate[x][t][r];
         float y = acc[x][t][r] * inv;
         if (a.w) y *= ld_dyn(a.w, a.w_dtype, e);
-        y *= gate / (1.0f + expf(-gate));
+        y *= gt / (1.0f + expf(-gt));
         const size_t at = size_t(r0 + i) * a.out_stride + head * a.E + e;
         if (a.out_dtype == SB_F32) ((float *)a.out)[at] = y;
         else ((bf16_t *)a.out)[at] = f32_to_bf16(y);

@@ -3,7 +3,7 @@
 //     S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t,          (S is D x E per head)
 //     out_t = o_t / sqrt(mean(o_t^2) + eps) (* w) * silu(g_t)
 // with alpha either one constant number per head (`decay`) or a number per head and key channel, given by its
-// logarithm (`log_decay` [rows, heads * D]).  q and k are read from float32 rows; with inv_freq the pairs
+// logarithm (`log_decay` [rows, heads * D]) or made here as sb_log_decay makes it from `inner` [rows, rank].  q and k are read from float32 rows; with inv_freq the pairs
 // (i, i + rot_dims / 2) of the first rot_dims numbers of every head turn by position * inv_freq[i]; then they are
 // multiplied by q_scale and k_scale.  The state of sequence s lies in state[slots[s]] and goes from step to step.
 //
@@ -26,10 +26,15 @@ constexpr int MAX_WAVES = 16;
 
 __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
 
+// rate * log(sigmoid(z)) = rate * (min(z, 0) - log(1 + exp(-|z|)))
+__device__ __forceinline__ float log_sigmoid(float z, float rate) { return (fminf(z, 0.0f) - log1pf(expf(-fabsf(z)))) * rate; }
+
 struct DecayArgs {
   void *out; int out_dtype, out_stride;                  // out_t[a * E + e]
   const float *q, *k, *v, *g; int row_stride;            // q_t[a * D + d], k_t[a * D + d], v_t[a * E + e], g_t[a * E + e]
-  const float *log_decay; int ld_stride;                 // [rows, heads * D], or NULL: decay
+  const float *log_decay; int ld_stride;                 // [rows, heads * D], or NULL: inner, or decay
+  const float *inner; int inner_stride;                  // [rows, rank]: log alpha = rate log(sigmoid(inner up + bias))
+  const float *up, *bias; int rank; float rate;          // [rank, heads * D], [heads * D]
   const float *decay;                                    // [heads]
   const float *inv_freq; int rot_dims; const int32_t *row_pos;
   float q_scale, k_scale;
@@ -85,7 +90,19 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
         }
         q *= a.q_scale;
         k *= a.k_scale;
-        if (CHANNEL) al = expf(a.log_decay[size_t(rb + i) * a.ld_stride + head * a.D + d]);
+        if (CHANNEL) {
+          float ld;
+          if (a.log_decay) {
+            ld = a.log_decay[size_t(rb + i) * a.ld_stride + head * a.D + d];
+          } else {
+            const float *in = a.inner + size_t(rb + i) * a.inner_stride, *up = a.up + head * a.D + d;
+            float z = 0.0f;
+#pragma unroll 16
+            for (int j = 0; j < a.rank; ++j) z = fmaf(in[j], up[size_t(j) * a.heads * a.D], z);
+            ld = log_sigmoid(z + a.bias[head * a.D + d], a.rate);
+          }
+          al = expf(ld);
+        }
       }
       qs[i][d] = q;
       ks[i][d] = k;
@@ -174,30 +191,29 @@ constexpr int LD_ROWS = 8;         // rows a block of the log-decay kernel takes
 __global__ void __launch_bounds__(256)
 log_decay_kernel(float *__restrict__ out, int out_stride, const float *__restrict__ a, int a_stride, const float *__restrict__ w,
                  const float *__restrict__ bias, int n_rows, int rank, int width, float rate) {
-  extern __shared__ float as[];    // [LD_ROWS][rank]
+  extern __shared__ __attribute__((aligned(16))) float as[];    // [rank][LD_ROWS]: a number's eight rows in two loads
   const int r0 = blockIdx.y * LD_ROWS, nr = min(LD_ROWS, n_rows - r0), c = blockIdx.x * 256 + threadIdx.x;
-  for (int idx = threadIdx.x; idx < nr * rank; idx += 256) {
+  for (int idx = threadIdx.x; idx < LD_ROWS * rank; idx += 256) {
     const int i = idx / rank, j = idx - i * rank;
-    as[idx] = a[size_t(r0 + i) * a_stride + j];
+    as[j * LD_ROWS + i] = a[size_t(r0 + min(i, nr - 1)) * a_stride + j];
   }
   __syncthreads();
   if (c >= width) return;
   float z[LD_ROWS];
 #pragma unroll
   for (int i = 0; i < LD_ROWS; ++i) z[i] = 0.0f;
-#pragma unroll 4
+#pragma unroll 8
   for (int j = 0; j < rank; ++j) {
     const float wv = w[size_t(j) * width + c];
-#pragma unroll
-    for (int i = 0; i < LD_ROWS; ++i) z[i] = fmaf(as[(i < nr ? i : 0) * rank + j], wv, z[i]);
+    const float4 lo = *(const float4 *)&as[j * LD_ROWS], hi = *(const float4 *)&as[j * LD_ROWS + 4];
+    z[0] = fmaf(lo.x, wv, z[0]); z[1] = fmaf(lo.y, wv, z[1]); z[2] = fmaf(lo.z, wv, z[2]); z[3] = fmaf(lo.w, wv, z[3]);
+    z[4] = fmaf(hi.x, wv, z[4]); z[5] = fmaf(hi.y, wv, z[5]); z[6] = fmaf(hi.z, wv, z[6]); z[7] = fmaf(hi.w, wv, z[7]);
   }
   const float b = bias ? bias[c] : 0.0f;
 #pragma unroll
   for (int i = 0; i < LD_ROWS; ++i)
     if (i < nr) {
-      const float zz = z[i] + b;
-      // log sigmoid(z) = min(z, 0) - log(1 + exp(-|z|))
-      out[size_t(r0 + i) * out_stride + c] = (fminf(zz, 0.0f) - log1pf(expf(-fabsf(zz)))) * rate;
+      out[size_t(r0 + i) * out_stride + c] = log_sigmoid(z[i] + b, rate);
     }
 }
 
@@ -206,11 +222,13 @@ log_decay_kernel(float *__restrict__ out, int out_stride, const float *__restric
 extern "C" int sb_decay_scan_max_side(void) { return MAX_SIDE; }
 
 extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v,
-                             const float *g, int row_stride, const float *log_decay, int ld_stride, const float *decay,
+                             const float *g, int row_stride, const float *log_decay, int ld_stride, const float *inner,
+                             int inner_stride, const float *up, const float *bias, int rank, float rate, const float *decay,
                              const float *inv_freq, int rot_dims, const int32_t *row_pos, float q_scale, float k_scale,
                              const void *w, int w_dtype, float eps, float *state, const int32_t *cu_rows,
                              const int32_t *slots, int n_seqs, int heads, int D, int E, void *stream) {
-  SB_REQUIRE(out && q && k && v && g && state && cu_rows && slots && (log_decay || decay), "sb_decay_scan: null pointer");
+  SB_REQUIRE(out && q && k && v && g && state && cu_rows && slots && (log_decay || inner || decay), "sb_decay_scan: null pointer");
+  SB_REQUIRE(!inner || (up && bias && rank > 0), "sb_decay_scan: decays without their matrix or bias");
   SB_REQUIRE(n_seqs >= 0 && heads > 0 && D > 0 && E > 0 && sb::valid_dtype(out_dtype) && (!w || sb::valid_dtype(w_dtype)),
              "sb_decay_scan: bad sizes heads=%d dim=%d vdim=%d", heads, D, E);
   SB_REQUIRE(!inv_freq || (row_pos && rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= D),
@@ -218,9 +236,10 @@ extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const flo
   SB_SUPPORT(D <= MAX_SIDE && E <= MAX_SIDE, "sb_decay_scan: a state of %d x %d a head is more than %d x %d", D, E, MAX_SIDE, MAX_SIDE);
   SB_SUPPORT(n_seqs <= 65535, "sb_decay_scan: more than 65535 sequences");
   if (n_seqs == 0) return SB_OK;
-  const DecayArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, log_decay, ld_stride, decay, inv_freq, inv_freq ? rot_dims : 0,
+  const DecayArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, log_decay, ld_stride, inner, inner_stride, up, bias,
+                    rank, rate, decay, inv_freq, inv_freq ? rot_dims : 0,
                     row_pos, q_scale, k_scale, w, w_dtype, eps, state, cu_rows, slots, heads, D, E};
-  if (log_decay) launch_walk<true>(a, n_seqs, (hipStream_t)stream);
+  if (log_decay || inner) launch_walk<true>(a, n_seqs, (hipStream_t)stream);
   else launch_walk<false>(a, n_seqs, (hipStream_t)stream);
   return sb::check_launch("sb_decay_scan");
 }

@@ -15,7 +15,7 @@
 namespace {
 
 constexpr int kMaxTerms = 3;
-constexpr int kMaxSlices = 8;
+constexpr int kMaxSlices = 24;         // of all branches together
 enum { THEN_NOTHING = 0, THEN_RMS = 1, THEN_LAYER = 2, THEN_COPY = 3 };
 
 struct Term {
@@ -28,6 +28,8 @@ struct JoinArgs {
   const void *vec; int vec_dtype;
   void *h; int h_dtype, then; const void *hw; int hw_dtype; float h_eps;
   int width;
+  // the branches' slices one after the other (places past the last hold the last again), and where each branch ends
+  const float *slice[kMaxSlices]; int end[kMaxTerms];
 };
 
 template <int THREADS, int N>
@@ -57,36 +59,44 @@ __device__ __forceinline__ void row_norm(const double (&s)[2], int width, int th
   inv = inv_root(var > 0.0 ? var : 0.0, eps);
 }
 
-template <int NT, int THREADS, int KEEP, int SL>      // SL: slices the unrolled loops ask for (>= every branch's)
+template <int NT, int THREADS, int KEEP, int SL>      // SL: slices the unrolled loops ask for (>= those of all branches)
 __global__ void __launch_bounds__(THREADS) join_kernel(JoinArgs a) {
   __shared__ double term_slots[THREADS / 64][NT > 0 ? NT : 1], row_slots[THREADS / 64][2];
   const int r = blockIdx.x, tid = threadIdx.x, n_groups = a.width / 4;
   const size_t from = size_t(a.rows ? a.rows[r] : r) * n_groups, at = size_t(r) * n_groups;
-  float4 in[NT > 0 ? NT : 1][KEEP][SL], base[KEEP];
+  float4 in[KEEP][NT > 0 ? SL : 1], base[KEEP];
 #pragma unroll
   for (int i = 0; i < KEEP; ++i) {
     const int g = min(tid + i * THREADS, n_groups - 1);
+    if (NT > 0)
 #pragma unroll
-    for (int b = 0; b < NT; ++b)
-#pragma unroll
-      for (int s = 0; s < SL; ++s)
-        in[b][i][s] = reinterpret_cast<const float4 *>(a.t[b].part)[size_t(min(s, a.t[b].n_slices - 1)) * (a.t[b].slice_stride / 4) + at + g];
+      for (int s = 0; s < SL; ++s) in[i][s] = reinterpret_cast<const float4 *>(a.slice[s])[at + g];
     base[i] = reinterpret_cast<const float4 *>(a.base)[from + g];
   }
   float4 y[NT > 0 ? NT : 1][KEEP];
   double sq[NT > 0 ? NT : 1];
   bool any_norm = false;
 #pragma unroll
+  for (int b = 0; b < NT; ++b)
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) y[b][i] = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (NT > 0) {
+#pragma unroll
+    for (int s = 0; s < SL; ++s)
+#pragma unroll
+      for (int b = 0; b < NT; ++b)
+        if (s < a.end[b] && (b == 0 || s >= a.end[b > 0 ? b - 1 : 0])) {      // (the same for all lanes)
+#pragma unroll
+          for (int i = 0; i < KEEP; ++i) { y[b][i].x += in[i][s].x; y[b][i].y += in[i][s].y; y[b][i].z += in[i][s].z; y[b][i].w += in[i][s].w; }
+        }
+  }
+#pragma unroll
   for (int b = 0; b < NT; ++b) {
     sq[b] = 0.0;
     any_norm = any_norm || a.t[b].norm;
 #pragma unroll
     for (int i = 0; i < KEEP; ++i) {
-      float4 v = in[b][i][0];
-#pragma unroll
-      for (int s = 1; s < SL; ++s)
-        if (s < a.t[b].n_slices) { v.x += in[b][i][s].x; v.y += in[b][i][s].y; v.z += in[b][i][s].z; v.w += in[b][i][s].w; }
-      y[b][i] = v;
+      const float4 v = y[b][i];
       if (tid + i * THREADS < n_groups)
         sq[b] += double(v.x * v.x) + double(v.y * v.y) + double(v.z * v.z) + double(v.w * v.w);
     }
@@ -209,7 +219,7 @@ __global__ void __launch_bounds__(256) join_any_kernel(JoinArgs a, int n_terms) 
 // the branches' loads of a thread that its registers hold (four numbers each): the rest goes through LDS
 template <int NT, int THREADS, int KEEP, int SL>
 bool launch_keep(const JoinArgs &a, int n_rows, hipStream_t s) {
-  if constexpr (NT * KEEP * SL > (THREADS > 256 ? (KEEP == 1 ? 24 : 14) : 48)) return false;
+  if constexpr (KEEP * SL > (THREADS > 256 ? (KEEP == 1 ? 24 : 14) : 48)) return false;
   else join_kernel<NT, THREADS, KEEP, SL><<<n_rows, THREADS, 0, s>>>(a);
   return true;
 }
@@ -225,34 +235,35 @@ bool launch_sl(const JoinArgs &a, int n_rows, hipStream_t s) {
 
 template <int NT, int THREADS>
 bool launch_threads(const JoinArgs &a, int slices, int n_rows, hipStream_t s) {
-  if (slices <= 1) return launch_sl<NT, THREADS, 1>(a, n_rows, s);
-  if constexpr (NT > 0) {
-    if (slices <= 2) return launch_sl<NT, THREADS, 2>(a, n_rows, s);
-    if (slices <= 4) return launch_sl<NT, THREADS, 4>(a, n_rows, s);
-    return launch_sl<NT, THREADS, 8>(a, n_rows, s);
-  }
-  return false;
+  if constexpr (NT == 0) return launch_sl<NT, THREADS, 1>(a, n_rows, s);
+  if (slices <= NT) return launch_sl<NT, THREADS, NT == 0 ? 1 : NT>(a, n_rows, s);
+  if (slices <= 6) return launch_sl<NT, THREADS, 6>(a, n_rows, s);
+  if (slices <= 12) return launch_sl<NT, THREADS, 12>(a, n_rows, s);
+  if (slices <= 18) return launch_sl<NT, THREADS, 18>(a, n_rows, s);
+  return launch_sl<NT, THREADS, 24>(a, n_rows, s);
 }
 
 template <int NT>
 bool launch_fast(const JoinArgs &a, int slices, int n_rows, bool few, hipStream_t s) {
-  if (few && launch_threads<NT, 1024>(a, slices, n_rows, s)) return true;
-  if (!few && a.width > 4096) {             // wide rows: one shape for all row counts
-    return launch_threads<NT, 1024>(a, slices, n_rows, s);
-  }
-  return launch_threads<NT, 256>(a, slices, n_rows, s);
+  if (few && a.width <= 2048 && launch_threads<NT, 512>(a, slices, n_rows, s)) return true;
+  if ((few || a.width > 4096) && launch_threads<NT, 1024>(a, slices, n_rows, s)) return true;
+  return a.width <= 4096 && launch_threads<NT, 256>(a, slices, n_rows, s);       // (wide rows: one shape for all row counts)
 }
 
-int launch_join(const JoinArgs &a, int n_terms, int n_rows, int few, hipStream_t s, const char *what) {
-  int slices = 1;
+int launch_join(JoinArgs &a, int n_terms, int n_rows, int few, hipStream_t s, const char *what) {
+  int slices = 0;
   bool ok = a.width % 4 == 0;
   const auto aligned = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   ok = ok && aligned(a.base) && aligned(a.out) && aligned(a.h);
   for (int b = 0; b < n_terms; ++b) {
-    slices = a.t[b].n_slices > slices ? a.t[b].n_slices : slices;
+    for (int i = 0; i < a.t[b].n_slices; ++i, ++slices)
+      if (slices < kMaxSlices) a.slice[slices] = a.t[b].part + size_t(i) * a.t[b].slice_stride;
+    a.end[b] = slices;
     ok = ok && aligned(a.t[b].part) && a.t[b].slice_stride % 4 == 0;
   }
   if (ok && slices <= kMaxSlices) {
+    if (slices > 0)
+      for (int i = slices; i < kMaxSlices; ++i) a.slice[i] = a.slice[slices - 1];
     bool done = false;
     const bool f = few && n_rows <= 64;
     if (n_terms == 0) done = launch_fast<0>(a, 1, n_rows, f, s);
@@ -269,8 +280,8 @@ int launch_join(const JoinArgs &a, int n_terms, int n_rows, int few, hipStream_t
 }  // namespace
 
 // n_terms <= 3; term_ptrs: per branch {part, weight or NULL}; term_ints: per branch {slices, weight dtype, norm};
-// slice strides in numbers; base may be out.  few: blocks of 1024 threads a row for up to 64 rows (the order of a
-// row's sums then depends on the number of rows).
+// slice strides in numbers; base may be out.  few: wider blocks for up to 64 rows (the order of a row's sums
+// then depends on the number of rows).
 extern "C" int sb_join(float *out, const float *base, const void *const *term_ptrs, const int *term_ints,
                        const float *term_scales, const size_t *slice_strides, int n_terms, float term_eps, const void *vec,
                        int vec_dtype, void *h, int h_dtype, int then, const void *h_weight, int h_w_dtype, float h_eps,

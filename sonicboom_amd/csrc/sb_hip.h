@@ -533,7 +533,7 @@ int sb_moe_router_grouped(int32_t *ids, float *weights, const void *h, int h_dty
  *   square, term_eps inside the root} each; slice_strides in numbers); then h = what the next block reads:
  *   0 nothing, 1 RMS norm, 2 layer norm, 3 out itself in h_dtype.  base may be out.
  * sb_layernorm: (x - mean) / sqrt(mean((x - mean)^2) + eps) * w of the rows named by `rows` (NULL: all).
- * few != 0: up to 64 rows take blocks of 1024 threads (a row's sums are then ordered otherwise). */
+ * few != 0: up to 64 rows take wider blocks (a row's sums are then ordered otherwise). */
 int sb_join(float *out, const float *base, const void *const *term_ptrs, const int *term_ints, const float *term_scales,
             const size_t *slice_strides, int n_terms, float term_eps, const void *vec, int vec_dtype, void *h, int h_dtype,
             int then, const void *h_weight, int h_w_dtype, float h_eps, int n_rows, int width, int few, void *stream);
@@ -542,8 +542,9 @@ int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dt
 
 /* ---- linear attention with decays (csrc/decay_scan.hip, csrc/decay_chunks.hip) --------------------
  * sb_decay_scan: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t per head (S f32 D x E in
- *   state[slots[s]]), out_t = o_t / rms(o_t) (* w) * silu(g_t); alpha from log_decay f32 [rows, heads * D], or one
- *   number a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
+ *   state[slots[s]]), out_t = o_t / rms(o_t) (* w) * silu(g_t); alpha from log_decay f32 [rows, heads * D], or made
+ *   as sb_log_decay makes it from inner f32 [rows, rank] (up f32 [rank, heads * D], bias f32 [heads * D]), or one number
+ *   a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
  *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart.
  * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width].
  * sb_decay_chunks: the same scan over runs of sb_decay_chunk_rows(D) rows (chunks int32 [n_chunks, 4], sequence after
@@ -552,7 +553,8 @@ int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dt
  *   [n_chunks, heads, D] are scratch. */
 int sb_decay_scan_max_side(void);
 int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
-                  int row_stride, const float *log_decay, int ld_stride, const float *decay, const float *inv_freq,
+                  int row_stride, const float *log_decay, int ld_stride, const float *inner, int inner_stride,
+                  const float *up, const float *bias, int rank, float rate, const float *decay, const float *inv_freq,
                   int rot_dims, const int32_t *row_pos, float q_scale, float k_scale, const void *w, int w_dtype, float eps,
                   float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E,
                   void *stream);

@@ -1956,16 +1956,20 @@ def log_decay(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], ra
     return out
 
 
+_log_decay = log_decay          # (an argument below has the function's name)
+
+
 def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, state: torch.Tensor, ctx, heads: int,
                dim: int, v_dim: int, eps: float, out_dtype: torch.dtype, log_decay: Optional[torch.Tensor] = None,
                decay: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, q_scale: float = 1.0,
                k_scale: float = 1.0, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
-               chunks: Optional[torch.Tensor] = None, angles: Optional[torch.Tensor] = None) -> torch.Tensor:
+               chunks: Optional[torch.Tensor] = None, angles: Optional[torch.Tensor] = None, decay_from=None) -> torch.Tensor:
     """S = alpha S + k v^T, o = S^T q per head over every sequence's rows of the step, from ``state`` float32
     [slots, heads, dim, v_dim], which moves on; returns o / rms(o) (* weight) * silu(g) [n, heads*v_dim] in ``out_dtype``.
 
     ``q``, ``k`` [n, heads*dim], ``v``, ``g`` [n, heads*v_dim]: float32 parts of the same wider rows.  alpha: the
-    exponential of ``log_decay`` float32 [n, heads*dim], or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
+    exponential of ``log_decay`` float32 [n, heads*dim], or of what :func:`log_decay` makes of ``decay_from`` (its
+    arguments: the walk makes it in its own kernel), or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
     pairs (i, i + rot_dims/2) of every head of q and k turn by position * inv_freq[i]; then q and k are multiplied by
     their scales.
 
@@ -1982,10 +1986,25 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     _dev(state, log_decay, decay, weight, inv_freq, ctx.cu_rows, ctx.slots, ctx.row_pos)
     if state.dtype != torch.float32 or tuple(state.shape[1:]) != (heads, dim, v_dim):
         raise KernelLibraryError(f"the state must be float32 [slots, {heads}, {dim}, {v_dim}]")
-    if (log_decay is None) == (decay is None):
-        raise KernelLibraryError("a decaying scan takes the logarithms of its decays, or one decay a head")
+    if sum(t is not None for t in (log_decay, decay, decay_from)) != 1:
+        raise KernelLibraryError("a decaying scan takes the logarithms of its decays, what they are made from, or one decay a head")
+    inner = up = bias = None
+    rank, rate = 0, 0.0
+    if decay_from is not None:
+        if chunks is not None:
+            log_decay = _log_decay(*decay_from)
+        else:
+            inner, up, bias, rate = decay_from
+            _dev(up, bias)
+            rank = up.shape[0]
+            _f32_rows(inner, n, rank, "a decay's inner numbers")
+            if up.dtype != torch.float32 or tuple(up.shape) != (rank, heads * dim):
+                raise KernelLibraryError(f"a decay's matrix must be float32 [{rank}, {heads * dim}]")
+            _f32_vec(bias, heads * dim, "a decay's bias")
     if log_decay is not None:
         _f32_rows(log_decay, n, heads * dim, "logarithms of decays")
+    elif inner is not None:
+        pass
     else:
         _f32_vec(decay, heads, "decays")
     if weight is not None and weight.numel() != v_dim:
@@ -2017,7 +2036,8 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
         return out
     check(library.core().sb_decay_scan(
         _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
-        log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
+        log_decay.stride(0) if log_decay is not None else 0, _p(inner), inner.stride(0) if inner is not None else 0, _p(up),
+        _p(bias), rank, float(rate), _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
         float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
         _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _stream()))
     return out

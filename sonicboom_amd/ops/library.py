@@ -99,7 +99,7 @@ _CORE_SIGNATURES = {
     "sb_join": [_P, _P, _P, _P, _P, _P, _I, _F, _P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P],
     "sb_layernorm": [_P, _I, _P, _P, _I, _P, _I, _I, _F, _I, _P],
     "sb_decay_scan_max_side": [],
-    "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
+    "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _I, _P, _P, _I, _F, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
                       _P],
     "sb_decay_chunk_rows": [_I],
     "sb_angle_table": [_P, _P, _P, _I, _I, _P],

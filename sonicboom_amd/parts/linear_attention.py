@@ -182,9 +182,8 @@ class GatedLinearAttention(_DecayMixer):
         """What the output product reads, from the stacked product's float32 rows (a column range of wider rows is fine)."""
         q, k, v, g = self._cut(rows)
         first = 2 * (self.qk_width + self.v_width)
-        log_decay = ops.log_decay(rows[:, first:first + self.rank], self.decay_up, self.decay_bias, self.rate)
         return ops.decay_scan(q, k, v, g, binding.state, ctx, self.heads, self.head_dim, self.v_dim, self.eps, self.rt.act_dtype,
-                              log_decay=log_decay, weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
+                              decay_from=(rows[:, first:first + self.rank], self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
 
 
 def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float, left_norm: str, right_norm: str,

@@ -500,6 +500,15 @@ def test_logarithms_of_decays(rank, width, rows):
     z = a.numpy()[:, 2:2 + rank].astype(np.float64) @ w.numpy().astype(np.float64) + b.numpy()
     want = np.where(z > 0, -np.log1p(np.exp(-np.abs(z))), z - np.log1p(np.exp(-np.abs(z)))) * 0.125
     assert np.allclose(got.cpu().numpy(), want, rtol=1e-5, atol=1e-6 * rank)
+    if width % 2 == 0:          # the walk makes the same decays in its own kernel
+        heads, D, E = 2, width // 2, 20
+        x = rand(rows, 2 * heads * (D + E), seed=3).to(DEV)
+        views = [x[:, c:c + heads * m] for c, m in ((0, D), (heads * D, D), (2 * heads * D, E), (2 * heads * D + heads * E, E))]
+        outs = []
+        for kw in (dict(log_decay=got), dict(decay_from=(a.to(DEV)[:, 2:2 + rank], w.to(DEV), b.to(DEV), 0.125))):
+            state = torch.ones(1, heads, D, E, device=DEV)
+            outs.append((ops.decay_scan(*views, state, scan_context([rows], [0], [0]), heads, D, E, 1e-5, F32, **kw), state))
+        assert torch.equal(outs[0][0], outs[1][0]) and torch.equal(outs[0][1], outs[1][1])
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
