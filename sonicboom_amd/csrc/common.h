@@ -76,6 +76,27 @@ __device__ __forceinline__ float ld_dyn(const void *p, int dtype, size_t i) {
   return dtype == SB_F32 ? ((const float *)p)[i] : bf16_to_f32(((const bf16_t *)p)[i]);
 }
 
+// The sum over a product's K slices of one number of a row, in ascending order: all loads (of up to eight slices; more: one
+// by one) asked for before any is added.
+constexpr int kSliceLoads = 8;
+__device__ __forceinline__ float sum_slices(const float *p, int n_slices, size_t slice_stride) {
+  if (n_slices == 1) return p[0];
+  if (n_slices == 2) return p[0] + p[slice_stride];
+  if (n_slices <= kSliceLoads) {
+    float in[kSliceLoads];
+#pragma unroll
+    for (int s = 0; s < kSliceLoads; ++s) in[s] = p[size_t(min(s, n_slices - 1)) * slice_stride];
+    float v = 0.0f;
+#pragma unroll
+    for (int s = 0; s < kSliceLoads; ++s)
+      if (s < n_slices) v += in[s];
+    return v;
+  }
+  float v = 0.0f;
+  for (int s = 0; s < n_slices; ++s) v += p[s * slice_stride];
+  return v;
+}
+
 // ---- wave (64 lanes) reductions with a fixed butterfly order -----------------
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -23,15 +23,28 @@ namespace {
 constexpr int RB = 8;              // rows staged in LDS at a time
 constexpr int MAX_SIDE = 256;      // rows and columns of a head's matrix at most
 constexpr int MAX_WAVES = 16;
+constexpr int MAX_RANK = 256;      // inner numbers of a decay that the walk takes
 
 __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
 
-// rate * log(sigmoid(z)) = rate * (min(z, 0) - log(1 + exp(-|z|)))
-__device__ __forceinline__ float log_sigmoid(float z, float rate) { return (fminf(z, 0.0f) - log1pf(expf(-fabsf(z)))) * rate; }
+// rate * log(sigmoid(z)) = rate * (min(z, 0) - log(1 + e)), e = exp(-|z|), by log(1 + e) = 2 artanh(s), s = e / (2 + e)
+// <= 1/3: 2 (s + s^3/3 + s^5/5 + ..), whose terms from s^17 on are below a float32 result's last digit.
+__device__ __forceinline__ float log_sigmoid(float z, float rate) {
+  const float e = expf(-fabsf(z)), s = e / (2.0f + e), s2 = s * s;
+  float p = 1.0f / 15.0f;
+  p = fmaf(p, s2, 1.0f / 13.0f);
+  p = fmaf(p, s2, 1.0f / 11.0f);
+  p = fmaf(p, s2, 1.0f / 9.0f);
+  p = fmaf(p, s2, 1.0f / 7.0f);
+  p = fmaf(p, s2, 1.0f / 5.0f);
+  p = fmaf(p, s2, 1.0f / 3.0f);
+  return (fminf(z, 0.0f) - 2.0f * fmaf(s * s2, p, s)) * rate;
+}
 
 struct DecayArgs {
   void *out; int out_dtype, out_stride;                  // out_t[a * E + e]
   const float *q, *k, *v, *g; int row_stride;            // q_t[a * D + d], k_t[a * D + d], v_t[a * E + e], g_t[a * E + e]
+  int n_slices; size_t slice_stride;                     // (and inner): slices of the rows, added here
   const float *log_decay; int ld_stride;                 // [rows, heads * D], or NULL: inner, or decay
   const float *inner; int inner_stride;                  // [rows, rank]: log alpha = rate log(sigmoid(inner up + bias))
   const float *up, *bias; int rank; float rate;          // [rank, heads * D], [heads * D]
@@ -48,7 +61,7 @@ struct DecayArgs {
 // Column groups of 64 and the rows of S that a wave takes.
 template <int NT, bool CHANNEL>
 __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_groups) {
-  __shared__ __attribute__((aligned(16))) float qs[RB][MAX_SIDE], ks[RB][MAX_SIDE], as[CHANNEL ? RB : 1][CHANNEL ? MAX_SIDE : 4];
+  __shared__ __attribute__((aligned(16))) float qs[RB][MAX_SIDE], ks[RB][MAX_SIDE], as[CHANNEL ? RB : 1][CHANNEL ? MAX_SIDE : 4], ins[CHANNEL ? RB : 1][CHANNEL ? MAX_RANK : 4];
   __shared__ float vs[RB][MAX_SIDE], os[RB][MAX_WAVES * 64];
   const int head = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x, lane = tid & 63, waves = blockDim.x >> 6;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);      // (the same for all lanes: rows of S are tested once a wave)
@@ -70,19 +83,27 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
   for (int rb = r0; rb < r1; rb += RB) {
     const int nr = min(RB, r1 - rb);
     __syncthreads();
+    if (CHANNEL && a.inner) {
+      for (int idx = tid; idx < nr * a.rank; idx += blockDim.x) {
+        const int i = idx / a.rank, j = idx - i * a.rank;
+        ins[i][j] = sum_slices(a.inner + size_t(rb + i) * a.inner_stride + j, a.n_slices, a.slice_stride);
+      }
+      __syncthreads();
+    }
     for (int idx = tid; idx < nr * padded; idx += blockDim.x) {
       const int i = idx / padded, d = idx - i * padded;
       const size_t at = size_t(rb + i) * a.row_stride + head * a.D + d;
-      float q = 0.0f, k = 0.0f, al = 1.0f;
+      float q = 0.0f, k = 0.0f;
       if (d < a.D) {
-        q = a.q[at];
-        k = a.k[at];
+        q = sum_slices(a.q + at, a.n_slices, a.slice_stride);
+        k = sum_slices(a.k + at, a.n_slices, a.slice_stride);
         if (d < 2 * half) {
           const int pair = d < half ? d : d - half, other = d < half ? half : -half;
           const float theta = float(a.row_pos[rb + i]) * a.inv_freq[pair];
           const float c = cosf(theta), s = sinf(theta);
           float y0, y1;
-          const float qo = a.q[at + other], ko = a.k[at + other];
+          const float qo = sum_slices(a.q + at + other, a.n_slices, a.slice_stride);
+          const float ko = sum_slices(a.k + at + other, a.n_slices, a.slice_stride);
           rotate_pair(d < half ? q : qo, d < half ? qo : q, c, s, y0, y1);
           q = d < half ? y0 : y1;
           rotate_pair(d < half ? k : ko, d < half ? ko : k, c, s, y0, y1);
@@ -90,27 +111,34 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
         }
         q *= a.q_scale;
         k *= a.k_scale;
-        if (CHANNEL) {
+      }
+      qs[i][d] = q;
+      ks[i][d] = k;
+    }
+    if (CHANNEL) {
+      // by other waves than those with the first queries and keys, where the block has as many
+      for (int idx = tid >= blockDim.x / 2 ? tid - blockDim.x / 2 : tid + (blockDim.x + 1) / 2; idx < nr * padded; idx += blockDim.x) {
+        const int i = idx / padded, d = idx - i * padded;
+        float al = 1.0f;
+        if (d < a.D) {
           float ld;
           if (a.log_decay) {
             ld = a.log_decay[size_t(rb + i) * a.ld_stride + head * a.D + d];
           } else {
-            const float *in = a.inner + size_t(rb + i) * a.inner_stride, *up = a.up + head * a.D + d;
+            const float *up = a.up + head * a.D + d;
             float z = 0.0f;
-#pragma unroll 16
-            for (int j = 0; j < a.rank; ++j) z = fmaf(in[j], up[size_t(j) * a.heads * a.D], z);
+#pragma unroll 8
+            for (int j = 0; j < a.rank; ++j) z = fmaf(ins[i][j], up[size_t(j) * a.heads * a.D], z);
             ld = log_sigmoid(z + a.bias[head * a.D + d], a.rate);
           }
           al = expf(ld);
         }
+        as[i][d] = al;
       }
-      qs[i][d] = q;
-      ks[i][d] = k;
-      if (CHANNEL) as[i][d] = al;
     }
     for (int idx = tid; idx < nr * a.E; idx += blockDim.x) {
       const int i = idx / a.E, e = idx - i * a.E;
-      vs[i][e] = a.v[size_t(rb + i) * a.row_stride + head * a.E + e];
+      vs[i][e] = sum_slices(a.v + size_t(rb + i) * a.row_stride + head * a.E + e, a.n_slices, a.slice_stride);
     }
     __syncthreads();
 #pragma unroll 1
@@ -132,8 +160,14 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
     __syncthreads();
     // a wave a row: the waves' shares added in ascending order of S's rows, the norm, the gate, the store
     for (int i = wave; i < nr; i += waves) {
-      float o[MAX_SIDE / 64];
+      float o[MAX_SIDE / 64], gate[MAX_SIDE / 64];
       float sq = 0.0f;
+#pragma unroll
+      for (int c = 0; c < MAX_SIDE / 64; ++c)
+        if (c < col_groups) {
+          const float *gp = a.g + size_t(rb + i) * a.row_stride + head * a.E + min(c * 64 + lane, a.E - 1);
+          gate[c] = sum_slices(gp, a.n_slices, a.slice_stride);
+        }
 #pragma unroll
       for (int c = 0; c < MAX_SIDE / 64; ++c) {
         o[c] = 0.0f;
@@ -149,7 +183,7 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
         if (c < col_groups && e < a.E) {
           float y = o[c] * inv;
           if (a.w) y *= ld_dyn(a.w, a.w_dtype, e);
-          y *= silu_f(a.g[size_t(rb + i) * a.row_stride + head * a.E + e]);
+          y *= silu_f(gate[c]);
           const size_t at = size_t(rb + i) * a.out_stride + head * a.E + e;
           if (a.out_dtype == SB_F32) ((float *)a.out)[at] = y;
           else ((bf16_t *)a.out)[at] = f32_to_bf16(y);
@@ -220,15 +254,19 @@ log_decay_kernel(float *__restrict__ out, int out_stride, const float *__restric
 }  // namespace
 
 extern "C" int sb_decay_scan_max_side(void) { return MAX_SIDE; }
+extern "C" int sb_decay_scan_max_rank(void) { return MAX_RANK; }
 
 extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v,
-                             const float *g, int row_stride, const float *log_decay, int ld_stride, const float *inner,
+                             const float *g, int row_stride, int n_slices, size_t slice_stride,
+                             const float *log_decay, int ld_stride, const float *inner,
                              int inner_stride, const float *up, const float *bias, int rank, float rate, const float *decay,
                              const float *inv_freq, int rot_dims, const int32_t *row_pos, float q_scale, float k_scale,
                              const void *w, int w_dtype, float eps, float *state, const int32_t *cu_rows,
                              const int32_t *slots, int n_seqs, int heads, int D, int E, void *stream) {
   SB_REQUIRE(out && q && k && v && g && state && cu_rows && slots && (log_decay || inner || decay), "sb_decay_scan: null pointer");
   SB_REQUIRE(!inner || (up && bias && rank > 0), "sb_decay_scan: decays without their matrix or bias");
+  SB_SUPPORT(!inner || rank <= MAX_RANK, "sb_decay_scan: a rank of %d is more than %d", rank, MAX_RANK);
+  SB_REQUIRE(n_slices >= 1, "sb_decay_scan: at least one slice");
   SB_REQUIRE(n_seqs >= 0 && heads > 0 && D > 0 && E > 0 && sb::valid_dtype(out_dtype) && (!w || sb::valid_dtype(w_dtype)),
              "sb_decay_scan: bad sizes heads=%d dim=%d vdim=%d", heads, D, E);
   SB_REQUIRE(!inv_freq || (row_pos && rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= D),
@@ -236,7 +274,7 @@ extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const flo
   SB_SUPPORT(D <= MAX_SIDE && E <= MAX_SIDE, "sb_decay_scan: a state of %d x %d a head is more than %d x %d", D, E, MAX_SIDE, MAX_SIDE);
   SB_SUPPORT(n_seqs <= 65535, "sb_decay_scan: more than 65535 sequences");
   if (n_seqs == 0) return SB_OK;
-  const DecayArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, log_decay, ld_stride, inner, inner_stride, up, bias,
+  const DecayArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, n_slices, slice_stride, log_decay, ld_stride, inner, inner_stride, up, bias,
                     rank, rate, decay, inv_freq, inv_freq ? rot_dims : 0,
                     row_pos, q_scale, k_scale, w, w_dtype, eps, state, cu_rows, slots, heads, D, E};
   if (log_decay || inner) launch_walk<true>(a, n_seqs, (hipStream_t)stream);

@@ -9,6 +9,7 @@
 //   divided without a weight);
 //   v <- (1 - lam) v + lam v_first when v_first is given (lam one number in memory), and the v of
 //   before the mixing is written to v_out when that is given (the first mixing layer's);
+//   with gate_out the gate_n numbers behind the values are added up over the slices and written there;
 //   q goes out in the activation type, k and v into the page of the row's position.
 // One block a row; a wave a head at a time.
 #include "common.h"
@@ -26,6 +27,7 @@ struct Args {
   void *k_cache, *v_cache;
   int heads_q, heads_kv, dk, dv, store;
   const float *inv_freq; int rot_dims; int unit;
+  float *gate_out; int gate_n;      // the row's numbers behind the values, slices added: [rows, gate_n] (or NULL)
 };
 
 // cosines and sines of the row's position, once per block
@@ -48,26 +50,6 @@ __device__ __forceinline__ float turned(float v, float other, int d, int half, c
   if (d < half) rotate_pair(v, other, cs[i], sn[i], y0, y1);
   else rotate_pair(other, v, cs[i], sn[i], y0, y1);
   return d < half ? y0 : y1;
-}
-
-constexpr int kMaxSlices = 8;      // slices whose loads the unrolled loops ask for together (more: the plain loop)
-
-// the sum over the slices of one number of a row: all loads asked for before any is added
-__device__ __forceinline__ float sum_slices(const float *p, int n_slices, size_t slice_stride) {
-  if (n_slices == 1) return p[0];
-  if (n_slices <= kMaxSlices) {
-    float in[kMaxSlices];
-#pragma unroll
-    for (int s = 0; s < kMaxSlices; ++s) in[s] = p[size_t(min(s, n_slices - 1)) * slice_stride];
-    float v = 0.0f;
-#pragma unroll
-    for (int s = 0; s < kMaxSlices; ++s)
-      if (s < n_slices) v += in[s];
-    return v;
-  }
-  float v = 0.0f;
-  for (int s = 0; s < n_slices; ++s) v += p[s * slice_stride];
-  return v;
 }
 
 template <typename TQ, typename TC, int THREADS>
@@ -118,6 +100,9 @@ __global__ void __launch_bounds__(THREADS) headnorm_kv_store_kernel(Args a) {
   if (!a.store) return;
   const int v0 = (a.heads_q + a.heads_kv) * a.dk, nv = a.heads_kv * a.dv;
   const float lam = a.v_first ? ld_dyn(a.lam, a.lam_dtype, 0) : 0.0f;
+  if (a.gate_out)
+    for (int e = threadIdx.x; e < a.gate_n; e += THREADS)
+      a.gate_out[size_t(row) * a.gate_n + e] = sum_slices(src + v0 + nv + e, a.n_slices, a.slice_stride);
   for (int e = threadIdx.x; e < nv; e += THREADS) {
     float v = sum_slices(src + v0 + e, a.n_slices, a.slice_stride);
     if (a.v_out) a.v_out[size_t(row) * nv + e] = v;
@@ -204,7 +189,9 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
                                     const int32_t *row_seq, void *k_cache, void *v_cache, int cache_dtype,
                                     const int32_t *page_table, int max_pages, int n_pages, int n_rows, int heads_q,
                                     int heads_kv, int dk, int dv, int store, const float *inv_freq, int rot_dims, int unit,
-                                    void *stream) {
+                                    float *gate_out, int gate_n, void *stream) {
+  SB_REQUIRE(!gate_out || (store && gate_n > 0 && row_stride >= heads_q * dk + heads_kv * (dk + dv) + gate_n),
+             "sb_headnorm_kv_store: rows of %d hold no gate of %d behind the values", row_stride, gate_n);
   SB_REQUIRE(!inv_freq || (row_pos && rot_dims > 0 && rot_dims % 2 == 0 && rot_dims <= dk),
              "sb_headnorm_kv_store: rotary width %d must be even and at most the head's %d", rot_dims, dk);
   SB_REQUIRE(q_out && qkv, "sb_headnorm_kv_store: null pointer");
@@ -220,7 +207,7 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
   if (n_rows == 0) return SB_OK;
   const Args a{q_out, qkv, row_stride, n_slices, size_t(n_rows) * row_stride, q_w, k_w, w_dtype, eps, v_first, lam, lam_dtype, v_out,
                row_pos, row_seq, page_table, max_pages, n_pages, k_cache, v_cache, heads_q, heads_kv, dk, dv, store ? 1 : 0,
-               inv_freq, inv_freq ? rot_dims : 0, unit};
+               inv_freq, inv_freq ? rot_dims : 0, unit, gate_out, gate_n};
   hipStream_t s = (hipStream_t)stream;
   const bool qf = q_dtype == SB_F32, cf = !store || cache_dtype == SB_F32;
   // (a wave a head: the sums do not depend on the block's size, so few rows may take more waves a row)
@@ -228,7 +215,7 @@ extern "C" int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, 
   else if (qf) headnorm_kv_store_kernel<float, bf16_t, 256><<<n_rows, 256, 0, s>>>(a);
   else if (cf && store) headnorm_kv_store_kernel<bf16_t, float, 256><<<n_rows, 256, 0, s>>>(a);
   else if (n_rows <= 64) headnorm_kv_store_kernel<bf16_t, bf16_t, 1024><<<n_rows, 1024, 0, s>>>(a);
-  else if (n_rows >= 512 && n_slices == 1 && dk % 8 == 0 && (!inv_freq || rot_dims % 16 == 0) && row_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(qkv) & 15) == 0 &&
+  else if (n_rows >= 512 && n_slices == 1 && !gate_out && dk % 8 == 0 && (!inv_freq || rot_dims % 16 == 0) && row_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(qkv) & 15) == 0 &&
            (reinterpret_cast<uintptr_t>(q_out) & 15) == 0 && (!store || (reinterpret_cast<uintptr_t>(k_cache) & 15) == 0)) {
     if (dk <= 64) headnorm_kv_store_wide_kernel<8><<<n_rows, 256, 0, s>>>(a);
     else if (dk <= 128) headnorm_kv_store_wide_kernel<16><<<n_rows, 256, 0, s>>>(a);

@@ -257,13 +257,15 @@ int sb_scale(float *x, float scale, size_t n, void *stream);
  * added in ascending order; with inv_freq the pairs (i, i + rot_dims / 2) of every head of q and k turn by
  * position * inv_freq[i]; every head of q and k is then divided by its root mean square (eps inside the root)
  * times q_w / k_w [dk] (NULL: as it is, or with `unit` divided without a weight); v <- (1 - lam) v + lam v_first when v_first is given; the v of
- * before the mixing to v_out when that is given; q out in q_dtype, k and v (store != 0) into the pages. */
+ * before the mixing to v_out when that is given; the gate_n numbers behind the values, slices added, to gate_out
+ * when that is given; q out in q_dtype, k and v (store != 0) into the pages. */
 int sb_headnorm_kv_store(void *q_out, int q_dtype, const float *qkv, int row_stride, int n_slices,
                          const void *q_w, const void *k_w, int w_dtype, float eps, const float *v_first,
                          const void *lam, int lam_dtype, float *v_out, const int32_t *row_pos,
                          const int32_t *row_seq, void *k_cache, void *v_cache, int cache_dtype,
                          const int32_t *page_table, int max_pages, int n_pages, int n_rows, int heads_q,
-                         int heads_kv, int dk, int dv, int store, const float *inv_freq, int rot_dims, int unit, void *stream);
+                         int heads_kv, int dk, int dv, int store, const float *inv_freq, int rot_dims, int unit,
+                         float *gate_out, int gate_n, void *stream);
 
 /* sb_attention with values of v_dim numbers a head (cache values [page][kv head][v_dim][position], out
  * [rows, heads_q * v_dim]), scores capped as softcap * tanh(s / softcap) when softcap > 0, and with `sink`
@@ -545,15 +547,17 @@ int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dt
  *   state[slots[s]]), out_t = o_t / rms(o_t) (* w) * silu(g_t); alpha from log_decay f32 [rows, heads * D], or made
  *   as sb_log_decay makes it from inner f32 [rows, rank] (up f32 [rank, heads * D], bias f32 [heads * D]), or one number
  *   a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
- *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart.
+ *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart (inner: inner_stride),
+ *   in n_slices slices slice_stride numbers apart that are added here in ascending order.
  * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width].
  * sb_decay_chunks: the same scan over runs of sb_decay_chunk_rows(D) rows (chunks int32 [n_chunks, 4], sequence after
  *   sequence, each sequence's runs full but its last) on the matrix cores in float32; q and k turn by `angles` f32
  *   [n_rows, half, 2] (sb_angle_table; NULL: not); part f32 [n_chunks, heads, D, E] and, with log_decay, part_decay f32
  *   [n_chunks, heads, D] are scratch. */
 int sb_decay_scan_max_side(void);
+int sb_decay_scan_max_rank(void);      /* of inner */
 int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
-                  int row_stride, const float *log_decay, int ld_stride, const float *inner, int inner_stride,
+                  int row_stride, int n_slices, size_t slice_stride, const float *log_decay, int ld_stride, const float *inner, int inner_stride,
                   const float *up, const float *bias, int rank, float rate, const float *decay, const float *inv_freq,
                   int rot_dims, const int32_t *row_pos, float q_scale, float k_scale, const void *w, int w_dtype, float eps,
                   float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E,

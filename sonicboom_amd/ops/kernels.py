@@ -1233,7 +1233,7 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
                       heads_q: int, heads_kv: int, head_dim: int, v_dim: int, store: bool = True,
                       v_first: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None,
                       v_out: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
-                      unit: bool = False) -> torch.Tensor:
+                      unit: bool = False, gate_n: int = 0):
     """From float32 rows [n, heads_q*head_dim + heads_kv*(head_dim + v_dim)] of a stacked product (or
     [slices, n, ...], added here): with ``inv_freq`` the pairs (i, i + rot_dims/2) of every head of q and k
     turned by position * inv_freq[i]; then every head of q and k divided by its root mean square and
@@ -1241,23 +1241,21 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
     weight), the values mixed as
     (1 - lam) v + lam v_first when ``v_first`` (float32 [n, heads_kv*v_dim]) is given, the values of
     before the mixing written to ``v_out``; returns q [n, heads_q*head_dim] in ``q_dtype`` and, with
-    ``store``, puts keys and values into the pages of the rows' positions."""
+    ``store``, puts keys and values into the pages of the rows' positions.  ``gate_n``: returns (q, the ``gate_n`` numbers
+    behind the values, slices added, float32 [n, gate_n])."""
     _dev(q_weight, k_weight, row_pos, row_seq, k_cache, v_cache, page_table, v_first, lam, v_out)
     if qkv.dtype != torch.float32:
         raise KernelLibraryError("the stacked product must be float32")
-    n_slices = 1
-    if qkv.dim() == 3:
-        _dev(qkv)
-        n_slices = qkv.shape[0]
-        qkv = qkv.view(-1, qkv.shape[2])
     _on_gpu(qkv)
-    if qkv.dim() != 2 or qkv.stride(1) != 1:            # (a column range of wider rows is fine)
+    if qkv.dim() not in (2, 3) or qkv.stride(-1) != 1:            # (a column range of wider rows is fine)
         raise KernelLibraryError("rows of the stacked product must be contiguous")
-    row_stride = qkv.stride(0) if qkv.shape[0] > 1 else qkv.shape[1]
-    n = qkv.shape[0] // n_slices
-    need = heads_q * head_dim + (heads_kv * (head_dim + v_dim) if store else 0)
-    if qkv.dim() != 2 or qkv.shape[1] < need:
-        raise KernelLibraryError(f"rows of the stacked product have {qkv.shape[1]} elements, {need} are needed")
+    n_slices, n = (qkv.shape[0] if qkv.dim() == 3 else 1), qkv.shape[-2]
+    row_stride = qkv.stride(-2)
+    if n_slices > 1 and qkv.stride(0) != n * row_stride:
+        raise KernelLibraryError("the slices of the stacked product must follow each other")
+    need = heads_q * head_dim + (heads_kv * (head_dim + v_dim) if store else 0) + gate_n
+    if qkv.shape[-1] < need:
+        raise KernelLibraryError(f"rows of the stacked product have {qkv.shape[-1]} elements, {need} are needed")
     for w in (q_weight, k_weight):
         if w is not None and w.numel() != head_dim:
             raise KernelLibraryError(f"a head norm's weight has {w.numel()} elements, a head has {head_dim}")
@@ -1282,13 +1280,14 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
         if not store:
             _i32(row_pos, n, "row positions")
     q = torch.empty((n, heads_q * head_dim), dtype=q_dtype, device=qkv.device)
+    gate = torch.empty((n, gate_n), dtype=torch.float32, device=qkv.device) if gate_n else None
     check(library.core().sb_headnorm_kv_store(
         _p(q), _dt(q), _p(qkv), row_stride, n_slices, _p(q_weight), _p(k_weight), _dt(wt) if wt is not None else 0,
         float(eps), _p(v_first), _p(lam) if v_first is not None else None, _dt(lam) if lam is not None else 0, _p(v_out),
         _p(row_pos), _p(row_seq), _p(k_cache), _p(v_cache), _dt(k_cache) if store else 0, _p(page_table), max_pages,
         n_pages, n, heads_q, heads_kv, head_dim, v_dim, 1 if store else 0, _p(inv_freq), int(rot_dims), 1 if unit else 0,
-        _stream()))
-    return q
+        _p(gate), gate_n, _stream()))
+    return q if gate is None else (q, gate)
 
 
 def attention_capped_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, page_table: torch.Tensor,
@@ -1926,6 +1925,11 @@ def decay_scan_max_side() -> int:
     return int(library.core().sb_decay_scan_max_side())
 
 
+def decay_scan_max_rank() -> int:
+    """Inner numbers of a channel's decay that the walk takes at most."""
+    return int(library.core().sb_decay_scan_max_rank())
+
+
 def decay_chunk_rows(dim: int) -> int:
     """The rows of a chunk of the chunked form of :func:`decay_scan` for heads of ``dim`` key channels."""
     return int(library.core().sb_decay_chunk_rows(int(dim)))
@@ -1967,7 +1971,8 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     """S = alpha S + k v^T, o = S^T q per head over every sequence's rows of the step, from ``state`` float32
     [slots, heads, dim, v_dim], which moves on; returns o / rms(o) (* weight) * silu(g) [n, heads*v_dim] in ``out_dtype``.
 
-    ``q``, ``k`` [n, heads*dim], ``v``, ``g`` [n, heads*v_dim]: float32 parts of the same wider rows.  alpha: the
+    ``q``, ``k`` [n, heads*dim], ``v``, ``g`` [n, heads*v_dim]: float32 parts of the same wider rows, or [slices, n, ...]
+    parts of the same K slices, which the walk adds.  alpha: the
     exponential of ``log_decay`` float32 [n, heads*dim], or of what :func:`log_decay` makes of ``decay_from`` (its
     arguments: the walk makes it in its own kernel), or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
     pairs (i, i + rot_dims/2) of every head of q and k turn by position * inv_freq[i]; then q and k are multiplied by
@@ -1976,13 +1981,19 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     ``chunks`` int32 [n, 4]: the step's rows in runs of :func:`decay_chunk_rows` rows; the scan then takes its chunked form
     (float32 throughout; it orders its sums otherwise than the walk, from which it differs by rounding), and turns by
     ``angles``, the step's :func:`angle_table`."""
-    n = q.shape[0]
-    _on_gpu(q, k, v, g)
+    n = q.shape[-2]
+    row_stride, n_slices, slice_stride = q.stride(-2), (q.shape[0] if q.dim() == 3 else 1), (q.stride(0) if q.dim() == 3 else 0)
+    if n_slices > 1 and chunks is not None:
+        raise KernelLibraryError("the chunked scan takes whole rows")
+
+    def part_of_rows(t, width, what):
+        for one in (t[0], t[-1]) if t.dim() == 3 else (t,):
+            _f32_rows(one, n, width, what)
+        if t.dim() != q.dim() or (n > 1 and t.stride(-2) != row_stride) or (n_slices > 1 and (t.shape[0] != n_slices or t.stride(0) != slice_stride)):
+            raise KernelLibraryError("queries, keys, values, gates and a decay's inner numbers must be parts of the same rows")
     for t, width, what in ((q, heads * dim, "queries"), (k, heads * dim, "keys"), (v, heads * v_dim, "values"),
                            (g, heads * v_dim, "gates")):
-        _f32_rows(t, n, width, what)
-        if n > 1 and t.stride(0) != q.stride(0):
-            raise KernelLibraryError("queries, keys, values and gates must be parts of the same rows")
+        part_of_rows(t, width, what)
     _dev(state, log_decay, decay, weight, inv_freq, ctx.cu_rows, ctx.slots, ctx.row_pos)
     if state.dtype != torch.float32 or tuple(state.shape[1:]) != (heads, dim, v_dim):
         raise KernelLibraryError(f"the state must be float32 [slots, {heads}, {dim}, {v_dim}]")
@@ -1991,21 +2002,24 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     inner = up = bias = None
     rank, rate = 0, 0.0
     if decay_from is not None:
-        if chunks is not None:
-            log_decay = _log_decay(*decay_from)
+        inner, up, bias, rate = decay_from
+        rank = up.shape[0]
+        if chunks is not None or rank > decay_scan_max_rank():
+            log_decay, inner = _log_decay(inner, up, bias, rate), None
         else:
-            inner, up, bias, rate = decay_from
             _dev(up, bias)
-            rank = up.shape[0]
-            _f32_rows(inner, n, rank, "a decay's inner numbers")
+            if inner.dim() == 3:
+                part_of_rows(inner, rank, "a decay's inner numbers")
+            else:
+                _f32_rows(inner, n, rank, "a decay's inner numbers")
+                if n_slices > 1:
+                    raise KernelLibraryError("a decay's inner numbers must come in the rows' slices")
             if up.dtype != torch.float32 or tuple(up.shape) != (rank, heads * dim):
                 raise KernelLibraryError(f"a decay's matrix must be float32 [{rank}, {heads * dim}]")
             _f32_vec(bias, heads * dim, "a decay's bias")
     if log_decay is not None:
         _f32_rows(log_decay, n, heads * dim, "logarithms of decays")
-    elif inner is not None:
-        pass
-    else:
+    elif inner is None:
         _f32_vec(decay, heads, "decays")
     if weight is not None and weight.numel() != v_dim:
         raise KernelLibraryError(f"the heads' norm has {weight.numel()} weights, a head has {v_dim}")
@@ -2028,16 +2042,16 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
         if log_decay is not None:
             part_decay = torch.empty((n_chunks, heads, dim), dtype=torch.float32, device=q.device)
         check(library.core().sb_decay_chunks(
-            _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
+            _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), row_stride, _p(log_decay),
             log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(angles), rot_dims // 2 if angles is not None else 0,
             float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
             _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _p(chunks), n_chunks, decay_chunk_rows(dim), _p(part),
             _p(part_decay), _stream()))
         return out
     check(library.core().sb_decay_scan(
-        _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), q.stride(0), _p(log_decay),
-        log_decay.stride(0) if log_decay is not None else 0, _p(inner), inner.stride(0) if inner is not None else 0, _p(up),
-        _p(bias), rank, float(rate), _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
+        _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), row_stride, n_slices, slice_stride, _p(log_decay),
+        log_decay.stride(0) if log_decay is not None else 0, _p(inner), inner.stride(-2) if inner is not None else 0,
+        _p(up) if inner is not None else None, _p(bias) if inner is not None else None, rank, float(rate), _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
         float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
         _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _stream()))
     return out

@@ -57,7 +57,7 @@ _CORE_SIGNATURES = {
     "sb_scale": [_P, _F, _Z, _P],
     "sb_embed_pos_norm": [_P, _P, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P, _I, _I, _F, _F, _I, _P],
     "sb_headnorm_kv_store": [_P, _I, _P, _I, _I, _P, _P, _I, _F, _P, _P, _I, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I,
-                             _I, _I, _I, _I, _I, _P, _I, _I, _P],
+                             _I, _I, _I, _I, _I, _P, _I, _I, _P, _I, _P],
     "sb_attention_capped": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P],
     "sb_moe_max_top": [],
     "sb_moe_route": [_P, _P, _P, _I, _I, _I, _I, _I, _P],
@@ -99,7 +99,8 @@ _CORE_SIGNATURES = {
     "sb_join": [_P, _P, _P, _P, _P, _P, _I, _F, _P, _I, _P, _I, _I, _P, _I, _F, _I, _I, _I, _P],
     "sb_layernorm": [_P, _I, _P, _P, _I, _P, _I, _I, _F, _I, _P],
     "sb_decay_scan_max_side": [],
-    "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _I, _P, _P, _I, _F, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
+    "sb_decay_scan_max_rank": [],
+    "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _I, _Z, _P, _I, _P, _I, _P, _P, _I, _F, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
                       _P],
     "sb_decay_chunk_rows": [_I],
     "sb_angle_table": [_P, _P, _P, _I, _I, _P],

@@ -201,10 +201,15 @@ class Attention(Mixer):
 
     def from_rows(self, rows, ctx, binding):
         """The heads' results (what the output product reads) from the stacked input product's float32 rows
-        [rows, q | k | v (| gate)], whole, or a column range of wider rows."""
+        [rows, q | k | v (| gate)], a column range of wider rows, or, where takes_slices() says so, [slices, rows, ...]
+        K slices of them."""
         if not self.head_norm_path:
             return self._attend_rotating(None, ctx, binding, rows)
         return self._attend_extended(None, ctx, binding, rows)
+
+    def takes_slices(self, ctx) -> bool:
+        """Whether from_rows() adds a product's K slices itself."""
+        return self.head_norm_path
 
     def produce(self, h, ctx, binding):
         """attention(h) in float32 (whole, or in K slices of the output product), for a block that
@@ -253,7 +258,7 @@ class Attention(Mixer):
         qkv = rows
         if rows is None:
             proj = self.qkv if writes else self._q_only
-            qkv = None if self.out_gate else proj.partial(h)
+            qkv = proj.partial(h)
             if qkv is None:
                 qkv = proj(h, torch.float32)
         v_first = v_out = None
@@ -268,12 +273,18 @@ class Attention(Mixer):
                     raise RuntimeError(f"no earlier layer of this step has left its values under {self.value_mix_key!r}")
         page_table = ctx.page_table(binding.group)
         inv_freq, _, rot_dims = self.position.rotary_tables()
+        # (the gate's columns: read where they lie in whole rows; from K slices the storing kernel adds them up)
+        sliced_gate = self.gate_width if self.out_gate and qkv.dim() == 3 else 0
         q = ops.headnorm_kv_store(qkv, rt.act_dtype, self.q_norm, self.k_norm, self.qk_norm_eps, ctx.row_pos, ctx.row_seq,
                                   binding.k_cache, binding.v_cache, page_table, self.heads_q, self.heads_kv,
                                   self.head_dim, self.v_dim, store=writes, v_first=v_first, lam=self.lam, v_out=v_out,
                                   inv_freq=inv_freq, rot_dims=rot_dims if inv_freq is not None else 0,
-                                  unit=self.qk_norm and self.q_norm is None)
-        gate = qkv[:, self.g_off:self.g_off + self.gate_width] if self.out_gate else None
+                                  unit=self.qk_norm and self.q_norm is None, gate_n=sliced_gate)
+        gate = None
+        if sliced_gate:
+            q, gate = q
+        elif self.out_gate:
+            gate = qkv[:, self.g_off:self.g_off + self.gate_width]
         return ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
                                     self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
                                     fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate)

@@ -21,7 +21,7 @@ it differs from the walk by rounding); the 32-bit path always walks.
 the model's width with a weight of its own.  Their input matrices are stacked into one product; the pass that joins
 the block's branches norms both results.  At most one of the two keeps keys and values; states of both are kept
 under "left." and "right.".  Any two mixers that can take their stacked product's rows (``given_input``,
-``input_weight``, ``from_rows``) fit.
+``input_weight``, ``takes_slices``, ``from_rows``) fit.
 """
 from __future__ import annotations
 
@@ -110,20 +110,29 @@ class _DecayMixer(Mixer):
 
     def _cut(self, rows):
         qk, vw = self.qk_width, self.v_width
-        return rows[:, :qk], rows[:, qk:2 * qk], rows[:, 2 * qk:2 * qk + vw], rows[:, 2 * qk + vw:2 * (qk + vw)]
+        return rows[..., :qk], rows[..., qk:2 * qk], rows[..., 2 * qk:2 * qk + vw], rows[..., 2 * qk + vw:2 * (qk + vw)]
+
+    def takes_slices(self, ctx) -> bool:
+        """Whether from_rows() adds a product's K slices itself (the walk does)."""
+        return self._chunks(ctx) is None
+
+    def _rows(self, h, ctx):
+        """The stacked product: in K slices where a kernel cuts K over the grid and the scan adds them, else whole."""
+        part = self.inp.partial(h) if self.takes_slices(ctx) else None
+        return part if part is not None else self.inp(h, torch.float32)
 
     def from_rows(self, rows, ctx, binding):
         raise NotImplementedError
 
     def forward(self, h, x, ctx, binding, then_norm=None):
-        y = self.from_rows(self.inp(h, torch.float32), ctx, binding)
+        y = self.from_rows(self._rows(h, ctx), ctx, binding)
         return self.out.add_into(y, x, then_norm, self.rt.act_dtype, scale=self.out_scale)
 
     def produce(self, h, ctx, binding):
         """The mixer's result in float32 (whole, or in K slices), for a block that adds it up itself."""
         if self.out_scale != 1.0:
             raise ValueError("a mixer that hands its result over has no multiplier of its own")
-        return self.out.raw(self.from_rows(self.inp(h, torch.float32), ctx, binding))
+        return self.out.raw(self.from_rows(self._rows(h, ctx), ctx, binding))
 
 
 @register_part("mixer", "retention")
@@ -150,7 +159,8 @@ class Retention(_DecayMixer):
         return shared[self.turns]
 
     def from_rows(self, rows, ctx, binding):
-        """What the output product reads, from the stacked product's float32 rows (a column range of wider rows is fine)."""
+        """What the output product reads, from the stacked product's float32 rows (a column range of wider rows, or K
+        slices of them)."""
         q, k, v, g = self._cut(rows)
         chunks = self._chunks(ctx)
         angles = self._angles(ctx) if chunks is not None and self.turns is not None else None
@@ -179,11 +189,12 @@ class GatedLinearAttention(_DecayMixer):
         return [tensors["decay_down"]]
 
     def from_rows(self, rows, ctx, binding):
-        """What the output product reads, from the stacked product's float32 rows (a column range of wider rows is fine)."""
+        """What the output product reads, from the stacked product's float32 rows (a column range of wider rows, or K
+        slices of them)."""
         q, k, v, g = self._cut(rows)
         first = 2 * (self.qk_width + self.v_width)
         return ops.decay_scan(q, k, v, g, binding.state, ctx, self.heads, self.head_dim, self.v_dim, self.eps, self.rt.act_dtype,
-                              decay_from=(rows[:, first:first + self.rank], self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
+                              decay_from=(rows[..., first:first + self.rank], self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
 
 
 def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float, left_norm: str, right_norm: str,
@@ -238,8 +249,10 @@ class SideBySide(Mixer):
 
     def produce(self, h, ctx, binding):
         """Both results, each with its norm, for the pass that joins a block's branches."""
-        rows = self.inp(h, torch.float32)
-        cut = (rows[:, :self.split], rows[:, self.split:])
+        rows = self.inp.partial(h) if all(m.takes_slices(ctx) for _, m in self.sides) else None
+        if rows is None:
+            rows = self.inp(h, torch.float32)
+        cut = (rows[..., :self.split], rows[..., self.split:])
         out = []
         for (name, m), part, norm in zip(self.sides, cut, self.norms):
             y = m.out.raw(m.from_rows(part, ctx, self._binding(name, binding)))

@@ -788,3 +788,38 @@ def test_a_block_whose_branches_do_not_hand_their_results_over(dtype):
     got = x.to(DEV)
     block.forward(got, SimpleNamespace(trace=None), None)
     part_close(got, x.numpy() + 3.5 * P.layer_norm(x.numpy(), ref["n"], 1e-4), dtype, "the block", bf16=1e-2)
+
+
+@pytest.mark.parametrize("slices", [1, 3, 9])
+def test_a_products_slices_are_added_where_they_are_read(slices):
+    """The rows of the stacked product in K slices, handed to the storing kernel and to the walk, give the bits of the rows
+    added up before."""
+    from sonicboom_amd import ops
+    heads, kv, dim, vdim, rows = 4, 2, 32, 16, 9
+    width = heads * dim + kv * (dim + vdim) + heads
+    parts = rand(slices, rows, width + 12).to(DEV)
+    whole = parts[0].clone()
+    for s in range(1, slices):
+        whole += parts[s]
+    t = lambda a: torch.tensor(np.asarray(a), dtype=torch.int32, device=DEV)
+    outs = []
+    for src in (parts[..., 4:4 + width], whole[:, 4:4 + width]):
+        kc, vc = torch.zeros(1, kv, 64, dim, device=DEV), torch.zeros(1, kv, vdim, 64, device=DEV)
+        inv = torch.tensor([0.5 ** i for i in range(8)], device=DEV)
+        q, gate = ops.headnorm_kv_store(src, F32, None, None, 1e-3, t(np.arange(rows)), t(np.zeros(rows)), kc, vc, t([[0]]), heads, kv, dim, vdim,
+                                        inv_freq=inv, rot_dims=16, unit=True, gate_n=heads)
+        outs.append((q, gate, kc, vc))
+    assert all(torch.equal(a, b) for a, b in zip(*outs))
+    assert torch.equal(outs[0][1], whole[:, 4 + width - heads:4 + width])
+    H, D, E, rank = 2, 20, 36, 5
+    parts = rand(slices, rows, 2 * H * (D + E) + rank + 3, seed=2).to(DEV)
+    whole = parts[0].clone()
+    for s in range(1, slices):
+        whole += parts[s]
+    up, bias = rand(rank, H * D).to(DEV), rand(H * D, seed=1).to(DEV)
+    outs = []
+    for src in (parts[..., 3:], whole[:, 3:]):
+        cut = [src[..., c:c + n] for c, n in ((0, H * D), (H * D, H * D), (2 * H * D, H * E), (2 * H * D + H * E, H * E), (2 * H * (D + E), rank))]
+        state = torch.zeros(1, H, D, E, device=DEV)
+        outs.append((ops.decay_scan(*cut[:4], state, scan_context([rows], [0], [5]), H, D, E, 1e-5, F32, decay_from=(cut[4], up, bias, 0.25)), state))
+    assert torch.equal(outs[0][0], outs[1][0]) and torch.equal(outs[0][1], outs[1][1])
