@@ -480,16 +480,20 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
       if (col == 0) sq[16 * (t0 + t) + 4 * grp + r][ew] = s2;
     }
   __syncthreads();
+  if (tid < CR) {                         // a thread a row: one root for all its lanes
+    float s2 = 0.0f;
+#pragma unroll
+    for (int y = 0; y < WAVES / RSPLIT; ++y) s2 += sq[tid][y];
+    sq[tid][WAVES] = 1.0f / sqrtf(s2 / float(a.E) + a.eps);
+  }
+  __syncthreads();
 #pragma unroll
   for (int t = 0; t < RT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = 16 * (t0 + t) + 4 * grp + r;
       if (i >= nr) continue;
-      float s2 = 0.0f;
-#pragma unroll
-      for (int y = 0; y < WAVES / RSPLIT; ++y) s2 += sq[i][y];
-      const float inv = 1.0f / sqrtf(s2 / float(a.E) + a.eps);
+      const float inv = sq[i][WAVES];
 #pragma unroll
       for (int x = 0; x < ET; ++x) {
         const int e = (ew + x * (WAVES / RSPLIT)) * 16 + col;
@@ -497,7 +501,7 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
         const float gt = gate[x][t][r];
         float y = acc[x][t][r] * inv;
         if (a.w) y *= ld_dyn(a.w, a.w_dtype, e);
-        y *= gt / (1.0f + expf(-gt));
+        y *= gt * __builtin_amdgcn_rcpf(1.0f + exp2_f(-gt * kLog2e));
         const size_t at = size_t(r0 + i) * a.out_stride + head * a.E + e;
         if (a.out_dtype == SB_F32) ((float *)a.out)[at] = y;
         else ((bf16_t *)a.out)[at] = f32_to_bf16(y);

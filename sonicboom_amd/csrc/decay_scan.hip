@@ -29,8 +29,9 @@ __device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v));
 
 // rate * log(sigmoid(z)) = rate * (min(z, 0) - log(1 + e)), e = exp(-|z|), by log(1 + e) = 2 artanh(s), s = e / (2 + e)
 // <= 1/3: 2 (s + s^3/3 + s^5/5 + ..), whose terms from s^17 on are below a float32 result's last digit.
+// (The hardware's exponential and reciprocal are right to a few units of the last digit, and e is small where |z| is large.)
 __device__ __forceinline__ float log_sigmoid(float z, float rate) {
-  const float e = expf(-fabsf(z)), s = e / (2.0f + e), s2 = s * s;
+  const float e = __builtin_amdgcn_exp2f(-fabsf(z) * 1.4426950408889634f), s = e * __builtin_amdgcn_rcpf(2.0f + e), s2 = s * s;
   float p = 1.0f / 15.0f;
   p = fmaf(p, s2, 1.0f / 13.0f);
   p = fmaf(p, s2, 1.0f / 11.0f);
@@ -62,7 +63,7 @@ struct DecayArgs {
 template <int NT, bool CHANNEL>
 __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_groups) {
   __shared__ __attribute__((aligned(16))) float qs[RB][MAX_SIDE], ks[RB][MAX_SIDE], as[CHANNEL ? RB : 1][CHANNEL ? MAX_SIDE : 4], ins[CHANNEL ? RB : 1][CHANNEL ? MAX_RANK : 4];
-  __shared__ float vs[RB][MAX_SIDE], os[RB][MAX_WAVES * 64];
+  __shared__ float vs[RB][MAX_SIDE], gs[RB][MAX_SIDE], os[RB][MAX_WAVES * 64];
   const int head = blockIdx.x, seq = blockIdx.y, tid = threadIdx.x, lane = tid & 63, waves = blockDim.x >> 6;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);      // (the same for all lanes: rows of S are tested once a wave)
   const int cg = wave % col_groups, d0 = (wave / col_groups) * NT, col = cg * 64 + lane;
@@ -138,7 +139,10 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
     }
     for (int idx = tid; idx < nr * a.E; idx += blockDim.x) {
       const int i = idx / a.E, e = idx - i * a.E;
-      vs[i][e] = sum_slices(a.v + size_t(rb + i) * a.row_stride + head * a.E + e, a.n_slices, a.slice_stride);
+      const size_t at = size_t(rb + i) * a.row_stride + head * a.E + e;
+      const float v = sum_slices(a.v + at, a.n_slices, a.slice_stride), g = sum_slices(a.g + at, a.n_slices, a.slice_stride);
+      vs[i][e] = v;
+      gs[i][e] = silu_f(g);
     }
     __syncthreads();
 #pragma unroll 1
@@ -160,14 +164,8 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
     __syncthreads();
     // a wave a row: the waves' shares added in ascending order of S's rows, the norm, the gate, the store
     for (int i = wave; i < nr; i += waves) {
-      float o[MAX_SIDE / 64], gate[MAX_SIDE / 64];
+      float o[MAX_SIDE / 64];
       float sq = 0.0f;
-#pragma unroll
-      for (int c = 0; c < MAX_SIDE / 64; ++c)
-        if (c < col_groups) {
-          const float *gp = a.g + size_t(rb + i) * a.row_stride + head * a.E + min(c * 64 + lane, a.E - 1);
-          gate[c] = sum_slices(gp, a.n_slices, a.slice_stride);
-        }
 #pragma unroll
       for (int c = 0; c < MAX_SIDE / 64; ++c) {
         o[c] = 0.0f;
@@ -183,7 +181,7 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
         if (c < col_groups && e < a.E) {
           float y = o[c] * inv;
           if (a.w) y *= ld_dyn(a.w, a.w_dtype, e);
-          y *= silu_f(gate[c]);
+          y *= gs[i][e];
           const size_t at = size_t(rb + i) * a.out_stride + head * a.E + e;
           if (a.out_dtype == SB_F32) ((float *)a.out)[at] = y;
           else ((bf16_t *)a.out)[at] = f32_to_bf16(y);

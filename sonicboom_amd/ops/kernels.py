@@ -1981,15 +1981,17 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     ``chunks`` int32 [n, 4]: the step's rows in runs of :func:`decay_chunk_rows` rows; the scan then takes its chunked form
     (float32 throughout; it orders its sums otherwise than the walk, from which it differs by rounding), and turns by
     ``angles``, the step's :func:`angle_table`."""
-    n = q.shape[-2]
-    row_stride, n_slices, slice_stride = q.stride(-2), (q.shape[0] if q.dim() == 3 else 1), (q.stride(0) if q.dim() == 3 else 0)
+    q_shape, q_stride = q.shape, q.stride()
+    n, row_stride = q_shape[-2], q_stride[-2]
+    n_slices, slice_stride = (q_shape[0], q_stride[0]) if len(q_shape) == 3 else (1, 0)
     if n_slices > 1 and chunks is not None:
         raise KernelLibraryError("the chunked scan takes whole rows")
 
     def part_of_rows(t, width, what):
-        for one in (t[0], t[-1]) if t.dim() == 3 else (t,):
-            _f32_rows(one, n, width, what)
-        if t.dim() != q.dim() or (n > 1 and t.stride(-2) != row_stride) or (n_slices > 1 and (t.shape[0] != n_slices or t.stride(0) != slice_stride)):
+        shape, stride = t.shape, t.stride()
+        if t.dtype != torch.float32 or shape[-2] != n or shape[-1] < width or stride[-1] != 1 or not t.is_cuda:
+            raise KernelLibraryError(f"{what} must be float32 rows [{n}, {width}] on the GPU, not {tuple(shape)}")
+        if len(shape) != len(q_shape) or (n > 1 and stride[-2] != row_stride) or (n_slices > 1 and (shape[0] != n_slices or stride[0] != slice_stride)):
             raise KernelLibraryError("queries, keys, values, gates and a decay's inner numbers must be parts of the same rows")
     for t, width, what in ((q, heads * dim, "queries"), (k, heads * dim, "keys"), (v, heads * v_dim, "values"),
                            (g, heads * v_dim, "gates")):

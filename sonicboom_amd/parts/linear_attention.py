@@ -110,7 +110,7 @@ class _DecayMixer(Mixer):
 
     def _cut(self, rows):
         qk, vw = self.qk_width, self.v_width
-        return rows[..., :qk], rows[..., qk:2 * qk], rows[..., 2 * qk:2 * qk + vw], rows[..., 2 * qk + vw:2 * (qk + vw)]
+        return rows.narrow(-1, 0, qk), rows.narrow(-1, qk, qk), rows.narrow(-1, 2 * qk, vw), rows.narrow(-1, 2 * qk + vw, vw)
 
     def takes_slices(self, ctx) -> bool:
         """Whether from_rows() adds a product's K slices itself (the walk does)."""
@@ -194,7 +194,7 @@ class GatedLinearAttention(_DecayMixer):
         q, k, v, g = self._cut(rows)
         first = 2 * (self.qk_width + self.v_width)
         return ops.decay_scan(q, k, v, g, binding.state, ctx, self.heads, self.head_dim, self.v_dim, self.eps, self.rt.act_dtype,
-                              decay_from=(rows[..., first:first + self.rank], self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
+                              decay_from=(rows.narrow(-1, first, self.rank), self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
 
 
 def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float, left_norm: str, right_norm: str,
