@@ -188,6 +188,9 @@ class GatedLinearAttention(_DecayMixer):
     def further_inputs(self, tensors):
         return [tensors["decay_down"]]
 
+    def takes_slices(self, ctx) -> bool:
+        return super().takes_slices(ctx) and self.rank <= ops.decay_scan_max_rank()
+
     def from_rows(self, rows, ctx, binding):
         """What the output product reads, from the stacked product's float32 rows (a column range of wider rows, or K
         slices of them)."""

@@ -376,7 +376,7 @@ def test_layer_norm(dtype, width, rows):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("width", [96, 61, 2048, 4096, 8192])
 @pytest.mark.parametrize("rows", [5, 130])
-@pytest.mark.parametrize("slices", [(1, 1, 1), (4, 3, 2), (8, 1, 5), (9, 2, 1), (2,), (1, 7), ()])
+@pytest.mark.parametrize("slices", [(1, 1, 1), (4, 3, 2), (8, 1, 5), (9, 2, 1), (8, 8, 4), (9, 9, 9), (2,), (1, 7), (12, 8), ()])
 def test_branches_join_the_stream_in_one_pass(dtype, width, rows, slices):
     from sonicboom_amd import ops
     x, vec = rand(rows, width, scale=2.0), rand(width, seed=8).to(BF16)
@@ -612,7 +612,7 @@ GLAS = [gla(4, 48, 32, 16.0), gla(1, 10, 14, 1.0), gla(3, 24, 72, 3.0), gla(2, 1
 def test_mixers_alone(dtype, i):
     """Both mixers whole, in portions, and token by token; what each mechanism does to the result shows."""
     layer, width, n = (SIDES + GLAS)[i], 64, 200
-    weights = random_weights(config(10, width, [layer]), seed=40 + i, rank=9)
+    weights = random_weights(config(10, width, [layer]), seed=40 + i, rank=(9, 300)[i % 2])
     mixer, ref = mixer_of(layer, width, weights, dtype)
     feed = mixer_harness(mixer, dtype, width)
     h = rand(n, width, seed=i).to(TORCH_DT[dtype])
