@@ -11,11 +11,12 @@ per-sequence state of fixed size.
   values have a size of their own).  A mixer may keep something else per token instead:
   rows of a shape of its own, ``[entries, pages, PAGE, *shape]``, in groups by
   (shape, window).  A group
-  that only reads a window of keys gives pages back as the window leaves them.
+  that only reads a window of keys gives pages back as the window leaves them, one whose
+  positions read their own chunk of positions only as the next chunk begins.
 * ``max_tokens`` sizes the pools: the most tokens live sequences hold at any
   time, each sequence's count rounded up to a whole page (PAGE = 64 tokens).
-  A group that keeps every key gets that many pages.  A group with a window
-  never holds more of a sequence than its window and the rows of the step
+  A group that keeps every key gets that many pages.  A group with a window (or a chunk)
+  never holds more of a sequence than its window (its chunk) and the rows of the step
   that is running, so with ``max_slots`` sequences and steps of at most
   ``step_rows`` rows its pool is ``max_slots * (pages(window) + 2) +
   pages(step_rows)`` pages when that is less (:func:`pool_pages`).
@@ -81,6 +82,12 @@ class GroupSpec:
     entries: Tuple[int, ...]     # cache entry numbers stored in this group
     row_shape: Tuple[int, ...] = ()   # not empty: a row of this shape per token instead of keys and values
     v_dim: int = 0               # the values' size per head when it is not head_dim (0: the same)
+    chunk: int = 0               # > 0 (window 0): a position reads the keys of its own stretch of that many positions
+
+    @property
+    def span(self) -> int:
+        """The most keys a position reads (0: all of them)."""
+        return self.chunk or self.window
 
 
 @dataclass
@@ -91,7 +98,7 @@ class _Slot:
 
 def pool_pages(n_pages: int, window: int, max_slots: int, step_rows: int) -> int:
     """Pages of a group's pool in a cache of ``n_pages``: all of them for a group that keeps
-    every key (``window`` 0); for a windowed group what ``max_slots`` sequences can hold at
+    every key (``window``, the group's span, 0); for a windowed group what ``max_slots`` sequences can hold at
     once, if that is less: after a step a sequence keeps the pages its window touches
     (pages(window) + 1 at most), and a step of up to ``step_rows`` rows adds pages(rows) + 1 pages
     a sequence before the old ones are given back."""
@@ -112,7 +119,7 @@ class PagedCache:
         self.n_pages = pages_for(max_tokens)
         self.max_slots = max_slots if max_slots is not None else self.n_pages
         self.step_rows = int(step_rows)
-        self.pools = [PagePool(pool_pages(self.n_pages, g.window, self.max_slots, self.step_rows))
+        self.pools = [PagePool(pool_pages(self.n_pages, g.span, self.max_slots, self.step_rows))
                       for g in self.groups]
         self._slots: Dict[int, _Slot] = {}
         self._free_slots = list(range(self.max_slots - 1, -1, -1))
@@ -190,14 +197,16 @@ class PagedCache:
     # ---- a step ------------------------------------------------------------
     def _first_needed_page(self, g: int, length: int) -> int:
         """Logical page of the oldest key that a query at position ``length`` still reads."""
-        w = self.groups[g].window
+        chunk, w = self.groups[g].chunk, self.groups[g].window
+        if chunk > 0:
+            return length // chunk * chunk // PAGE
         if w <= 0:
             return 0
         return max(0, length - w + 1) // PAGE
 
     def windowed(self, flag: bool) -> List[int]:
-        """The groups that read a window of keys (``flag`` true) or every key (false)."""
-        return [g for g, spec in enumerate(self.groups) if (spec.window > 0) == flag]
+        """The groups that read a window (or a chunk) of keys (``flag`` true) or every key (false)."""
+        return [g for g, spec in enumerate(self.groups) if (spec.span > 0) == flag]
 
     def reserve(self, slots: Sequence[int], n_new: Sequence[int], groups: Optional[Sequence[int]] = None) -> None:
         """Pages for ``n_new[i]`` more tokens of ``slots[i]``, all or nothing; ``groups``: in
@@ -295,7 +304,7 @@ class PagedCache:
 
 
 def group_entries(specs: Dict[int, tuple]) -> List[GroupSpec]:
-    """Group cache entries {entry: (kv_heads, head_dim, window[, values' size])}, or {entry: ("rows",
+    """Group cache entries {entry: (kv_heads, head_dim, window[, values' size[, chunk]])}, or {entry: ("rows",
     shape, window)} for entries that keep a row of their own shape per token, by equal needs, in order
     of first use."""
     by_need: Dict[tuple, List[int]] = {}
@@ -304,5 +313,5 @@ def group_entries(specs: Dict[int, tuple]) -> List[GroupSpec]:
     def values_size(k):
         return k[3] if len(k) > 3 and k[3] != k[1] else 0
     return [GroupSpec(0, 0, k[2], tuple(v), tuple(k[1])) if k[0] == "rows"
-            else GroupSpec(k[0], k[1], k[2], tuple(v), v_dim=values_size(k))
+            else GroupSpec(k[0], k[1], k[2], tuple(v), v_dim=values_size(k), chunk=k[4] if len(k) > 4 else 0)
             for k, v in by_need.items()]

@@ -19,6 +19,9 @@
 // `all_values`: every query head's weights applied to the values of every kv head, not its own alone
 // (the grid then holds a block per value head too, and the result is [rows, heads_q, heads_kv, dv]).
 //
+// A row sees the keys up to its own, with `window` > 0 that many at most, with `chunk` > 0 those of its own stretch of
+// `chunk` positions ([chunk * (p / chunk), p]).
+//
 // Softmax in float32, running maximum and sum per query column, scores kept times log2(e) so that the
 // weights are powers of two; a sink starts the maximum at 0 and the sum at 1.  Steps of few rows
 // share the pages of a sequence out over `chunks` blocks, which leave (unnormed result, maximum,
@@ -70,6 +73,7 @@ struct Args {
   const float *sink_scores;            // [heads_q] or NULL: the sink's score a head (NULL: 0)
   const float *gate; int gate_stride;  // [rows, gate_stride] or NULL: the result times sigmoid(gate[row][h * DV + d]),
   int gate_per_head;                   // or, when set, times sigmoid(gate[row][h])
+  int key_chunk;               // > 0 (window 0): position p sees the keys from key_chunk * (p / key_chunk) on
   unsigned round_blocks;       // blocks the GPU takes one of per CU
 };
 
@@ -80,6 +84,12 @@ constexpr float kLog2e = 1.4426950408889634f;
 __device__ __forceinline__ float capped(float s, float cap, float two_log2e_over_cap) {
   const float t = fminf(s * two_log2e_over_cap, 60.0f);          // 2^60 + 1 is 2^60 in float32: tanh is 1 by then
   return cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(t) + 1.0f));
+}
+
+// oldest key that position p sees
+__device__ __forceinline__ int oldest_key(const Args &a, int p) {
+  if (a.key_chunk > 0) return p - p % a.key_chunk;
+  return (a.window > 0 && p >= a.window) ? p - a.window + 1 : 0;
 }
 
 __global__ void __launch_bounds__(kThreads) capped_attention_kernel(Args a) {
@@ -107,11 +117,12 @@ __global__ void __launch_bounds__(kThreads) capped_attention_kernel(Args a) {
   const int r0 = tile[0], nr = tile[1], seq = tile[2];
   const int chunk = blockIdx.z;
   const int p0 = a.row_pos[r0], p_last = p0 + nr - 1;
-  const int lo = (a.window > 0 && p0 >= a.window) ? p0 - a.window + 1 : 0;      // oldest key any row of the tile reads
+  const int lo = oldest_key(a, p0);               // oldest key any row of the tile reads (it never falls from row to row)
+  const int lo_last = oldest_key(a, p_last);      // oldest key that every row reads
   int page_lo = lo / SB_PAGE, page_hi = p_last / SB_PAGE;
-  if (a.chunk_pages > 0) {
-    page_lo = max(page_lo, chunk * a.chunk_pages);
-    page_hi = min(page_hi, (chunk + 1) * a.chunk_pages - 1);
+  if (a.chunk_pages > 0) {                        // shares are counted from the first page the tile reads
+    page_lo += chunk * a.chunk_pages;
+    page_hi = min(page_hi, page_lo + a.chunk_pages - 1);
   }
   const int32_t *table = a.page_table + size_t(seq) * a.max_pages;
 
@@ -123,7 +134,7 @@ __global__ void __launch_bounds__(kThreads) capped_attention_kernel(Args a) {
     qf[kc] = as_bf16x8(ld16(a.q + (size_t(r0 + col) * a.heads_q + h) * DK + d, has_head && col < nr && d < DK));
   }
   const int q_pos = p0 + col;
-  const int q_lo = (a.window > 0 && q_pos >= a.window) ? q_pos - a.window + 1 : 0;
+  const int q_lo = oldest_key(a, q_pos);
 
   const float neg_inf = -__builtin_inff();
   const bool with_sink = a.sink && chunk == 0;
@@ -202,7 +213,7 @@ __global__ void __launch_bounds__(kThreads) capped_attention_kernel(Args a) {
       const int first = c * SB_PAGE + 32 * hp;          // position of the half page's first key
       if (first > p_last || first + 31 < lo) continue;  // uniform over the block
       // every row of the tile sees every key of this half page: no score needs a test (uniform)
-      const bool whole = nr == kTile && first + 31 <= p0 && (a.window == 0 || first >= p_last - a.window + 1);
+      const bool whole = nr == kTile && first + 31 <= p0 && first >= lo_last;
       // every fragment of the half page is asked of LDS before the first product: the keys' for the
       // scores, and the values' too, which arrive while the softmax is worked out (read one by one
       // before its product, each fragment's trip through LDS showed in full: a CU holds few waves here)
@@ -421,12 +432,38 @@ extern "C" int sb_cattn_shared_bf16(void *out, const void *q, const void *k_cach
 // The same with a sink whose score is a number of the query head's own (sink_scores f32 [heads_q], as it is: not
 // scaled, not capped; NULL: 0), and with an output gate (f32 [rows, gate_stride] or NULL; not with all_values): the
 // result times sigmoid(gate[row * gate_stride + h * dv + d]), or with gate_per_head times sigmoid(gate[row * gate_stride + h]).
+extern "C" int sb_cattn_chunked_bf16(void *out, const void *q, const void *k_cache, const void *v_cache,
+                                     const int32_t *page_table, int max_pages, int n_pages, const int32_t *row_pos,
+                                     const int32_t *tiles, int n_tiles, int n_rows, int heads_q, int heads_kv, float scale,
+                                     int window, float softcap, int sink, int chunks, int chunk_pages, float *part_o,
+                                     float *part_ml, const float *dist_r1, const float *dist_r2, int all_values,
+                                     const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, int key_chunk,
+                                     void *stream);
+
 extern "C" int sb_cattn_sink_bf16(void *out, const void *q, const void *k_cache, const void *v_cache,
                                   const int32_t *page_table, int max_pages, int n_pages, const int32_t *row_pos,
                                   const int32_t *tiles, int n_tiles, int n_rows, int heads_q, int heads_kv, float scale,
                                   int window, float softcap, int sink, int chunks, int chunk_pages, float *part_o,
                                   float *part_ml, const float *dist_r1, const float *dist_r2, int all_values,
                                   const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, void *stream) {
+  return sb_cattn_chunked_bf16(out, q, k_cache, v_cache, page_table, max_pages, n_pages, row_pos, tiles, n_tiles, n_rows, heads_q,
+                               heads_kv, scale, window, softcap, sink, chunks, chunk_pages, part_o, part_ml, dist_r1, dist_r2,
+                               all_values, sink_scores, gate, gate_stride, gate_per_head, 0, stream);
+}
+
+// The same where, with key_chunk > 0 (and window 0), position p sees the keys from key_chunk * (p / key_chunk) on.  Where a
+// row sees a window or a chunk only, chunks * chunk_pages need cover no more pages than a tile's rows can touch.
+extern "C" int sb_cattn_chunked_bf16(void *out, const void *q, const void *k_cache, const void *v_cache,
+                                     const int32_t *page_table, int max_pages, int n_pages, const int32_t *row_pos,
+                                     const int32_t *tiles, int n_tiles, int n_rows, int heads_q, int heads_kv, float scale,
+                                     int window, float softcap, int sink, int chunks, int chunk_pages, float *part_o,
+                                     float *part_ml, const float *dist_r1, const float *dist_r2, int all_values,
+                                     const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, int key_chunk,
+                                     void *stream) {
+  SB_REQUIRE(key_chunk >= 0 && (key_chunk == 0 || window == 0), "sb_cattn_bf16: a window and a chunk at once");
+  const int span = key_chunk > 0 ? key_chunk : window;
+  // pages that span + kTile - 1 neighbouring keys can touch
+  const long long cover = span > 0 ? min((long long)max_pages, ((long long)span + kTile - 1 + 2 * SB_PAGE - 2) / SB_PAGE) : max_pages;
   SB_REQUIRE(!sink_scores || sink, "sb_cattn_bf16: scores of a sink that is switched off");
   SB_REQUIRE(!gate || (!all_values && gate_stride >= heads_q * (gate_per_head ? 1 : DV)), "sb_cattn_bf16: the gate's rows of %d are too short", gate_stride);
   SB_REQUIRE((dist_r1 == nullptr) == (dist_r2 == nullptr), "sb_cattn_bf16: the distance bias needs both of its numbers");
@@ -436,8 +473,8 @@ extern "C" int sb_cattn_sink_bf16(void *out, const void *q, const void *k_cache,
   SB_REQUIRE(heads_q % heads_kv == 0, "sb_cattn_bf16: %d query heads are not a multiple of %d kv heads", heads_q, heads_kv);
   SB_REQUIRE(softcap >= 0.0f, "sb_cattn_bf16: the cap of the scores must not be negative");
   SB_REQUIRE(chunks >= 1 && (chunks == 1 || (part_o && part_ml && chunk_pages > 0 &&
-                                             (long long)chunks * chunk_pages >= max_pages)),
-             "sb_cattn_bf16: %d chunks of %d pages do not cover %d pages, or have no scratch", chunks, chunk_pages, max_pages);
+                                             (long long)chunks * chunk_pages >= cover)),
+             "sb_cattn_bf16: %d chunks of %d pages do not cover %d pages, or have no scratch", chunks, chunk_pages, int(cover));
   if (n_tiles == 0 || n_rows == 0) return SB_OK;
   const int group = heads_q / heads_kv, zgroups = (group + NW - 1) / NW;
   const int value_heads = all_values ? heads_kv : 1;
@@ -451,6 +488,7 @@ extern "C" int sb_cattn_sink_bf16(void *out, const void *q, const void *k_cache,
   a.page_table = page_table; a.max_pages = max_pages; a.n_pages = n_pages; a.row_pos = row_pos; a.tiles = tiles;
   a.n_rows = n_rows; a.heads_q = heads_q; a.heads_kv = heads_kv; a.scale = scale; a.softcap = softcap;
   a.window = window; a.sink = sink; a.chunk_pages = chunks == 1 ? 0 : chunk_pages;
+  a.key_chunk = key_chunk;
   a.round_blocks = unsigned(sb::cu_count());
   a.dist_r1 = dist_r1; a.dist_r2 = dist_r2; a.all_values = all_values ? 1 : 0;
   a.sink_scores = sink_scores;

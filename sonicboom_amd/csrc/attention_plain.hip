@@ -5,7 +5,9 @@
 // Formula: /root/reference/core/src/nn/attention.cpp:26-105 and :121-181 —
 // query head h reads kv head h / group; s_j = dot(q, k_j) * scale; a key is
 // visible when j <= p and (window == 0 or p - j < window); softmax with the
-// maximum subtracted; a row without visible keys is zero.
+// maximum subtracted; a row without visible keys is zero.  With `chunk` > 0 (no
+// window then) the keys of position p's own stretch of that many positions are
+// visible, [chunk * (p / chunk), p].
 //
 // The cache holds keys as [page][kv head][position][d] and values transposed,
 // [page][kv head][d][position].
@@ -30,7 +32,7 @@ attention_plain_kernel(TA *__restrict__ out, const TA *__restrict__ q, int q_str
                        const int32_t *__restrict__ row_pos, const int32_t *__restrict__ row_seq,
                        int heads_q, int heads_kv, int head_dim, float scale, int window, int v_dim,
                        float softcap, int sink, const float *__restrict__ sink_scores,
-                       const float *__restrict__ gate, int gate_stride, int gate_per_head) {
+                       const float *__restrict__ gate, int gate_stride, int gate_per_head, int chunk) {
   __shared__ float qs[kMaxHeadDim];
   __shared__ float ps[64];
   const int row = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
@@ -39,7 +41,7 @@ attention_plain_kernel(TA *__restrict__ out, const TA *__restrict__ q, int q_str
   for (int d = lane; d < head_dim; d += 64) qs[d] = ld_f(q, size_t(row) * q_stride + size_t(h) * head_dim + d);
   __syncthreads();
 
-  const int lo = (window > 0 && pos >= window) ? pos - window + 1 : 0;
+  const int lo = chunk > 0 ? pos - pos % chunk : (window > 0 && pos >= window) ? pos - window + 1 : 0;
   const float neg_inf = -__builtin_inff();
   // a sink is one more key that has no value, of score 0 or, with sink_scores, of the head's own
   // number (as it is: no scale, no cap): the running maximum starts at its score and the running
@@ -96,6 +98,14 @@ attention_plain_kernel(TA *__restrict__ out, const TA *__restrict__ q, int q_str
 
 }  // namespace
 
+extern "C" int sb_attention_chunked(void *out, const void *q, int act_dtype, int q_stride, const void *k_cache,
+                                    const void *v_cache, int cache_dtype, const int32_t *page_table,
+                                    int max_pages, int n_pages_total, const int32_t *row_pos,
+                                    const int32_t *row_seq, int n_rows, int heads_q, int heads_kv,
+                                    int head_dim, int v_dim, float scale, int window, float softcap, int sink,
+                                    const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, int chunk,
+                                    void *stream);
+
 // The same with values of another size than the keys (v_dim; the cache then holds values
 // [page][kv head][v_dim][position] and out is [rows, heads_q * v_dim]), scores capped as
 // softcap * tanh(s / softcap) when softcap > 0, and with `sink` one more key of score 0 without a
@@ -145,6 +155,20 @@ extern "C" int sb_attention_sink(void *out, const void *q, int act_dtype, int q_
                                  const int32_t *row_seq, int n_rows, int heads_q, int heads_kv,
                                  int head_dim, int v_dim, float scale, int window, float softcap, int sink,
                                  const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, void *stream) {
+  return sb_attention_chunked(out, q, act_dtype, q_stride, k_cache, v_cache, cache_dtype, page_table, max_pages, n_pages_total, row_pos,
+                              row_seq, n_rows, heads_q, heads_kv, head_dim, v_dim, scale, window, softcap, sink, sink_scores, gate,
+                              gate_stride, gate_per_head, 0, stream);
+}
+
+// The same where, with chunk > 0 (and window 0), position p sees the keys from chunk * (p / chunk) on.
+extern "C" int sb_attention_chunked(void *out, const void *q, int act_dtype, int q_stride, const void *k_cache,
+                                    const void *v_cache, int cache_dtype, const int32_t *page_table,
+                                    int max_pages, int n_pages_total, const int32_t *row_pos,
+                                    const int32_t *row_seq, int n_rows, int heads_q, int heads_kv,
+                                    int head_dim, int v_dim, float scale, int window, float softcap, int sink,
+                                    const float *sink_scores, const float *gate, int gate_stride, int gate_per_head, int chunk,
+                                    void *stream) {
+  SB_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "sb_attention: a window and a chunk at once");
   SB_REQUIRE(!sink_scores || sink, "sb_attention: scores of a sink that is switched off");
   SB_REQUIRE(!gate || gate_stride >= heads_q * (gate_per_head ? 1 : v_dim), "sb_attention: the gate's rows of %d are too short", gate_stride);
   SB_REQUIRE(out && q && k_cache && v_cache && page_table && row_pos && row_seq,
@@ -169,7 +193,7 @@ extern "C" int sb_attention_sink(void *out, const void *q, int act_dtype, int q_
   attention_plain_kernel<TA, TC><<<grid, 64, 0, s>>>(                                            \
       (TA *)out, (const TA *)q, q_stride, (const TC *)k_cache, (const TC *)v_cache, page_table,  \
       max_pages, n_pages_total, row_pos, row_seq, heads_q, heads_kv, head_dim, scale, window, v_dim,  \
-      softcap, sink, sink_scores, gate, gate_stride, gate_per_head)
+      softcap, sink, sink_scores, gate, gate_stride, gate_per_head, chunk)
   if (act_dtype == SB_F32 && cache_dtype == SB_F32) SB_GO(float, float);
   else if (act_dtype == SB_BF16 && cache_dtype == SB_BF16) SB_GO(bf16_t, bf16_t);
   else if (act_dtype == SB_F32 && cache_dtype == SB_BF16) SB_GO(float, bf16_t);

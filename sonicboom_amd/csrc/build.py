@@ -12,8 +12,7 @@ Two kinds of library come out of it:
 A library lives in ``_build/`` beside the sources together with a stamp that
 holds the hash of the sources and flags it was made from.  :func:`ensure`
 loads nothing; it returns the path of an up-to-date library and compiles it
-first when the stamp does not match, printing a line per file and a line every
-few seconds while the compiler runs.  When the source folder cannot be written
+first when the stamp does not match, printing a line per file.  When the source folder cannot be written
 the libraries go to a per-user folder under the system's temporary directory.
 """
 from __future__ import annotations
@@ -24,7 +23,6 @@ import shutil
 import subprocess
 import sys
 import tempfile
-import threading
 import time
 from concurrent.futures import ThreadPoolExecutor
 
@@ -43,7 +41,7 @@ CORE_SOURCES = [
     "attention_plain.hip", "sampling.hip", "gemm_skinny.hip", "gemm_stream.hip", "gemm_mfma.hip",
     "random_fill.hip", "recurrent.hip", "attention_latent.hip", "attention_latent_mfma.hip",
     "outnorm.hip", "headnorm_kv.hip", "moe.hip", "moe_mfma.hip", "timeconv.hip", "state_space.hip",
-    "attention_mixed.hip", "join.hip", "decay_scan.hip", "decay_chunks.hip",
+    "attention_mixed.hip", "join.hip", "decay_scan.hip", "decay_chunks.hip", "streams.hip", "rownorm.hip", "gated_lru.hip",
 ]
 HEADERS = ["common.h", "sb_hip.h", "mfma.h"]
 ATTN_SOURCES = ["attention_mfma.hip"]
@@ -127,29 +125,18 @@ def _compile_library(lib_name, sources, defines, jobs) -> str:
     flags = FLAGS + [f"-D{d}" for d in defines] + [f'-DSB_BUILD_FLAGS="{ARCH} -O3 no-packed-fp32"', f"-I{HERE}"]
     _log(f"compiling {lib_name} for {ARCH}: {len(sources)} file(s), {jobs} at a time")
     t0 = time.time()
-    done = threading.Event()
-
-    def heartbeat():
-        while not done.wait(15.0):
-            _log(f"  ... still compiling {lib_name} ({time.time() - t0:.0f} s)")
-
-    hb = threading.Thread(target=heartbeat, daemon=True)
-    hb.start()
-    try:
-        def one(src):
-            obj = os.path.join(obj_dir, src.replace(".hip", ".o"))
-            _run([cc, *flags, "-c", os.path.join(HERE, src), "-o", obj], f"compiling {src}")
-            _log(f"  compiled {src} ({time.time() - t0:.0f} s)")
-            return obj
-        with ThreadPoolExecutor(max_workers=max(1, jobs)) as ex:
-            objs = list(ex.map(one, sources))
-        tmp = lib + f".tmp{os.getpid()}"
-        _run([cc, "-shared", "-fPIC", f"--offload-arch={ARCH}", *objs, "-o", tmp], f"linking {lib_name}")
-        os.replace(tmp, lib)
-        with open(stamp, "w") as f:
-            f.write(want)
-    finally:
-        done.set()
+    def one(src):
+        obj = os.path.join(obj_dir, src.replace(".hip", ".o"))
+        _run([cc, *flags, "-c", os.path.join(HERE, src), "-o", obj], f"compiling {src}")
+        _log(f"  compiled {src} ({time.time() - t0:.0f} s)")
+        return obj
+    with ThreadPoolExecutor(max_workers=max(1, jobs)) as ex:
+        objs = list(ex.map(one, sources))
+    tmp = lib + f".tmp{os.getpid()}"
+    _run([cc, "-shared", "-fPIC", f"--offload-arch={ARCH}", *objs, "-o", tmp], f"linking {lib_name}")
+    os.replace(tmp, lib)
+    with open(stamp, "w") as f:
+        f.write(want)
     _log(f"built {lib} in {time.time() - t0:.0f} s")
     return lib
 

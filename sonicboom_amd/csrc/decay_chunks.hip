@@ -12,6 +12,7 @@
 // exp(L_i - R) and exp(R - L_j) with R = L at the row before the tile's first row i, and the pairs of a tile on the
 // diagonal are summed one by one on the vector units with exp(L_i - L_j) as it is.
 //
+// With `act_in` q, k and v are the silu of what is read; with `plain` o goes out as it is, float32, and g is not read.
 // q and k may turn on the way in, by a table of the rows' cosines and sines (sb_angle_table, once a step).
 // Operands in LDS: rows a multiple of 64 numbers and four further on, so that the sixteen rows and four columns a
 // wave's operand takes lie in distinct banks; where the rows are summed over, sixteen further on.
@@ -44,7 +45,10 @@ struct ChunkArgs {
   float *part;                               // [n_chunks, heads, D, E]: A_c, then S_in(c)
   float *part_decay;                         // [n_chunks, heads, D]: exp(L_last) (a decay a channel only)
   int vec4;                                  // rows can be read four numbers at a time
+  int act_in, plain;                         // silu on q, k and v; out is o as it is
 };
+
+__device__ __forceinline__ float silu_f(float v) { return v / (1.0f + expf(-v)); }
 
 // What a thread needs for four numbers of a head's row: themselves, what they turn with, cosines and sines.
 struct Four { float4 x, o, t0, t1; };
@@ -68,9 +72,18 @@ __device__ __forceinline__ void fetch_four(Four &f, const ChunkArgs &a, const fl
 
 __device__ __forceinline__ float4 finish_four(const Four &f, const ChunkArgs &a, int d, bool live, float scale, bool turning) {
   float x[4] = {f.x.x, f.x.y, f.x.z, f.x.w};
+  if (a.act_in) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[e] = silu_f(x[e]);
+  }
   if (turning) {
     const bool lo = d < a.half, on = d < 2 * a.half;
-    const float o[4] = {f.o.x, f.o.y, f.o.z, f.o.w}, c[4] = {f.t0.x, f.t0.z, f.t1.x, f.t1.z}, s[4] = {f.t0.y, f.t0.w, f.t1.y, f.t1.w};
+    float o[4] = {f.o.x, f.o.y, f.o.z, f.o.w};
+    if (a.act_in) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] = silu_f(o[e]);
+    }
+    const float c[4] = {f.t0.x, f.t0.z, f.t1.x, f.t1.z}, s[4] = {f.t0.y, f.t0.w, f.t1.y, f.t1.w};
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       float y0, y1;
@@ -89,11 +102,12 @@ __device__ __forceinline__ float4 load_single(const ChunkArgs &a, const float *h
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
     if (d + e >= a.D) continue;
-    x[e] = src[d + e];
+    x[e] = a.act_in ? silu_f(src[d + e]) : src[d + e];
     if (d + e < 2 * a.half) {
       const bool lo = d + e < a.half;
       const int i = lo ? d + e : d + e - a.half;
-      const float ov = src[lo ? d + e + a.half : d + e - a.half];
+      float ov = src[lo ? d + e + a.half : d + e - a.half];
+      if (a.act_in) ov = silu_f(ov);
       const float2 t = a.angles[size_t(row) * a.half + i];
       float y0, y1;
       rotate_pair(lo ? x[e] : ov, lo ? ov : x[e], t.x, t.y, y0, y1);
@@ -180,13 +194,15 @@ __global__ void __launch_bounds__(THREADS) chunk_local_kernel(ChunkArgs a) {
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int idx = tid + u * THREADS, i = idx / (EP / 4), e = (idx % (EP / 4)) * 4;
+      if (a.act_in) x[u] = make_float4(silu_f(x[u].x), silu_f(x[u].y), silu_f(x[u].z), silu_f(x[u].w));
       *(float4 *)&vs[i][e] = (i < nr && e < a.E) ? x[u] : make_float4(0.f, 0.f, 0.f, 0.f);
     }
   } else {
     stage_heads<DP, CR, KS>(a, nullptr, kp, r0, nr, nullptr, &ks[0][0]);
     for (int idx = tid; idx < CR * EP; idx += THREADS) {
       const int i = idx / EP, e = idx % EP;
-      vs[i][e] = (i < nr && e < a.E) ? vp[size_t(r0 + i) * a.row_stride + e] : 0.0f;
+      float v = (i < nr && e < a.E) ? vp[size_t(r0 + i) * a.row_stride + e] : 0.0f;
+      vs[i][e] = a.act_in ? silu_f(v) : v;
     }
   }
   __syncthreads();
@@ -421,6 +437,12 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
     }
   }
   __syncthreads();
+  if (a.act_in) {
+#pragma unroll
+    for (int x = 0; x < ET; ++x)
+#pragma unroll
+      for (int u = 0; u < CR / 4; ++u) vv[x][u] = silu_f(vv[x][u]);
+  }
   // ---- o = q S_in (scaled) + P v
   f32x4_t acc[ET][RT];
   bool live[ET];
@@ -452,6 +474,21 @@ __global__ void __launch_bounds__(THREADS) chunk_from_kernel(ChunkArgs a) {
         for (int s = 0; s < 4; ++s)
           acc[x][t] = mfma_f32(ps[(16 * (t0 + t) + col) * PS + 16 * J + 4 * s + grp], vv[x][4 * J + s], acc[x][t]);
       }
+  }
+  if (a.plain) {
+#pragma unroll
+    for (int x = 0; x < ET; ++x) {
+      const int e = (ew + x * (WAVES / RSPLIT)) * 16 + col;
+      if (!live[x] || e >= a.E) continue;
+#pragma unroll
+      for (int t = 0; t < RT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int i = 16 * (t0 + t) + 4 * grp + r;
+          if (i < nr) ((float *)a.out)[size_t(r0 + i) * a.out_stride + head * a.E + e] = acc[x][t][r];
+        }
+    }
+    return;
   }
   // the gate's numbers arrive while the norms are worked out
   float gate[ET][RT][4];
@@ -560,8 +597,9 @@ extern "C" int sb_decay_chunks(void *out, int out_dtype, int out_stride, const f
                                const float *angles, int half, float q_scale, float k_scale, const void *w, int w_dtype,
                                float eps, float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads,
                                int D, int E, const int32_t *chunks, int n_chunks, int chunk_rows, float *part,
-                               float *part_decay, void *stream) {
-  SB_REQUIRE(out && q && k && v && g && state && cu_rows && slots && chunks && part && (log_decay ? part_decay != nullptr : decay != nullptr),
+                               float *part_decay, int act_in, int plain, void *stream) {
+  SB_REQUIRE(!plain || out_dtype == SB_F32, "sb_decay_chunks: what is read goes out in float32");
+  SB_REQUIRE(out && q && k && v && (g || plain) && state && cu_rows && slots && chunks && part && (log_decay ? part_decay != nullptr : decay != nullptr),
              "sb_decay_chunks: null pointer");
   SB_REQUIRE(n_seqs >= 0 && n_chunks >= 0 && heads > 0 && D > 0 && E > 0 && sb::valid_dtype(out_dtype) && (!w || sb::valid_dtype(w_dtype)),
              "sb_decay_chunks: bad sizes heads=%d dim=%d vdim=%d", heads, D, E);
@@ -576,7 +614,7 @@ extern "C" int sb_decay_chunks(void *out, int out_dtype, int out_stride, const f
                    (!angles || half % 4 == 0);
   const ChunkArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, log_decay, ld_stride, decay, (const float2 *)angles,
                     angles ? half : 0, q_scale, k_scale, w, w_dtype, eps, state, cu_rows, slots, heads, D, E, chunks, part,
-                    log_decay ? part_decay : nullptr, vec4};
+                    log_decay ? part_decay : nullptr, vec4, act_in, plain};
   if (log_decay) launch_by_dim<true>(a, n_chunks, n_seqs, (hipStream_t)stream);
   else launch_by_dim<false>(a, n_chunks, n_seqs, (hipStream_t)stream);
   return sb::check_launch("sb_decay_chunks");

@@ -5,7 +5,8 @@
 // with alpha either one constant number per head (`decay`) or a number per head and key channel, given by its
 // logarithm (`log_decay` [rows, heads * D]) or made here as sb_log_decay makes it from `inner` [rows, rank].  q and k are read from float32 rows; with inv_freq the pairs
 // (i, i + rot_dims / 2) of the first rot_dims numbers of every head turn by position * inv_freq[i]; then they are
-// multiplied by q_scale and k_scale.  The state of sequence s lies in state[slots[s]] and goes from step to step.
+// multiplied by q_scale and k_scale.  With `act_in` q, k and v are the silu of what is read (before anything turns); with
+// `plain` out is o itself, float32, and g is not read.  The state of sequence s lies in state[slots[s]] and goes from step to step.
 //
 // The walk: a block a (sequence, head), rows in order.  A wave holds NT rows of S for 64 neighbouring columns
 // in registers (its loads and stores of the state are whole lines); up to sixteen waves share a head.  Eight rows
@@ -57,6 +58,7 @@ struct DecayArgs {
   float *state;                                          // [slots, heads, D, E]
   const int32_t *cu_rows, *slots;
   int heads, D, E;
+  int act_in, plain;                                     // silu on q, k and v; out is o as it is
 };
 
 // Column groups of 64 and the rows of S that a wave takes.
@@ -98,13 +100,15 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
       if (d < a.D) {
         q = sum_slices(a.q + at, a.n_slices, a.slice_stride);
         k = sum_slices(a.k + at, a.n_slices, a.slice_stride);
+        if (a.act_in) { q = silu_f(q); k = silu_f(k); }
         if (d < 2 * half) {
           const int pair = d < half ? d : d - half, other = d < half ? half : -half;
           const float theta = float(a.row_pos[rb + i]) * a.inv_freq[pair];
           const float c = cosf(theta), s = sinf(theta);
           float y0, y1;
-          const float qo = sum_slices(a.q + at + other, a.n_slices, a.slice_stride);
-          const float ko = sum_slices(a.k + at + other, a.n_slices, a.slice_stride);
+          float qo = sum_slices(a.q + at + other, a.n_slices, a.slice_stride);
+          float ko = sum_slices(a.k + at + other, a.n_slices, a.slice_stride);
+          if (a.act_in) { qo = silu_f(qo); ko = silu_f(ko); }
           rotate_pair(d < half ? q : qo, d < half ? qo : q, c, s, y0, y1);
           q = d < half ? y0 : y1;
           rotate_pair(d < half ? k : ko, d < half ? ko : k, c, s, y0, y1);
@@ -140,9 +144,9 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
     for (int idx = tid; idx < nr * a.E; idx += blockDim.x) {
       const int i = idx / a.E, e = idx - i * a.E;
       const size_t at = size_t(rb + i) * a.row_stride + head * a.E + e;
-      const float v = sum_slices(a.v + at, a.n_slices, a.slice_stride), g = sum_slices(a.g + at, a.n_slices, a.slice_stride);
-      vs[i][e] = v;
-      gs[i][e] = silu_f(g);
+      const float v = sum_slices(a.v + at, a.n_slices, a.slice_stride);
+      vs[i][e] = a.act_in ? silu_f(v) : v;
+      if (!a.plain) gs[i][e] = silu_f(sum_slices(a.g + at, a.n_slices, a.slice_stride));
     }
     __syncthreads();
 #pragma unroll 1
@@ -174,11 +178,15 @@ __global__ void __launch_bounds__(1024) decay_walk_kernel(DecayArgs a, int col_g
           sq = fmaf(o[c], o[c], sq);
         }
       }
-      const float inv = 1.0f / sqrtf(wave_sum(sq) / float(a.E) + a.eps);
+      const float inv = a.plain ? 1.0f : 1.0f / sqrtf(wave_sum(sq) / float(a.E) + a.eps);
 #pragma unroll
       for (int c = 0; c < MAX_SIDE / 64; ++c) {
         const int e = c * 64 + lane;
         if (c < col_groups && e < a.E) {
+          if (a.plain) {
+            ((float *)a.out)[size_t(rb + i) * a.out_stride + head * a.E + e] = o[c];
+            continue;
+          }
           float y = o[c] * inv;
           if (a.w) y *= ld_dyn(a.w, a.w_dtype, e);
           y *= gs[i][e];
@@ -260,8 +268,9 @@ extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const flo
                              int inner_stride, const float *up, const float *bias, int rank, float rate, const float *decay,
                              const float *inv_freq, int rot_dims, const int32_t *row_pos, float q_scale, float k_scale,
                              const void *w, int w_dtype, float eps, float *state, const int32_t *cu_rows,
-                             const int32_t *slots, int n_seqs, int heads, int D, int E, void *stream) {
-  SB_REQUIRE(out && q && k && v && g && state && cu_rows && slots && (log_decay || inner || decay), "sb_decay_scan: null pointer");
+                             const int32_t *slots, int n_seqs, int heads, int D, int E, int act_in, int plain, void *stream) {
+  SB_REQUIRE(out && q && k && v && (g || plain) && state && cu_rows && slots && (log_decay || inner || decay), "sb_decay_scan: null pointer");
+  SB_REQUIRE(!plain || out_dtype == SB_F32, "sb_decay_scan: what is read goes out in float32");
   SB_REQUIRE(!inner || (up && bias && rank > 0), "sb_decay_scan: decays without their matrix or bias");
   SB_SUPPORT(!inner || rank <= MAX_RANK, "sb_decay_scan: a rank of %d is more than %d", rank, MAX_RANK);
   SB_REQUIRE(n_slices >= 1, "sb_decay_scan: at least one slice");
@@ -274,7 +283,7 @@ extern "C" int sb_decay_scan(void *out, int out_dtype, int out_stride, const flo
   if (n_seqs == 0) return SB_OK;
   const DecayArgs a{out, out_dtype, out_stride, q, k, v, g, row_stride, n_slices, slice_stride, log_decay, ld_stride, inner, inner_stride, up, bias,
                     rank, rate, decay, inv_freq, inv_freq ? rot_dims : 0,
-                    row_pos, q_scale, k_scale, w, w_dtype, eps, state, cu_rows, slots, heads, D, E};
+                    row_pos, q_scale, k_scale, w, w_dtype, eps, state, cu_rows, slots, heads, D, E, act_in, plain};
   if (log_decay || inner) launch_walk<true>(a, n_seqs, (hipStream_t)stream);
   else launch_walk<false>(a, n_seqs, (hipStream_t)stream);
   return sb::check_launch("sb_decay_scan");

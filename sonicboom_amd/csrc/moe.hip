@@ -106,12 +106,82 @@ __device__ __forceinline__ void load8(const bf16_t *p, float (&v)[8]) {
   for (int i = 0; i < 4; ++i) { v[2 * i] = __uint_as_float(u[i] << 16); v[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u); }
 }
 
+// The choice of one row by corrected sigmoid scores, by the first wave of a block of 256 (all threads must come along):
+// score_e = sigmoid(z_e), choice score c_e = score_e + correction_e; a group of neighbours counts by the sum of its two
+// largest choice scores; among the experts of the keep_groups best groups the `top` with the largest choice scores are
+// chosen (ties to the lower number), their weights are score_scale * score / (the chosen scores' sum + 1e-20).
+// scores, choice: n_experts numbers each in LDS.
+__device__ __forceinline__ void route_row_corrected(int32_t *__restrict__ ids, float *__restrict__ weights, const float *zr,
+                                                    const float *__restrict__ correction, float *scores, float *choice, int r,
+                                                    int n_experts, int top, float score_scale, int n_groups, int keep_groups) {
+  const int tid = threadIdx.x, lane = tid & 63;
+  for (int e = tid; e < n_experts; e += 256) {
+    const float s = 1.0f / (1.0f + expf(-zr[e]));
+    scores[e] = s;
+    choice[e] = s + correction[e];
+  }
+  __syncthreads();
+  if (tid >= 64) return;
+  const float neg_inf = -__builtin_inff();
+  // the largest of the lanes' candidates (value, number), ties to the lower number; number -1: none
+  auto best_of_lanes = [&](float v, int e) {
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ov = __shfl_xor(v, off, 64);
+      const int oe = __shfl_xor(e, off, 64);
+      if (oe >= 0 && (e < 0 || ov > v || (ov == v && oe < e))) { v = ov; e = oe; }
+    }
+    return e;
+  };
+  unsigned long long open_groups = ~0ull;
+  const int per_group = n_experts / n_groups;
+  if (keep_groups < n_groups) {
+    float sum = neg_inf;
+    if (lane < n_groups) {            // a group a lane (at most 64)
+      float first = neg_inf, second = neg_inf;
+      for (int e = lane * per_group; e < (lane + 1) * per_group; ++e) {
+        const float v = choice[e];
+        if (v > first) { second = first; first = v; }
+        else if (v > second) second = v;
+      }
+      sum = per_group > 1 ? first + second : first;
+    }
+    open_groups = 0ull;
+    for (int k = 0; k < keep_groups; ++k) {
+      const int g = best_of_lanes(sum, (lane < n_groups && !((open_groups >> lane) & 1ull)) ? lane : -1);
+      if (g >= 0) open_groups |= 1ull << g;
+    }
+  }
+  float sum = 0.0f, mine = 0.0f;       // the score of choice number `lane`
+  int my_id = 0;
+  for (int k = 0; k < top; ++k) {
+    float bv = neg_inf;
+    int be = -1;
+    for (int e = lane; e < n_experts; e += 64) {
+      if (!((open_groups >> (e / per_group)) & 1ull)) continue;
+      const float v = choice[e];
+      if (v == neg_inf) continue;      // taken
+      if (be < 0 || v > bv) { be = e; bv = v; }
+    }
+    int e = best_of_lanes(bv, be);
+    if (e < 0) e = 0;                  // (scores that are no numbers)
+    if (lane == (e & 63)) choice[e] = neg_inf;      // only this lane reads it again
+    const float s = scores[e];
+    sum += s;
+    if (lane == k) { mine = s; my_id = e; }
+  }
+  if (lane < top) {
+    ids[size_t(r) * top + lane] = my_id;
+    weights[size_t(r) * (top + 1) + lane] = mine / (sum + 1e-20f) * score_scale;
+  }
+}
+
 template <typename TX>
 __global__ void __launch_bounds__(256)
 moe_router_kernel(int32_t *__restrict__ ids, float *__restrict__ weights, const TX *__restrict__ h,
                   const float *__restrict__ w, int n_rows, int n_in, int n_experts, int top, int has_gate, int score_kind,
-                  float score_scale, int n_groups, int keep_groups) {
-  extern __shared__ float zs[];                 // [n_z] scores, then [4][8] the waves' sums of a pass
+                  float score_scale, int n_groups, int keep_groups, const float *__restrict__ correction) {
+  extern __shared__ float zs[];                 // [n_z] scores, then [4][8] the waves' sums of a pass, then what a choice by corrected scores keeps
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int r = blockIdx.x;
   const int n_z = n_experts + (has_gate ? 1 : 0);
@@ -150,6 +220,11 @@ moe_router_kernel(int32_t *__restrict__ ids, float *__restrict__ weights, const 
     __syncthreads();
     if (tid < 8 && e0 + tid < n_z) z[e0 + tid] = ((part[tid] + part[8 + tid]) + part[16 + tid]) + part[24 + tid];
     __syncthreads();
+  }
+  if (score_kind == 3) {
+    route_row_corrected(ids, weights, z, correction, part + 32, part + 32 + n_experts, r, n_experts, top, score_scale, n_groups, keep_groups);
+    if (tid == 0) weights[size_t(r) * (top + 1) + top] = has_gate ? 1.0f / (1.0f + expf(-z[n_experts])) : 0.0f;
+    return;
   }
   if (tid == 0) route_row(ids, weights, z, r, n_experts, top, has_gate, score_kind, score_scale, n_groups, keep_groups);
 }
@@ -254,23 +329,37 @@ extern "C" int sb_moe_router_scored(int32_t *ids, float *weights, const void *h,
                                stream);
 }
 
+extern "C" int sb_moe_router_corrected(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows,
+                                     int n_in, int n_experts, int top, int has_gate, int score_kind, float score_scale,
+                                     int n_groups, int keep_groups, const float *correction, void *stream);
 extern "C" int sb_moe_router_grouped(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows,
                                      int n_in, int n_experts, int top, int has_gate, int score_kind, float score_scale,
                                      int n_groups, int keep_groups, void *stream) {
+  SB_REQUIRE(score_kind <= 2, "sb_moe_router: unknown kind of score %d", score_kind);
+  return sb_moe_router_corrected(ids, weights, h, h_dtype, w, n_rows, n_in, n_experts, top, has_gate, score_kind, score_scale, n_groups,
+                                 keep_groups, nullptr, stream);
+}
+
+// The same with score_kind 3: sigmoid scores, chosen by score + correction[e] (f32 [n_experts]); a group's score is the sum
+// of its two largest choice scores; the weights are score_scale * score / (the chosen scores' sum + 1e-20).
+extern "C" int sb_moe_router_corrected(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows,
+                                     int n_in, int n_experts, int top, int has_gate, int score_kind, float score_scale,
+                                     int n_groups, int keep_groups, const float *correction, void *stream) {
   SB_REQUIRE(ids && weights && h && w, "sb_moe_router: null pointer");
-  SB_REQUIRE(score_kind >= 0 && score_kind <= 2, "sb_moe_router: unknown kind of score %d", score_kind);
+  SB_REQUIRE(score_kind >= 0 && score_kind <= 3, "sb_moe_router: unknown kind of score %d", score_kind);
   SB_REQUIRE(check_groups(n_experts, top, n_groups, keep_groups) == 0, "sb_moe_router: %d of %d groups do not fit %d experts and %d choices",
              keep_groups, n_groups, n_experts, top);
+  SB_REQUIRE(score_kind != 3 || correction, "sb_moe_router: corrected scores need their correction");
   SB_REQUIRE(n_rows >= 0 && n_in > 0 && n_experts > 0 && top > 0 && top <= n_experts && sb::valid_dtype(h_dtype),
              "sb_moe_router: bad sizes rows=%d in=%d experts=%d top=%d", n_rows, n_in, n_experts, top);
   SB_SUPPORT(top <= kMaxTop && n_experts < 2048, "sb_moe_router: %d choices of %d experts are more than %d of 2047", top,
              n_experts, kMaxTop);
   if (n_rows == 0) return SB_OK;
   hipStream_t s = (hipStream_t)stream;
-  const size_t lds = size_t(n_experts + 1 + 32) * sizeof(float);
+  const size_t lds = size_t(n_experts + 1 + 32 + (score_kind == 3 ? 2 * n_experts : 0)) * sizeof(float);
   const unsigned blocks = n_rows;
-  if (h_dtype == SB_F32) moe_router_kernel<float><<<blocks, 256, lds, s>>>(ids, weights, (const float *)h, w, n_rows, n_in, n_experts, top, has_gate, score_kind, score_scale, n_groups, keep_groups);
-  else moe_router_kernel<bf16_t><<<blocks, 256, lds, s>>>(ids, weights, (const bf16_t *)h, w, n_rows, n_in, n_experts, top, has_gate, score_kind, score_scale, n_groups, keep_groups);
+  if (h_dtype == SB_F32) moe_router_kernel<float><<<blocks, 256, lds, s>>>(ids, weights, (const float *)h, w, n_rows, n_in, n_experts, top, has_gate, score_kind, score_scale, n_groups, keep_groups, correction);
+  else moe_router_kernel<bf16_t><<<blocks, 256, lds, s>>>(ids, weights, (const bf16_t *)h, w, n_rows, n_in, n_experts, top, has_gate, score_kind, score_scale, n_groups, keep_groups, correction);
   return sb::check_launch("sb_moe_router");
 }
 

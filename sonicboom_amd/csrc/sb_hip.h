@@ -497,6 +497,9 @@ int sb_random_normal(void *out, int out_kind, uint64_t n, uint64_t first, uint64
  * sb_moe_route_grouped / sb_moe_router_grouped: score_kind 0 softmax over the chosen, 1 sigmoid, 2 softmax
  *   over all experts (weights not renormalized); experts in n_groups equal groups of neighbours of which
  *   the keep_groups with the largest best score can be chosen from.
+ * sb_moe_router_corrected: also score_kind 3, sigmoid scores chosen by score + correction[e], a group's score the sum of
+ *   its two largest choice scores, weights score_scale * score / (the chosen scores' sum + 1e-20).
+ * sb_attention_chunked: with chunk > 0 (window 0) position p sees the keys from chunk * (p / chunk) on.
  * The experts' products' `gated`: 0 as it is, 1 and 2 pairs, 3 one matrix row an output and max(z, 0)^2. */
 int sb_rmsnorm_pair(void *y1, void *y2, int out_dtype, const float *x, int x_stride, const void *w1, const void *w2,
                     int w_dtype, int n_rows, int width, float eps, void *stream);
@@ -528,6 +531,14 @@ int sb_moe_route_grouped(int32_t *ids, float *weights, const float *z, int n_row
 int sb_moe_router_grouped(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows, int n_in,
                           int n_experts, int top, int has_gate, int score_kind, float score_scale, int n_groups,
                           int keep_groups, void *stream);
+int sb_moe_router_corrected(int32_t *ids, float *weights, const void *h, int h_dtype, const float *w, int n_rows, int n_in,
+                            int n_experts, int top, int has_gate, int score_kind, float score_scale, int n_groups,
+                            int keep_groups, const float *correction, void *stream);
+int sb_attention_chunked(void *out, const void *q, int act_dtype, int q_stride, const void *k_cache, const void *v_cache,
+                         int cache_dtype, const int32_t *page_table, int max_pages, int n_pages_total,
+                         const int32_t *row_pos, const int32_t *row_seq, int n_rows, int heads_q, int heads_kv, int head_dim,
+                         int v_dim, float scale, int window, float softcap, int sink, const float *sink_scores,
+                         const float *gate, int gate_stride, int gate_per_head, int chunk, void *stream);
 
 /* ---- the pass that ends a block of branches, and the layer norm (csrc/join.hip) -------------------
  * sb_join: out[r,:] = base[r,:] + sum_b scale_b N_b(sum of branch b's slices) + vec, for up to three branches
@@ -548,7 +559,8 @@ int sb_layernorm(void *y, int out_dtype, const float *x, const void *w, int w_dt
  *   as sb_log_decay makes it from inner f32 [rows, rank] (up f32 [rank, heads * D], bias f32 [heads * D]), or one number
  *   a head (decay f32 [heads]).  With inv_freq the pairs (i, i + rot_dims / 2) of q and k turn first; q and k
  *   are multiplied by q_scale and k_scale.  q, k, v, g: parts of f32 rows that lie row_stride apart (inner: inner_stride),
- *   in n_slices slices slice_stride numbers apart that are added here in ascending order.
+ *   in n_slices slices slice_stride numbers apart that are added here in ascending order.  act_in: q, k and v are the
+ *   silu of what is read; plain: out is o itself, float32 (g may be NULL).
  * sb_log_decay: out = rate * log(sigmoid(a w + bias)), w f32 [rank, width].
  * sb_decay_chunks: the same scan over runs of sb_decay_chunk_rows(D) rows (chunks int32 [n_chunks, 4], sequence after
  *   sequence, each sequence's runs full but its last) on the matrix cores in float32; q and k turn by `angles` f32
@@ -561,16 +573,64 @@ int sb_decay_scan(void *out, int out_dtype, int out_stride, const float *q, cons
                   const float *up, const float *bias, int rank, float rate, const float *decay, const float *inv_freq,
                   int rot_dims, const int32_t *row_pos, float q_scale, float k_scale, const void *w, int w_dtype, float eps,
                   float *state, const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E,
-                  void *stream);
+                  int act_in, int plain, void *stream);
 int sb_decay_chunk_rows(int D);
 int sb_angle_table(float *out, const int32_t *row_pos, const float *inv_freq, int n_rows, int half, void *stream);
 int sb_decay_chunks(void *out, int out_dtype, int out_stride, const float *q, const float *k, const float *v, const float *g,
                     int row_stride, const float *log_decay, int ld_stride, const float *decay, const float *angles, int half,
                     float q_scale, float k_scale, const void *w, int w_dtype, float eps, float *state,
                     const int32_t *cu_rows, const int32_t *slots, int n_seqs, int heads, int D, int E, const int32_t *chunks,
-                    int n_chunks, int chunk_rows, float *part, float *part_decay, void *stream);
+                    int n_chunks, int chunk_rows, float *part, float *part_decay, int act_in, int plain, void *stream);
 int sb_log_decay(float *out, int out_stride, const float *a, int a_stride, const float *w, const float *bias, int n_rows,
                  int rank, int width, float rate, void *stream);
+
+/* ---- a residual of several streams that mix (csrc/streams.hip) -----------------------------------------
+ * A row of x is `streams` rows of `width` float32 numbers X_1 .. X_S side by side.
+ * sb_streams_embed: all of them table[id].
+ * sb_streams_join: y = sum_i part_scales[i] (* part_ws[i][r * part_w_strides[i]]) parts[i][r * part_strides[i] ..] + vec, then
+ *   X_t <- sum_s mix[s][t] X_s + out[t] y from the old streams, then (h not NULL) h = r(sum_t in[t] X_t) * w, r the division
+ *   by the root mean square with eps inside the root.  The arrays of parts are host arrays.
+ * sb_streams_read: h alone, of the rows named by `rows` (NULL: all), in NULL: the sum of the streams.
+ * few != 0: up to 64 rows take wider blocks (a row's sums are then ordered otherwise). */
+int sb_streams_max(void);
+int sb_streams_max_parts(void);
+int sb_streams_embed(float *x, const void *table, int table_dtype, const int32_t *ids, int n_rows, int streams, int width, int vocab,
+                     void *stream);
+int sb_streams_join(float *x, const void *const *parts, const int *part_strides, const float *part_scales, const void *const *part_ws,
+                    const int *part_w_strides, int n_parts, const void *vec, int vec_dtype, const float *mix, const float *out,
+                    const float *in, void *h, int h_dtype, const void *w, int w_dtype, float eps, int n_rows, int streams, int width,
+                    int few, void *stream);
+int sb_streams_read(void *h, int h_dtype, const float *x, const int32_t *rows, const float *in, const void *w, int w_dtype, float eps,
+                    int n_rows, int streams, int width, int few, void *stream);
+
+/* ---- norms over a whole projection (csrc/rownorm.hip) ----------------------------------------------------
+ * sb_rownorm_kv_store: from f32 rows [q: heads_q x dk | k: heads_kv x dk | v: heads_kv x dv] (in n_slices slices slice_stride
+ *   numbers apart, added here): all of q, and all of k, divided by its root mean square and multiplied by a weight as long
+ *   as it, then turned by head (pairs (i, i + rot_dims / 2)); q out, k and v into the pages of the rows' positions.
+ * sb_rownorm_gate: out = o / rms(o) * w * sigmoid(g). */
+int sb_rownorm_kv_store(void *q_out, int q_dtype, const float *qkv, int row_stride, int n_slices, size_t slice_stride, const void *q_w,
+                        const void *k_w, int w_dtype, float eps, const float *inv_freq, int rot_dims, const int32_t *row_pos,
+                        const int32_t *row_seq, void *k_cache, void *v_cache, int cache_dtype, const int32_t *page_table,
+                        int max_pages, int n_pages, int n_rows, int heads_q, int heads_kv, int dk, int dv, void *stream);
+int sb_rownorm_gate(void *out, int out_dtype, const float *o, const void *w, int w_dtype, float eps, const float *g, int g_stride,
+                    int n_slices, size_t slice_stride, int n_rows, int width, void *stream);
+
+/* ---- a gated linear recurrence behind a short convolution (csrc/gated_lru.hip) -----------------------------
+ * u = conv(x + x_bias) + taps_b over time (taps_w f32 [width, taps], the last on the current row); in blocks of `block`
+ *   channels r = sigmoid(ra u + ra_b), i = sigmoid(ri u + ri_b) (ra, ri [width / block, block, block], [out][in]);
+ *   log a = -rate r; S <- a S + sqrt(1 - a^2) i u; out = S gelu(y + y_bias).  state f32 [slots, width]; ring f32
+ *   [slots, taps, width]: the input of position p in row p % taps, zeros for a new sequence.
+ * Every sequence one row: one launch.  Else ab f32 [rows, width, 2] is scratch, and with chunks (int32 [n_chunks, 4], runs of
+ *   up to sb_gated_lru_chunk_rows() rows, sequence after sequence) the chunked form runs: folded f32 [n_chunks, width, 2]. */
+int sb_gated_lru_max_taps(void);
+int sb_gated_lru_max_block(void);
+int sb_gated_lru_chunk_rows(void);
+int sb_gated_lru_chunked_ok(int m, int w_dtype);
+int sb_gated_lru(void *out, int out_dtype, const float *x, const float *y, int row_stride, int n_slices, size_t slice_stride,
+                 const float *x_bias, const float *y_bias, const float *taps_w, const float *taps_b, int taps, const void *ra,
+                 const void *ri, int w_dtype, const float *ra_b, const float *ri_b, const float *rate, float *state, float *ring,
+                 const int32_t *row_pos, const int32_t *row_seq, const int32_t *cu_rows, const int32_t *slots, int n_rows, int n_seqs,
+                 int width, int block, float *ab, const int32_t *chunks, int n_chunks, float *folded, void *stream);
 
 #ifdef __cplusplus
 }

@@ -81,7 +81,7 @@ class DecoderModel:
                 cs = mixer.cache_spec()
                 if cs is None:
                     raise ValueError(f"order entry {i} names cache {e.cache} but its mixer keeps no keys")
-                need = cs.key()          # (kv heads, head size, window, values' size), or ("rows", shape, window)
+                need = cs.key()          # (kv heads, head size, window, values' size[, chunk]), or ("rows", shape, window)
                 have = self.cache_specs.get(e.cache)
                 if have is not None and have[:2] + have[3:] != need[:2] + need[3:]:
                     raise ValueError(f"order entry {i} uses cache {e.cache} whose heads (or rows) differ from its own")

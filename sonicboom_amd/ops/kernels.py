@@ -1293,12 +1293,14 @@ def headnorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: Optiona
 def attention_capped_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, page_table: torch.Tensor,
                            row_pos: torch.Tensor, row_seq: torch.Tensor, heads_q: int, heads_kv: int, head_dim: int,
                            v_dim: int, scale: float, window: int, softcap: float, sink: bool,
-                           sink_scores: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                           sink_scores: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None,
+                           chunk: int = 0) -> torch.Tensor:
     """Attention of rows ``q`` [n, hq*hd] over the cache by the plain kernel, values of ``v_dim``,
     scores capped as softcap tanh(s / softcap) (0: not), with ``sink`` one more key of score 0
     without a value in every softmax (``sink_scores`` float32 [hq]: of the head's own score instead); [n, hq*v_dim].
     ``gate`` float32 [n, hq*v_dim] (a view of wider rows is fine): the result times sigmoid(gate); [n, hq]: every
-    number of a head times the head's one."""
+    number of a head times the head's one.  ``chunk`` > 0 (and no window): position p sees the keys from
+    chunk * (p // chunk) on."""
     _dev(q, k_cache, v_cache, page_table, row_pos, row_seq, sink_scores)
     _check_sink(sink, sink_scores, heads_q)
     g_stride, per_head = _check_gate(gate, q.shape[0], heads_q, v_dim)
@@ -1308,11 +1310,11 @@ def attention_capped_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
     _check_cache_kv(k_cache, v_cache, heads_kv, head_dim, v_dim)
     _check_rows(row_pos, row_seq, page_table, n)
     out = torch.empty((n, heads_q * v_dim), dtype=q.dtype, device=q.device)
-    check(library.core().sb_attention_sink(
+    check(library.core().sb_attention_chunked(
         _p(out), _p(q), _dt(q), q.shape[1], _p(k_cache), _p(v_cache), _dt(k_cache), _p(page_table),
         page_table.shape[1], k_cache.shape[0], _p(row_pos), _p(row_seq), n, heads_q, heads_kv, head_dim, v_dim,
         float(scale), int(window), float(softcap), 1 if sink else 0, _p(sink_scores), _p(gate), g_stride, per_head,
-        _stream()))
+        int(chunk), _stream()))
     return out
 
 
@@ -1428,16 +1430,16 @@ def moe_product(x: torch.Tensor, w: MoEWeight, plan: MoEPlan, x_div: int, out_dt
 def attention_capped(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, page_table: torch.Tensor, ctx,
                      heads_q: int, heads_kv: int, head_dim: int, v_dim: int, scale: float, window: int,
                      softcap: float, sink: bool, fast: bool = True, sink_scores: Optional[torch.Tensor] = None,
-                     gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                     gate: Optional[torch.Tensor] = None, chunk: int = 0) -> torch.Tensor:
     """Attention of a step's rows over the cache with values of their own size, capped scores and a
     sink (see :func:`attention_capped_plain`).  bfloat16 with key and value sizes in steps of 16
     runs on the matrix cores; everything else takes the plain kernel."""
     if fast and capped_attention_mfma_ok(q.dtype, k_cache.dtype, head_dim, v_dim):
         return attention_capped_mfma(q, k_cache, v_cache, page_table, ctx.row_pos, ctx.row_tiles(CAPPED_ROW_TILE),
                                      heads_q, heads_kv, head_dim, v_dim, scale, window, softcap, sink,
-                                     sink_scores=sink_scores, gate=gate)
+                                     sink_scores=sink_scores, gate=gate, key_chunk=chunk)
     return attention_capped_plain(q, k_cache, v_cache, page_table, ctx.row_pos, ctx.row_seq, heads_q, heads_kv,
-                                  head_dim, v_dim, scale, window, softcap, sink, sink_scores, gate)
+                                  head_dim, v_dim, scale, window, softcap, sink, sink_scores, gate, chunk)
 
 
 CAPPED_ROW_TILE = 16        # rows of a run that a block of the matrix-core kernel takes (sb_cattn_tile_rows)
@@ -1453,8 +1455,8 @@ def attention_capped_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch
                           row_pos: torch.Tensor, tiles: torch.Tensor, heads_q: int, heads_kv: int, head_dim: int,
                           v_dim: int, scale: float, window: int, softcap: float, sink: bool,
                           chunks: Optional[int] = None, sink_scores: Optional[torch.Tensor] = None,
-                          gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """The matrix-core form of :func:`attention_capped_plain`.  ``tiles`` int32 [n, 4]: the rows in
+                          gate: Optional[torch.Tensor] = None, key_chunk: int = 0) -> torch.Tensor:
+    """The matrix-core form of :func:`attention_capped_plain` (``key_chunk``: its ``chunk``).  ``tiles`` int32 [n, 4]: the rows in
     runs of up to 16 consecutive rows of one sequence.  ``chunks``: over how many blocks a run's
     pages are shared out (None: chosen from the shapes alone, so that a recorded step replays)."""
     _dev(q, k_cache, v_cache, page_table, row_pos, tiles, sink_scores)
@@ -1474,20 +1476,23 @@ def attention_capped_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch
     n_tiles, max_pages = tiles.shape[0], page_table.shape[1]
     group = heads_q // heads_kv
     blocks = max(1, n_tiles * heads_kv * ((group + 3) // 4))
+    # the pages a tile's rows can touch: all of a sequence, or those of a window or a chunk and a tile
+    span = key_chunk or window
+    pages = min(max_pages, (span + CAPPED_ROW_TILE - 1 + 2 * PAGE - 2) // PAGE) if span else max_pages
     if chunks is None:
-        chunks = max(1, min(max_pages, CAPPED_SPLIT_BLOCKS // blocks))
-    chunk_pages = (max_pages + chunks - 1) // chunks
-    chunks = (max_pages + chunk_pages - 1) // chunk_pages
+        chunks = max(1, min(pages, CAPPED_SPLIT_BLOCKS // blocks))
+    chunk_pages = (pages + chunks - 1) // chunks
+    chunks = (pages + chunk_pages - 1) // chunk_pages
     part_o = part_ml = None
     if chunks > 1:
         part_o = torch.empty((chunks, n, heads_q, v_dim), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((chunks, n, heads_q, 2), dtype=torch.float32, device=q.device)
     out = torch.empty((n, heads_q * v_dim), dtype=torch.bfloat16, device=q.device)
     lib = library.capped_attention_library(head_dim, v_dim)
-    check(lib.sb_cattn_sink_bf16(_p(out), _p(q), _p(k_cache), _p(v_cache), _p(page_table), max_pages, k_cache.shape[0],
-                                 _p(row_pos), _p(tiles), n_tiles, n, heads_q, heads_kv, float(scale), int(window),
-                                 float(softcap), 1 if sink else 0, chunks, chunk_pages, _p(part_o), _p(part_ml), None, None, 0,
-                                 _p(sink_scores), _p(gate), g_stride, per_head, _stream()),
+    check(lib.sb_cattn_chunked_bf16(_p(out), _p(q), _p(k_cache), _p(v_cache), _p(page_table), max_pages, k_cache.shape[0],
+                                    _p(row_pos), _p(tiles), n_tiles, n, heads_q, heads_kv, float(scale), int(window),
+                                    float(softcap), 1 if sink else 0, chunks, chunk_pages, _p(part_o), _p(part_ml), None, None, 0,
+                                    _p(sink_scores), _p(gate), g_stride, per_head, int(key_chunk), _stream()),
           lib, "sb_cattn_last_error")
     return out
 
@@ -1518,19 +1523,26 @@ def moe_route(z: torch.Tensor, n_experts: int, top: int, has_gate: bool, score: 
 
 
 def moe_router(h: torch.Tensor, w: torch.Tensor, n_experts: int, top: int, has_gate: bool, score: str = "softmax_chosen",
-               score_scale: float = 1.0, groups: int = 1, keep_groups: int = 1):
+               score_scale: float = 1.0, groups: int = 1, keep_groups: int = 1, correction: Optional[torch.Tensor] = None):
     """The router in one launch: z = h w^T in float32 (``w`` float32 [n_experts (+ 1 with
-    ``has_gate``), width], ``h`` rows of either type), then what :func:`moe_route` gives."""
-    _dev(h, w)
+    ``has_gate``), width], ``h`` rows of either type), then what :func:`moe_route` gives.  ``score``
+    "sigmoid_corrected" with ``correction`` float32 [n_experts]: the scores are s = sigmoid(z), the largest
+    s + correction are chosen, a group's score is the sum of its two largest of them, and the weights are
+    ``score_scale`` s / (the sum of the chosen s + 1e-20)."""
+    _dev(h, w, correction)
+    if (score == "sigmoid_corrected") != (correction is not None):
+        raise KernelLibraryError("corrected scores, and no others, take a correction")
+    if correction is not None:
+        _f32_vec(correction, n_experts, "corrections")
     if w.dtype != torch.float32 or w.dim() != 2 or h.dim() != 2 or h.shape[1] != w.shape[1] \
             or w.shape[0] != n_experts + (1 if has_gate else 0):
         raise KernelLibraryError(f"the router's matrix must be float32 [{n_experts + (1 if has_gate else 0)}, {h.shape[-1]}]")
     n = h.shape[0]
     ids = torch.empty((n, top), dtype=torch.int32, device=h.device)
     weights = torch.empty((n, top + 1), dtype=torch.float32, device=h.device)
-    check(library.core().sb_moe_router_grouped(_p(ids), _p(weights), _p(h), _dt(h), _p(w), n, h.shape[1], int(n_experts),
-                                               int(top), 1 if has_gate else 0, ROUTER_SCORES[score], float(score_scale),
-                                               int(groups), int(keep_groups), _stream()))
+    check(library.core().sb_moe_router_corrected(_p(ids), _p(weights), _p(h), _dt(h), _p(w), n, h.shape[1], int(n_experts),
+                                                 int(top), 1 if has_gate else 0, ROUTER_SCORES[score], float(score_scale),
+                                                 int(groups), int(keep_groups), _p(correction), _stream()))
     return ids, weights
 
 
@@ -1568,7 +1580,7 @@ def moe_product_plain(x: torch.Tensor, w: torch.Tensor, ids: Optional[torch.Tens
 
 
 # ---- short convolutions over time, recurrences with a matrix state, attention with shared weights ----
-ROUTER_SCORES = {"softmax_chosen": 0, "sigmoid": 1, "softmax_all": 2}      # score_kind of sb_moe_route_grouped
+ROUTER_SCORES = {"softmax_chosen": 0, "sigmoid": 1, "softmax_all": 2, "sigmoid_corrected": 3}      # score_kind of sb_moe_router_corrected
 EXPERT_PAIRS = {"swish_clamp": 1, "silu": 2}             # `gated` of the experts' products: pairs of a gate and an up row
 EXPERT_SINGLES = {"relu_sq": 3}                          # the same argument for experts without a gate: one row an output
 
@@ -1967,7 +1979,8 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
                dim: int, v_dim: int, eps: float, out_dtype: torch.dtype, log_decay: Optional[torch.Tensor] = None,
                decay: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, q_scale: float = 1.0,
                k_scale: float = 1.0, inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0,
-               chunks: Optional[torch.Tensor] = None, angles: Optional[torch.Tensor] = None, decay_from=None) -> torch.Tensor:
+               chunks: Optional[torch.Tensor] = None, angles: Optional[torch.Tensor] = None, decay_from=None,
+               act_in: bool = False) -> torch.Tensor:
     """S = alpha S + k v^T, o = S^T q per head over every sequence's rows of the step, from ``state`` float32
     [slots, heads, dim, v_dim], which moves on; returns o / rms(o) (* weight) * silu(g) [n, heads*v_dim] in ``out_dtype``.
 
@@ -1976,7 +1989,8 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
     exponential of ``log_decay`` float32 [n, heads*dim], or of what :func:`log_decay` makes of ``decay_from`` (its
     arguments: the walk makes it in its own kernel), or one number a head, ``decay`` float32 [heads].  ``inv_freq``: the
     pairs (i, i + rot_dims/2) of every head of q and k turn by position * inv_freq[i]; then q and k are multiplied by
-    their scales.
+    their scales.  ``act_in``: q, k and v are the silu of what is given.  ``g`` None: the result is o itself, float32,
+    neither normed nor gated.
 
     ``chunks`` int32 [n, 4]: the step's rows in runs of :func:`decay_chunk_rows` rows; the scan then takes its chunked form
     (float32 throughout; it orders its sums otherwise than the walk, from which it differs by rounding), and turns by
@@ -1993,9 +2007,13 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
             raise KernelLibraryError(f"{what} must be float32 rows [{n}, {width}] on the GPU, not {tuple(shape)}")
         if len(shape) != len(q_shape) or (n > 1 and stride[-2] != row_stride) or (n_slices > 1 and (shape[0] != n_slices or stride[0] != slice_stride)):
             raise KernelLibraryError("queries, keys, values, gates and a decay's inner numbers must be parts of the same rows")
+    plain = g is None
+    if plain and (out_dtype != torch.float32 or weight is not None):
+        raise KernelLibraryError("a scan without a gate gives float32 results that are not normed")
     for t, width, what in ((q, heads * dim, "queries"), (k, heads * dim, "keys"), (v, heads * v_dim, "values"),
                            (g, heads * v_dim, "gates")):
-        part_of_rows(t, width, what)
+        if t is not None:
+            part_of_rows(t, width, what)
     _dev(state, log_decay, decay, weight, inv_freq, ctx.cu_rows, ctx.slots, ctx.row_pos)
     if state.dtype != torch.float32 or tuple(state.shape[1:]) != (heads, dim, v_dim):
         raise KernelLibraryError(f"the state must be float32 [slots, {heads}, {dim}, {v_dim}]")
@@ -2048,12 +2066,213 @@ def decay_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tenso
             log_decay.stride(0) if log_decay is not None else 0, _p(decay), _p(angles), rot_dims // 2 if angles is not None else 0,
             float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
             _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _p(chunks), n_chunks, decay_chunk_rows(dim), _p(part),
-            _p(part_decay), _stream()))
+            _p(part_decay), 1 if act_in else 0, 1 if plain else 0, _stream()))
         return out
     check(library.core().sb_decay_scan(
         _p(out), _dt(out), heads * v_dim, _p(q), _p(k), _p(v), _p(g), row_stride, n_slices, slice_stride, _p(log_decay),
         log_decay.stride(0) if log_decay is not None else 0, _p(inner), inner.stride(-2) if inner is not None else 0,
         _p(up) if inner is not None else None, _p(bias) if inner is not None else None, rank, float(rate), _p(decay), _p(inv_freq), int(rot_dims), _p(ctx.row_pos),
         float(q_scale), float(k_scale), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(state),
-        _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, _stream()))
+        _p(ctx.cu_rows), _p(ctx.slots), ctx.n_seqs, heads, dim, v_dim, 1 if act_in else 0, 1 if plain else 0, _stream()))
+    return out
+
+
+# --------------------------------------------------------------------------
+# a residual of several streams; norms over a whole projection; a gated linear recurrence
+# --------------------------------------------------------------------------
+def streams_max() -> int:
+    """Streams a residual can have at most."""
+    return int(library.core().sb_streams_max())
+
+
+def streams_embed(table: torch.Tensor, ids: torch.Tensor, streams: int) -> torch.Tensor:
+    """Rows of ``table`` [vocab, width] named by ``ids`` [n], ``streams`` times side by side: float32 [n, streams * width]."""
+    _dev(table, ids)
+    if table.dim() != 2:
+        raise KernelLibraryError("embedding table must be [vocab, width]")
+    n = ids.numel()
+    _i32(ids, n, "token ids")
+    vocab, width = table.shape
+    x = torch.empty((n, streams * width), dtype=torch.float32, device=table.device)
+    check(library.core().sb_streams_embed(_p(x), _p(table), _dt(table), _p(ids), n, int(streams), width, vocab, _stream()))
+    return x
+
+
+def _check_streams(x, streams, weight):
+    if x.dtype != torch.float32 or x.dim() != 2 or x.shape[1] % streams:
+        raise KernelLibraryError(f"a residual of {streams} streams must be float32 [rows, {streams} * width]")
+    width = x.shape[1] // streams
+    if weight is not None and weight.numel() != width:
+        raise KernelLibraryError(f"the norm's weight has {weight.numel()} elements, a stream has {width}")
+    return width
+
+
+def streams_read(x: torch.Tensor, streams: int, read: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps: float,
+                 out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """The RMS norm of sum_s read[s] X_s (``read`` float32 [streams]; None: the sum of the streams) of the rows of ``x``
+    float32 [n, streams * width], or of those ``rows`` picks."""
+    _dev(x, read, weight, rows)
+    width = _check_streams(x, streams, weight)
+    if read is not None:
+        _f32_vec(read, streams, "multipliers of the streams")
+    n = x.shape[0] if rows is None else rows.numel()
+    if rows is not None:
+        _i32(rows, n, "row index")
+    h = torch.empty((n, width), dtype=out_dtype, device=x.device)
+    check(library.core().sb_streams_read(_p(h), _dt(h), _p(x), _p(rows), _p(read), _p(weight), _dt(weight) if weight is not None else 0,
+                                         float(eps), n, int(streams), width, 1 if out_dtype == torch.bfloat16 else 0, _stream()))
+    return h
+
+
+def streams_join(x: torch.Tensor, streams: int, terms, mix: torch.Tensor, out: torch.Tensor, vec: Optional[torch.Tensor] = None,
+                 read: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None, eps: float = 0.0,
+                 act_dtype: torch.dtype = torch.float32) -> Optional[torch.Tensor]:
+    """X_t <- sum_s mix[s, t] X_s + out[t] y in place, y the sum of ``terms`` and of ``vec`` [width]; returns the RMS norm of
+    sum_t read[t] X_t times ``weight`` in ``act_dtype`` when ``read`` is given.
+
+    A term is (part, scale, by_row, weights): float32 [rows, width]; or slices that are added, [slices, rows, width], or
+    with ``by_row`` [rows, slices, width]; ``weights`` float32 [rows, slices] multiplies them (None: ones).
+    ``act_dtype`` bfloat16: few rows may take another block shape than many."""
+    _dev(x, mix, out, vec, read, weight)
+    width = _check_streams(x, streams, weight)
+    n = x.shape[0]
+    _f32_vec(mix, streams * streams, "mixing matrices")
+    _f32_vec(out, streams, "multipliers of the sublayer's result")
+    if vec is not None and vec.numel() != width:
+        raise KernelLibraryError(f"the vector has {vec.numel()} elements, a stream has {width}")
+    ptrs, strides, scales, wptrs, wstrides = [], [], [], [], []
+    for part, scale, by_row, weights in terms:
+        _dev(part)
+        _on_gpu(weights)
+        slices = 1 if part.dim() == 2 else part.shape[1 if by_row else 0]
+        shape = (n, width) if part.dim() == 2 else (n, slices, width) if by_row else (slices, n, width)
+        if part.dtype != torch.float32 or tuple(part.shape) != shape:
+            raise KernelLibraryError(f"a sublayer's result {tuple(part.shape)} does not fit a stream of {(n, width)}")
+        if weights is not None and (weights.dtype != torch.float32 or tuple(weights.shape) != (n, slices) or weights.stride(1) != 1):
+            raise KernelLibraryError(f"multipliers of slices must be float32 [{n}, {slices}]")
+        base, step = part.data_ptr(), width if by_row else n * width
+        for i in range(slices):
+            ptrs.append(base + 4 * step * i)
+            strides.append(slices * width if by_row else width)
+            scales.append(float(scale))
+            wptrs.append(None if weights is None else weights.data_ptr() + 4 * i)
+            wstrides.append(0 if weights is None else weights.stride(0))
+    k = len(ptrs)
+    h = None
+    if read is not None:
+        _f32_vec(read, streams, "multipliers of the streams")
+        h = torch.empty((n, width), dtype=act_dtype, device=x.device)
+    check(library.core().sb_streams_join(
+        _p(x), (ctypes.c_void_p * max(1, k))(*ptrs), (ctypes.c_int * max(1, k))(*strides), (ctypes.c_float * max(1, k))(*scales),
+        (ctypes.c_void_p * max(1, k))(*wptrs), (ctypes.c_int * max(1, k))(*wstrides), k, _p(vec), _dt(vec) if vec is not None else 0,
+        _p(mix), _p(out), _p(read), _p(h), _dt(h) if h is not None else 0, _p(weight), _dt(weight) if weight is not None else 0,
+        float(eps), n, int(streams), width, 1 if act_dtype == torch.bfloat16 else 0, _stream()))
+    return h
+
+
+def _rows_of(t: torch.Tensor, need: int, what: str):
+    """(rows, distance between rows, slices, distance between slices) of float32 rows [n, >= need], a column range of wider
+    rows, or K slices of such."""
+    _on_gpu(t)
+    shape, stride = t.shape, t.stride()
+    if t.dtype != torch.float32 or len(shape) not in (2, 3) or shape[-1] < need or stride[-1] != 1:
+        raise KernelLibraryError(f"{what} must be float32 rows of at least {need} numbers, not {tuple(shape)}")
+    slices, slice_stride = (shape[0], stride[0]) if len(shape) == 3 else (1, 0)
+    return shape[-2], max(stride[-2], need), slices, slice_stride
+
+
+def rownorm_kv_store(qkv: torch.Tensor, q_dtype: torch.dtype, q_weight: torch.Tensor, k_weight: torch.Tensor, eps: float,
+                     row_pos: torch.Tensor, row_seq: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                     page_table: torch.Tensor, heads_q: int, heads_kv: int, head_dim: int, v_dim: int,
+                     inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0) -> torch.Tensor:
+    """From float32 rows [n, heads_q*head_dim + heads_kv*(head_dim + v_dim)] of a stacked product (a column range of wider
+    rows, or K slices, added here): all of q and all of k divided by its root mean square over the row and multiplied by
+    weights as long as they are, then with ``inv_freq`` the pairs (i, i + rot_dims/2) of every head turned by position *
+    inv_freq[i]; returns q in ``q_dtype`` and puts keys and values into the pages of the rows' positions."""
+    _dev(q_weight, k_weight, row_pos, row_seq, k_cache, v_cache, page_table, inv_freq)
+    n, row_stride, slices, slice_stride = _rows_of(qkv, heads_q * head_dim + heads_kv * (head_dim + v_dim), "the stacked product")
+    if q_weight.numel() != heads_q * head_dim or k_weight.numel() != heads_kv * head_dim or q_weight.dtype != k_weight.dtype:
+        raise KernelLibraryError("norms over a whole projection take weights as long as it, of one type")
+    _check_cache_kv(k_cache, v_cache, heads_kv, head_dim, v_dim)
+    _check_rows(row_pos, row_seq, page_table, n)
+    if inv_freq is not None:
+        _f32_vec(inv_freq, rot_dims // 2, "frequencies")
+    q = torch.empty((n, heads_q * head_dim), dtype=q_dtype, device=qkv.device)
+    check(library.core().sb_rownorm_kv_store(
+        _p(q), _dt(q), _p(qkv), row_stride, slices, slice_stride, _p(q_weight), _p(k_weight), _dt(q_weight), float(eps), _p(inv_freq),
+        int(rot_dims), _p(row_pos), _p(row_seq), _p(k_cache), _p(v_cache), _dt(k_cache), _p(page_table), page_table.shape[1],
+        k_cache.shape[0], n, heads_q, heads_kv, head_dim, v_dim, _stream()))
+    return q
+
+
+def rownorm_gate(o: torch.Tensor, weight: Optional[torch.Tensor], eps: float, g: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """o / rms(o) * weight * sigmoid(g) for float32 rows ``o`` [n, width]; ``g``: float32 rows of the same width (a column
+    range of wider rows, or K slices, added here)."""
+    _dev(o, weight)
+    if o.dtype != torch.float32 or o.dim() != 2 or (weight is not None and weight.numel() != o.shape[1]):
+        raise KernelLibraryError("a gated row norm takes float32 rows and a weight as long as they are")
+    width = o.shape[1]
+    n, g_stride, slices, slice_stride = _rows_of(g, width, "the gate")
+    if n != o.shape[0]:
+        raise KernelLibraryError(f"the gate has {n} rows for {o.shape[0]}")
+    out = torch.empty(o.shape, dtype=out_dtype, device=o.device)
+    check(library.core().sb_rownorm_gate(_p(out), _dt(out), _p(o), _p(weight), _dt(weight) if weight is not None else 0, float(eps), _p(g),
+                                         g_stride, slices, slice_stride, n, width, _stream()))
+    return out
+
+
+def gated_lru_chunk_rows() -> int:
+    """The rows of a run of the chunked form of :func:`gated_lru`."""
+    return int(library.core().sb_gated_lru_chunk_rows())
+
+
+def gated_lru_limits():
+    """(taps, channels of a block) that :func:`gated_lru` takes at most."""
+    return int(library.core().sb_gated_lru_max_taps()), int(library.core().sb_gated_lru_max_block())
+
+
+def gated_lru_chunked_ok(block: int, w_dtype: torch.dtype) -> bool:
+    """Whether the chunked form takes blocks of that many channels with weights of that type."""
+    return bool(library.core().sb_gated_lru_chunked_ok(int(block), _DT[w_dtype]))
+
+
+def gated_lru(x: torch.Tensor, y: torch.Tensor, x_bias: torch.Tensor, y_bias: torch.Tensor, taps: torch.Tensor, taps_bias: torch.Tensor,
+              ra: torch.Tensor, ri: torch.Tensor, ra_bias: torch.Tensor, ri_bias: torch.Tensor, rate: torch.Tensor, state: torch.Tensor,
+              ring: torch.Tensor, ctx, out_dtype: torch.dtype, chunks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A gated linear recurrence over the rows of a step: u = conv(x + x_bias) + taps_bias over time (``taps`` float32
+    [width, taps]), r = sigmoid(ra u + ra_bias) and i = sigmoid(ri u + ri_bias) in blocks of channels (``ra``, ``ri``
+    [blocks, m, m]), a = exp(-rate r), S = a S + sqrt(1 - a^2) i u; returns S gelu(y + y_bias) [n, width].
+
+    ``x``, ``y``: float32 columns of the same wider rows, whole or in K slices.  ``state`` float32 [slots, width] and ``ring``
+    float32 [slots, taps, width] (the input of position p in row p % taps) move on.  ``chunks`` int32 [n, 4]: the step's rows
+    in runs of :func:`gated_lru_chunk_rows` rows, for the chunked form."""
+    width, n_taps = taps.shape
+    blocks, m = ra.shape[0], ra.shape[1]
+    _dev(x_bias, y_bias, taps, taps_bias, ra, ri, ra_bias, ri_bias, rate, state, ring, ctx.row_pos, ctx.row_seq, ctx.cu_rows, ctx.slots)
+    n, row_stride, slices, slice_stride = _rows_of(x, width, "the convolution's input")
+    if _rows_of(y, width, "the output's gate") != (n, row_stride, slices, slice_stride):
+        raise KernelLibraryError("the convolution's input and the output's gate must be parts of the same rows")
+    for t, what in ((x_bias, "input biases"), (y_bias, "gate biases"), (taps_bias, "convolution biases"), (ra_bias, "biases"),
+                    (ri_bias, "biases"), (rate, "decay rates")):
+        _f32_vec(t, width, what)
+    if tuple(ra.shape) != (blocks, m, m) or ra.shape != ri.shape or ra.dtype != ri.dtype or blocks * m != width or taps.dtype != torch.float32:
+        raise KernelLibraryError(f"gates of {blocks} blocks of {m} channels and taps {tuple(taps.shape)} do not fit each other")
+    if state.dtype != torch.float32 or tuple(state.shape[1:]) != (width,) or ring.dtype != torch.float32 \
+            or tuple(ring.shape[1:]) != (n_taps, width):
+        raise KernelLibraryError(f"the state must be float32 [slots, {width}] and [slots, {n_taps}, {width}]")
+    _i32(ctx.row_pos, n, "row positions")
+    _i32(ctx.row_seq, n, "row sequences")
+    _i32(ctx.cu_rows, ctx.n_seqs + 1, "first rows")
+    _i32(ctx.slots, ctx.n_seqs, "slots")
+    out = torch.empty((n, width), dtype=out_dtype, device=x.device)
+    n_chunks = _scan_chunks(chunks)
+    ab = folded = None
+    if n_chunks or n != ctx.n_seqs:
+        ab = torch.empty((n, width, 2), dtype=torch.float32, device=x.device)
+    if n_chunks:
+        folded = torch.empty((n_chunks, width, 2), dtype=torch.float32, device=x.device)
+    check(library.core().sb_gated_lru(
+        _p(out), _dt(out), _p(x), _p(y), row_stride, slices, slice_stride, _p(x_bias), _p(y_bias), _p(taps), _p(taps_bias), n_taps, _p(ra),
+        _p(ri), _dt(ra), _p(ra_bias), _p(ri_bias), _p(rate), _p(state), _p(ring), _p(ctx.row_pos), _p(ctx.row_seq), _p(ctx.cu_rows),
+        _p(ctx.slots), n, ctx.n_seqs, width, m, _p(ab), _p(chunks), n_chunks, _p(folded), _stream()))
     return out

@@ -101,12 +101,27 @@ _CORE_SIGNATURES = {
     "sb_decay_scan_max_side": [],
     "sb_decay_scan_max_rank": [],
     "sb_decay_scan": [_P, _I, _I, _P, _P, _P, _P, _I, _I, _Z, _P, _I, _P, _I, _P, _P, _I, _F, _P, _P, _I, _P, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I,
-                      _P],
+                      _I, _I, _P],
     "sb_decay_chunk_rows": [_I],
     "sb_angle_table": [_P, _P, _P, _I, _I, _P],
     "sb_decay_chunks": [_P, _I, _I, _P, _P, _P, _P, _I, _P, _I, _P, _P, _I, _F, _F, _P, _I, _F, _P, _P, _P, _I, _I, _I, _I, _P,
-                        _I, _I, _P, _P, _P],
+                        _I, _I, _P, _P, _I, _I, _P],
     "sb_log_decay": [_P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P],
+    "sb_moe_router_corrected": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P],
+    "sb_attention_chunked": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _P, _I, _I, _I, _P],
+    "sb_streams_max": [],
+    "sb_streams_max_parts": [],
+    "sb_streams_embed": [_P, _P, _I, _P, _I, _I, _I, _I, _P],
+    "sb_streams_join": [_P, _P, _P, _P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _P],
+    "sb_streams_read": [_P, _I, _P, _P, _P, _P, _I, _F, _I, _I, _I, _I, _P],
+    "sb_rownorm_kv_store": [_P, _I, _P, _I, _I, _Z, _P, _P, _I, _F, _P, _I, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+    "sb_rownorm_gate": [_P, _I, _P, _P, _I, _F, _P, _I, _I, _Z, _I, _I, _P],
+    "sb_gated_lru_max_taps": [],
+    "sb_gated_lru_max_block": [],
+    "sb_gated_lru_chunk_rows": [],
+    "sb_gated_lru_chunked_ok": [_I, _I],
+    "sb_gated_lru": [_P, _I, _P, _P, _I, _I, _Z, _P, _P, _P, _P, _I, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P,
+                     _I, _P, _P],
 }
 # Entry points of later kernels; declared when the library has them.
 _OPTIONAL_SIGNATURES = {
@@ -149,6 +164,9 @@ _CAPPED_ATTN_SIGNATURES = {
     # the same, then sink_scores, gate, gate_stride, gate_per_head, stream
     "sb_cattn_sink_bf16": [_P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
                            _P, _I, _I, _P],
+    # the same, then key_chunk, stream
+    "sb_cattn_chunked_bf16": [_P, _P, _P, _P, _P, _I, _I, _P, _P, _I, _I, _I, _I, _F, _I, _F, _I, _I, _I, _P, _P, _P, _P, _I, _P,
+                              _P, _I, _I, _I, _P],
     "sb_cattn_tile_rows": [],
     "sb_cattn_key_dim": [],
     "sb_cattn_value_dim": [],

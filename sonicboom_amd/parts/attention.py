@@ -11,13 +11,14 @@ Every size and switch is a parameter of the spec:
     qkv_bias, out_bias, out_scale (the multiplier of the branch, 1 unless given),
     v_dim (the values' size per head when it is not the keys'), qk_norm (every head of q and k
     divided by its root mean square, eps ``qk_norm_eps`` inside the root, times a weight of the head's
-    size that the heads share), softcap (scores become softcap * tanh(score / softcap); 0: not),
+    size that the heads share, after the rotation; "row": all of q, and all of k, divided by its root mean square
+    over the row and multiplied by a weight as long as it, before the rotation), softcap (scores become softcap * tanh(score / softcap); 0: not),
     sink (one more key of score 0 without a value in every softmax: the weights are
     exp(s_j) / (1 + sum exp(s_j))), value_mix ("first": the values of this step's rows are kept
     for later layers under ``value_mix_key``; "mix": v <- (1 - lam) v + lam v_first with the layer's
     own number lam; what is mixed is what the cache keeps), sink_scores (the sink's score is a number of
     the query head's own, a tensor of heads_q numbers, as it is: weights exp(s_j) / (exp(sink_a) + sum
-    exp(s_j))), out_gate (True: the heads' results side by side times sigmoid(W_g h), number by number, before
+    exp(s_j))), chunk (> 0, no window then: position p sees the keys from chunk * (p // chunk) on), out_gate (True: the heads' results side by side times sigmoid(W_g h), number by number, before
     the output product; "head": head a's result times sigmoid((W_g h)_a), one number a head; W_g is
     stacked under q, k and v), qk_norm_weight (False: the head norms have no weight), given_input (the
     mixer's stacked input matrix is part of a larger one: see ``input_weight`` below)
@@ -35,7 +36,7 @@ import numpy as np
 import torch
 
 from .. import ops
-from .base import KVSpec, Mixer, register_part
+from .base import Joined, KVSpec, Mixer, register_part
 from .linear import Linear
 from .spec import PartSpec, TensorSpec
 
@@ -46,15 +47,16 @@ NAMES = {"q_weight": "q_proj.weight", "k_weight": "k_proj.weight", "v_weight": "
          "sink": "sink", "g_weight": "g"}
 
 HEAD_GATE = "head"           # an output gate of one number a head
+ROW_NORM = "row"             # a norm of q and of k over the whole projection, before the rotation
 
 
 def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_dim: int,
                    position: PartSpec, window: int = 0, scale: Optional[float] = None,
                    qkv_bias: bool = True, out_bias: bool = False, out_scale: float = 1.0,
-                   v_dim: Optional[int] = None, qk_norm: bool = False, qk_norm_eps: float = 0.0,
+                   v_dim: Optional[int] = None, qk_norm=False, qk_norm_eps: float = 0.0,
                    softcap: float = 0.0, sink: bool = False, value_mix: Optional[str] = None,
                    value_mix_key: str = "values", names: Optional[dict] = None, sink_scores: bool = False,
-                   out_gate=False, qk_norm_weight: bool = True, given_input: bool = False) -> PartSpec:
+                   out_gate=False, qk_norm_weight: bool = True, given_input: bool = False, chunk: int = 0) -> PartSpec:
     """``names``: what the file calls a role's tensor after ``prefix``, where that is not what
     ``NAMES`` says."""
     nm = dict(NAMES, **(names or {}))
@@ -72,9 +74,14 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
         tensors["v_bias"] = TensorSpec(prefix + nm["v_bias"], (vw,))
     if out_bias:
         tensors["o_bias"] = TensorSpec(prefix + nm["o_bias"], (width,))
+    if chunk and window:
+        raise ValueError("a mixer sees a window or a chunk of keys, not both")
+    if qk_norm == ROW_NORM and not qk_norm_weight:
+        raise ValueError("a norm over a whole projection has a weight")
     if qk_norm and qk_norm_weight:
-        tensors["q_norm"] = TensorSpec(prefix + nm["q_norm"], (head_dim,), init=(1.0, 0.02))
-        tensors["k_norm"] = TensorSpec(prefix + nm["k_norm"], (head_dim,), init=(1.0, 0.02))
+        q_norm, k_norm = (qw, kw) if qk_norm == ROW_NORM else (head_dim, head_dim)
+        tensors["q_norm"] = TensorSpec(prefix + nm["q_norm"], (q_norm,), init=(1.0, 0.02))
+        tensors["k_norm"] = TensorSpec(prefix + nm["k_norm"], (k_norm,), init=(1.0, 0.02))
     if sink_scores:
         if not sink:
             raise ValueError("scores of a sink belong to a mixer that has one")
@@ -89,7 +96,8 @@ def attention_spec(prefix: str, width: int, heads_q: int, heads_kv: int, head_di
     return PartSpec("mixer", "attention", {
         "width": width, "heads_q": heads_q, "heads_kv": heads_kv, "head_dim": head_dim,
         "window": int(window), "scale": scale, "qkv_bias": qkv_bias, "out_bias": out_bias,
-        "out_scale": float(out_scale), "v_dim": v_dim, "qk_norm": bool(qk_norm), "qk_norm_eps": float(qk_norm_eps),
+        "out_scale": float(out_scale), "v_dim": v_dim, "qk_norm": ROW_NORM if qk_norm == ROW_NORM else bool(qk_norm),
+        "qk_norm_eps": float(qk_norm_eps), "chunk": int(chunk),
         "softcap": float(softcap), "sink": bool(sink), "value_mix": value_mix, "value_mix_key": value_mix_key,
         "sink_scores": bool(sink_scores), "out_gate": HEAD_GATE if out_gate == HEAD_GATE else bool(out_gate),
         "given_input": bool(given_input),
@@ -108,7 +116,7 @@ class Attention(Mixer):
         self.heads_q, self.heads_kv, self.head_dim = int(p["heads_q"]), int(p["heads_kv"]), int(p["head_dim"])
         if self.heads_q % self.heads_kv:
             raise ValueError(f"{self.heads_q} query heads are not a multiple of {self.heads_kv} kv heads")
-        self.window = int(p.get("window") or 0)
+        self.window, self.chunk = int(p.get("window") or 0), int(p.get("chunk") or 0)
         self.position = parts["position"]
         base_scale = p.get("scale")
         if base_scale is None:
@@ -117,7 +125,8 @@ class Attention(Mixer):
         self.q_width = self.heads_q * self.head_dim
         self.kv_width = self.heads_kv * self.head_dim
         self.v_dim = int(p.get("v_dim") or self.head_dim)
-        self.qk_norm = bool(p.get("qk_norm", False))
+        self.row_norm = p.get("qk_norm") == ROW_NORM
+        self.qk_norm = bool(p.get("qk_norm", False)) and not self.row_norm
         self.qk_norm_eps = float(p.get("qk_norm_eps", 0.0))
         self.q_norm, self.k_norm = tensors.get("q_norm"), tensors.get("k_norm")
         self.softcap = float(p.get("softcap", 0.0) or 0.0)
@@ -132,7 +141,7 @@ class Attention(Mixer):
         # whose kernels take them.  With head norms or mixed values one kernel rotates, then norms, mixes and
         # stores; the others rotate and store with the kernel of the plain path.
         self.extended = bool(self.qk_norm or self.softcap or self.sink or self.value_mix or self.v_dim != self.head_dim
-                             or self.out_gate or p.get("given_input"))
+                             or self.out_gate or p.get("given_input") or self.chunk or self.row_norm)
         self.head_norm_path = bool(self.qk_norm or self.value_mix)
         if self.extended:
             tables = self.position.rotary_tables()
@@ -142,9 +151,15 @@ class Attention(Mixer):
             if self.position.rotary_tables() is None:
                 raise ValueError("capped scores, sinks, gates and values of their own size take a rotary position "
                                  "encoding, or none")
-            if self.head_norm_path and p.get("qkv_bias", True):
-                raise ValueError("head norms and mixed values are built for mixers without biases on q, k and v")
-        if rt.fast_kernels and not self.extended:
+            if (self.head_norm_path or self.row_norm) and p.get("qkv_bias", True):
+                raise ValueError("norms of queries and keys and mixed values are built for mixers without biases on q, k and v")
+            if self.row_norm and (self.head_norm_path or self.out_gate or tables[1] is not None or self.position.interleaved
+                                  or getattr(self.position, "magnitude", 1.0) != 1.0):
+                raise ValueError("norms over a whole projection take no rotation, or the rotate-half one by plain "
+                                 "frequencies, no head norms, mixed values or gates")
+        # past the norms and the rotation: the attention kernels of the plain path, where nothing asks for the others
+        self.plain_scores = not (self.softcap or self.sink or self.chunk or self.out_gate or self.v_dim != self.head_dim)
+        if rt.fast_kernels and (not self.extended or (self.row_norm and self.plain_scores)):
             # (groups of one and two heads per kv head take higher tiles on the matrix cores)
             self.row_tile = ops.attention_row_tiles(self.heads_q, self.heads_kv, self.head_dim, rt.act_dtype)
 
@@ -187,7 +202,7 @@ class Attention(Mixer):
         self.input_weight = None
 
     def cache_spec(self) -> KVSpec:
-        return KVSpec(self.heads_kv, self.head_dim, self.window, self.v_dim)
+        return KVSpec(self.heads_kv, self.head_dim, self.window, self.v_dim, self.chunk)
 
     fuses_norm = True
     graph_safe = True     # its launches depend on device buffers only
@@ -203,20 +218,42 @@ class Attention(Mixer):
         """The heads' results (what the output product reads) from the stacked input product's float32 rows
         [rows, q | k | v (| gate)], a column range of wider rows, or, where takes_slices() says so, [slices, rows, ...]
         K slices of them."""
+        if self.row_norm:
+            return self._attend_row_normed(rows, ctx, binding)
         if not self.head_norm_path:
             return self._attend_rotating(None, ctx, binding, rows)
         return self._attend_extended(None, ctx, binding, rows)
 
     def takes_slices(self, ctx) -> bool:
         """Whether from_rows() adds a product's K slices itself."""
-        return self.head_norm_path
+        return self.head_norm_path or self.row_norm
 
     def produce(self, h, ctx, binding):
         """attention(h) in float32 (whole, or in K slices of the output product), for a block that
         adds it up itself."""
         if self.out_scale != 1.0:
             raise ValueError("a mixer that hands its result over has no multiplier of its own")
-        return self.out.raw(self._attend(h, ctx, binding))
+        a = self._attend(h, ctx, binding)
+        part = self.out.partial(a) if self.out.bias is not None else None
+        if part is not None:
+            return Joined(part, bias=self.out.bias)      # the pass that adds the slices adds the bias
+        return self.out.raw(a)
+
+    def _attend_row_normed(self, rows, ctx, binding):
+        rt = self.rt
+        if not binding.writes_cache:
+            raise RuntimeError("this mixer stores the keys and values it reads")
+        page_table = ctx.page_table(binding.group)
+        inv_freq, _, rot_dims = self.position.rotary_tables()
+        q = ops.rownorm_kv_store(rows, rt.act_dtype, self.q_norm, self.k_norm, self.qk_norm_eps, ctx.row_pos, ctx.row_seq,
+                                 binding.k_cache, binding.v_cache, page_table, self.heads_q, self.heads_kv, self.head_dim, self.v_dim,
+                                 inv_freq=inv_freq, rot_dims=rot_dims if inv_freq is not None else 0)
+        if self.plain_scores:
+            return ops.attention(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
+                                 self.head_dim, self.scale, self.window, fast=rt.fast_kernels, row_tile=self.row_tile)
+        return ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
+                                    self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
+                                    fast=rt.fast_kernels, sink_scores=self.sink_scores, chunk=self.chunk)
 
     def _attend_rotating(self, h, ctx, binding, rows=None):
         """The extended path of mixers that rotate (or have no position encoding and no head norms): the plain path's
@@ -243,10 +280,13 @@ class Attention(Mixer):
         gate = qkv[:, self.g_off:self.g_off + self.gate_width] if self.out_gate else None
         a = ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
                                  self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
-                                 fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate)
+                                 fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate, chunk=self.chunk)
         return a
 
     def _attend_extended(self, h, ctx, binding, rows=None):
+        if self.row_norm:
+            rows = self.qkv.partial(h)
+            return self._attend_row_normed(self.qkv(h, torch.float32) if rows is None else rows, ctx, binding)
         if not self.head_norm_path:
             return self._attend_rotating(h, ctx, binding, rows)
         rt = self.rt
@@ -287,7 +327,7 @@ class Attention(Mixer):
             gate = qkv[:, self.g_off:self.g_off + self.gate_width]
         return ops.attention_capped(q, binding.k_cache, binding.v_cache, page_table, ctx, self.heads_q, self.heads_kv,
                                     self.head_dim, self.v_dim, self.scale, self.window, self.softcap, self.sink,
-                                    fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate)
+                                    fast=rt.fast_kernels, sink_scores=self.sink_scores, gate=gate, chunk=self.chunk)
 
     def _attend(self, h, ctx, binding):
         """The heads' results [rows, heads_q * v_dim] in the activation type; keys and values of the

@@ -26,7 +26,7 @@ copy in the activation type, ``ctx`` the step's
                 result (a float32 tensor, K slices of it, a :class:`Branch`, or a list of :class:`Joined`)
                 instead of adding it: blocks that norm a sublayer's output, or join their branches in one
                 pass, need it.
-* **block**     ``mixer`` attribute and ``forward(x, ctx, binding, h=None, next_norm=None)``;
+* **block**     ``mixer`` attribute (and ``ffn``, where it has one) and ``forward(x, ctx, binding, h=None, next_norm=None)``;
                 optionally ``first_norm``, the norm the block starts with (the block before
                 may then hand over ``h`` = first_norm(x) from its last pass), ``state_specs() ->
                 {name: StateSpec}`` for per-sequence state the block itself keeps (it finds it at
@@ -69,15 +69,18 @@ class Runtime:
 class KVSpec:
     """What a mixer keeps per token: keys and values of ``kv_heads`` heads of
     ``head_dim``; ``window`` > 0 when only the last ``window`` keys are read; ``v_dim``: the
-    values' size per head when it is not the keys' (0: the same)."""
+    values' size per head when it is not the keys' (0: the same); ``chunk`` > 0 when a position
+    reads the keys of its own stretch of that many positions only."""
     kv_heads: int
     head_dim: int
     window: int = 0
     v_dim: int = 0
+    chunk: int = 0
 
     def key(self):
-        """(kv heads, head size, window, values' size)"""
-        return (int(self.kv_heads), int(self.head_dim), int(self.window), int(self.v_dim or self.head_dim))
+        """(kv heads, head size, window, values' size[, chunk])"""
+        key = (int(self.kv_heads), int(self.head_dim), int(self.window), int(self.v_dim or self.head_dim))
+        return key + (int(self.chunk),) if self.chunk else key
 
 
 @dataclass(frozen=True)
@@ -118,11 +121,13 @@ class Branch:
 class Joined:
     """What a sublayer hands to a block that joins several branches in one pass: ``scale`` times the sum of
     ``part``'s slices (float32 [rows, width], or [slices, rows, width]), divided by its root mean square and
-    multiplied by ``norm_weight`` first when that is given (``eps`` inside the root)."""
+    multiplied by ``norm_weight`` first when that is given (``eps`` inside the root).  ``bias`` [width], which
+    is neither scaled nor normed, joins as well."""
     part: torch.Tensor
     scale: float = 1.0
     norm_weight: Optional[torch.Tensor] = None
     eps: float = 0.0
+    bias: Optional[torch.Tensor] = None
 
     def term(self):
         return (self.part, self.scale, self.norm_weight is not None, self.norm_weight)

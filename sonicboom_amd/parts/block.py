@@ -21,6 +21,12 @@ mean square is the same, the weights differ); the mixer and the feed-forward the
 one after the other.  Without a second norm both sublayers read the first one's result, x += mixer(h) + ffn(h)
 with h = norm1(x): they hand their results over (``produce``) and one pass adds the slices of all of
 them, norms those that are normed, adds the sum into the stream and leaves what the next block reads.
+
+``streams``: the residual is S streams X_1 .. X_S side by side in a row (hyper-connections).  A sublayer f with its numbers
+in [S], out [S] and mix [S, S] (from, to) reads u = sum_s in_s X_s through its norm and leaves
+X_t <- sum_s mix[s, t] X_s + out_t f(norm(u)), all t from the old streams.  The sublayers hand their results over
+(``produce``); one pass adds the result's slices up, mixes the streams and leaves what the sublayer after it reads, across
+the block's end too.
 """
 from __future__ import annotations
 
@@ -149,6 +155,10 @@ class OutNormBlock(Part):
 
     def _join(self, x, y, norm, copy_dtype):
         """x += norm(y); the new stream in ``copy_dtype`` (x itself when that is float32)."""
+        if isinstance(y, Joined):
+            if y.scale != 1.0 or y.norm_weight is not None:
+                raise ValueError("a block that norms outputs takes results without a scale or a norm of their own")
+            y = Branch(y.part, extra=None if y.bias is None else y.bias.float().expand(x.shape).contiguous())
         b = y if isinstance(y, Branch) else Branch(y)
         return ops.norm_add(x, b.part, norm.weight, norm.eps, getattr(norm, "offset", 0.0), copy_dtype,
                             part_weights=b.part_weights, extra=b.extra, extra_weights=b.extra_weights, by_row=b.by_row)
@@ -195,6 +205,13 @@ def _terms(y):
     return [Joined(y)]
 
 
+def _one_bias(terms):
+    biases = [t.bias for t in terms if t.bias is not None]
+    if len(biases) > 1:
+        raise ValueError("one of the branches that join in a pass may bring a bias")
+    return biases[0] if biases else None
+
+
 def join_branches(x, results, act_dtype, next_norm=None):
     """x += the sublayers' ``results`` in one pass over the row; next_norm(x) in ``act_dtype`` when that pass can make
     it, else None."""
@@ -211,9 +228,10 @@ def join_branches(x, results, act_dtype, next_norm=None):
         raise ValueError("the branches of a block are normed with one eps")
     # (the pass takes a few branches; what is more goes first)
     while len(terms) > ops.JOIN_MAX_TERMS:
-        ops.join(x, x, [t.term() for t in terms[:ops.JOIN_MAX_TERMS]], act_dtype, max(epses, default=0.0))
+        first = terms[:ops.JOIN_MAX_TERMS]
+        ops.join(x, x, [t.term() for t in first], act_dtype, max(epses, default=0.0), vec=_one_bias(first))
         terms = terms[ops.JOIN_MAX_TERMS:]
-    return ops.join(x, x, [t.term() for t in terms], act_dtype, max(epses, default=0.0), then=kind,
+    return ops.join(x, x, [t.term() for t in terms], act_dtype, max(epses, default=0.0), vec=_one_bias(terms), then=kind,
                     then_weight=next_norm.weight if kind else None, then_eps=next_norm.eps if kind else 0.0,
                     out_dtype=act_dtype)
 
@@ -288,3 +306,89 @@ class ParallelBlock(Part):
         if trace is not None:
             trace("after_ffn", x)
         return out
+
+
+def streams_block_spec(streams: int, mixer_norm: PartSpec, mixer: PartSpec, mixer_names: dict, ffn_norm: PartSpec = None,
+                       ffn: PartSpec = None, ffn_names: dict = None) -> PartSpec:
+    """``mixer_names``, ``ffn_names``: the file's names of a sublayer's "in" [streams], "out" [streams] and "mix"
+    [streams, streams]."""
+    S = int(streams)
+    parts, tensors = {"mixer_norm": mixer_norm, "mixer": mixer}, {}
+    if ffn is not None:
+        if ffn_norm is None or ffn_names is None:
+            raise ValueError("a block with a feed-forward needs the norm before it and its numbers")
+        parts.update(ffn_norm=ffn_norm, ffn=ffn)
+    for which, names in (("mixer", mixer_names), ("ffn", ffn_names if ffn is not None else None)):
+        if names is not None:
+            tensors[which + "_in"] = TensorSpec(names["in"], (S,), init=(1.0 / S, 0.1))
+            tensors[which + "_out"] = TensorSpec(names["out"], (S,), init=(1.0, 0.1))
+            tensors[which + "_mix"] = TensorSpec(names["mix"], (S, S), init=(1.0 / S, 0.1))
+    return PartSpec("block", "streams", {"streams": S}, tensors, parts)
+
+
+class StreamsRead:
+    """What a sublayer of a ``streams`` block reads: norm(sum_s read[s] X_s)."""
+    fusable = False
+    join_kind = None
+
+    def __init__(self, read, norm):
+        self.read, self.norm = read, norm
+        if getattr(norm, "groups", 1) != 1 or not hasattr(norm, "eps") or not getattr(norm, "fusable", False):
+            raise ValueError("a block of several streams takes RMS norms over whole rows with plain weights")
+
+
+@register_part("block", "streams")
+class StreamsBlock(Part):
+    category = "block"
+
+    def __init__(self, spec, tensors, parts, rt):
+        super().__init__(spec, tensors, parts, rt)
+        self.streams = int(spec.params["streams"])
+        if not 0 < self.streams <= ops.streams_max():
+            raise ValueError(f"{self.streams} streams: the kernels take 1 to {ops.streams_max()}")
+        self.mixer, self.ffn = parts["mixer"], parts.get("ffn")
+        for part, what in ((self.mixer, "mixer"), (self.ffn, "feed-forward")):
+            if part is not None and not hasattr(part, "produce"):
+                raise ValueError(f"a block of several streams needs a {what} that hands its result over (produce)")
+        self.numbers = {role: t.float().contiguous() for role, t in tensors.items()}
+        self.first_norm = StreamsRead(self.numbers["mixer_in"], parts["mixer_norm"])
+        self.ffn_read = StreamsRead(self.numbers["ffn_in"], parts["ffn_norm"]) if self.ffn is not None else None
+
+    def _join(self, which, x, y, then):
+        terms, biases = [], []
+        for one in (y if isinstance(y, (list, tuple)) else [y]):
+            if isinstance(one, Branch):
+                terms.append((one.part, 1.0, one.by_row, one.part_weights))
+                if one.extra is not None:
+                    terms.append((one.extra, 1.0, False, one.extra_weights))
+                continue
+            one = one if isinstance(one, Joined) else Joined(one)
+            if one.norm_weight is not None:
+                raise ValueError("a block of several streams does not norm its branches")
+            terms.append((one.part, one.scale, False, None))
+            if one.bias is not None:
+                biases.append(one.bias)
+        if len(biases) > 1:
+            raise ValueError("one of a sublayer's branches may bring a bias")
+        read = isinstance(then, StreamsRead)
+        return ops.streams_join(x, self.streams, terms, self.numbers[which + "_mix"], self.numbers[which + "_out"],
+                                vec=biases[0] if biases else None, read=then.read if read else None,
+                                weight=then.norm.weight if read else None, eps=then.norm.eps if read else 0.0,
+                                act_dtype=self.rt.act_dtype)
+
+    def forward(self, x, ctx, binding, h=None, next_norm=None):
+        """Run the block on the streams ``x`` [rows, streams * width] in place.  ``h``: what the mixer reads when the block
+        before has left it.  Returns what the next block's mixer reads when that is a block of several streams too."""
+        trace = getattr(ctx, "trace", None)
+        if h is None:
+            first = self.first_norm
+            h = ops.streams_read(x, self.streams, first.read, first.norm.weight, first.norm.eps, self.rt.act_dtype)
+        h = self._join("mixer", x, self.mixer.produce(h, ctx, binding), self.ffn_read if self.ffn is not None else next_norm)
+        if trace is not None:
+            trace("after_mixer", x)
+        if self.ffn is None:
+            return h
+        h = self._join("ffn", x, self.ffn.produce(h, ctx), next_norm)
+        if trace is not None:
+            trace("after_ffn", x)
+        return h

@@ -42,6 +42,26 @@ def positional_embedding_spec(name: str, vocab: int, width: int, scale: float = 
                                                 "norm_offset": float(norm_offset)}, tensors)
 
 
+def streams_embedding_spec(name: str, vocab: int, width: int, streams: int) -> PartSpec:
+    """The residual is ``streams`` streams side by side, all of them the token's row at the start."""
+    return PartSpec("embedding", "streams", {"vocab": vocab, "width": width, "streams": int(streams)},
+                    {"table": TensorSpec(name, (vocab, width))})
+
+
+@register_part("embedding", "streams")
+class StreamsEmbedding(Part):
+    category = "embedding"
+
+    def __init__(self, spec, tensors, parts, rt):
+        super().__init__(spec, tensors, parts, rt)
+        self.table = tensors["table"]
+        self.vocab, self.width = self.table.shape
+        self.streams = int(spec.params["streams"])
+
+    def forward(self, ids: torch.Tensor, ctx=None) -> torch.Tensor:
+        return ops.streams_embed(self.table, ids, self.streams)
+
+
 @register_part("embedding", "lookup")
 class Embedding(Part):
     category = "embedding"

@@ -16,14 +16,15 @@ numbers (p, q) from a tensor of the layer: softplus(p) z^2 + z/2 for z > 0 and
 (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2 else.  The up product leaves in float32, the activation
 kernel rounds once to the activation type.
 
-Both add ``out_scale`` times their result into the stream (1 unless the spec says otherwise).
+Both add ``out_scale`` times their result into the stream (1 unless the spec says otherwise), or hand it over to a block
+that adds it up itself (``produce``).
 """
 from __future__ import annotations
 
 import torch
 
 from .. import ops
-from .base import Part, register_part
+from .base import Joined, Part, register_part
 from .linear import Linear
 from .spec import PartSpec, TensorSpec
 
@@ -119,3 +120,11 @@ class DenseFFN(Part):
         apply the norm in its last pass, else None."""
         mid = ops.activate(self.up(h, torch.float32), self.rt.act_dtype, self.activation, self.act_params)
         return self.down.add_into(mid, x, then_norm, self.rt.act_dtype, scale=self.out_scale)
+
+    def produce(self, h, ctx):
+        """ffn(h) in float32 (whole, or in K slices), for a block that adds it up itself."""
+        if self.out_scale != 1.0:
+            raise ValueError("a feed-forward that hands its result over has no multiplier of its own")
+        mid = ops.activate(self.up(h, torch.float32), self.rt.act_dtype, self.activation, self.act_params)
+        part = self.down.partial(mid) if self.down.bias is not None else None
+        return self.down.raw(mid) if part is None else Joined(part, bias=self.down.bias)

@@ -9,6 +9,9 @@
 ``gated_linear_attention``: a decay per head and key channel, alpha = sigmoid(W_a2 (W_a1 h) + b)^(1/tau); q is
 multiplied by head_dim^(-1/2); the norm's weight has v_dim numbers that the heads share.
 
+``lightning``: alpha is one constant number per head, q, k and v are the silu of their products; all heads side by side
+are RMS-normed together (one root mean square, a weight as long as the row) and multiplied by sigmoid(W_g h).
+
 The input projections are stacked into one matrix, so a step runs one product; its rows leave in float32 and
 everything that follows up to the output product's operand is float32: rotation, the decays' second product, their
 logarithms and exponentials, the state, the read-out, the norm and the gate.  The state is per-sequence state of the
@@ -18,7 +21,7 @@ that brings a sequence more rows than a chunk takes the scan's chunked form on t
 it differs from the walk by rounding); the 32-bit path always walks.
 
 ``side_by_side``: two mixers that read the same input and meet as weight * (n(left) + n(right)), n the RMS norm over
-the model's width with a weight of its own.  Their input matrices are stacked into one product; the pass that joins
+the model's width with a weight of its own, or, without norms, as a left + b right (``weight`` a pair of numbers).  Their input matrices are stacked into one product; the pass that joins
 the block's branches norms both results.  At most one of the two keeps keys and values; states of both are kept
 under "left." and "right.".  Any two mixers that can take their stacked product's rows (``given_input``,
 ``input_weight``, ``takes_slices``, ``from_rows``) fit.
@@ -57,6 +60,17 @@ def retention_spec(prefix: str, width: int, heads: int, head_dim: int, v_dim: in
         "width": width, "heads": heads, "head_dim": head_dim, "v_dim": v_dim, "decay": [float(d) for d in decay],
         "eps": float(eps), "out_scale": float(out_scale), "given_input": bool(given_input)},
         _tensors(prefix, nm, width, heads, head_dim, v_dim), {"position": position})
+
+
+def lightning_spec(prefix: str, width: int, heads: int, head_dim: int, v_dim: int, decay, eps: float, out_scale: float = 1.0,
+                   names: dict = None, given_input: bool = False) -> PartSpec:
+    """``decay``: a number a head."""
+    nm = dict(NAMES, **(names or {}))
+    tensors = _tensors(prefix, nm, width, heads, head_dim, v_dim)
+    tensors["norm"] = TensorSpec(prefix + nm["norm"], (heads * v_dim,), init=(1.0, 0.02))
+    return PartSpec("mixer", "lightning", {
+        "width": width, "heads": heads, "head_dim": head_dim, "v_dim": v_dim, "decay": [float(d) for d in decay],
+        "eps": float(eps), "out_scale": float(out_scale), "given_input": bool(given_input)}, tensors)
 
 
 def gated_linear_attention_spec(prefix: str, width: int, heads: int, head_dim: int, v_dim: int, tau: float, eps: float,
@@ -169,6 +183,25 @@ class Retention(_DecayMixer):
                               chunks=chunks, angles=angles)
 
 
+@register_part("mixer", "lightning")
+class Lightning(_DecayMixer):
+    def __init__(self, spec, tensors, parts, rt):
+        super().__init__(spec, tensors, parts, rt)
+        decay = spec.params["decay"]
+        if len(decay) != self.heads:
+            raise ValueError(f"{len(decay)} decays for {self.heads} heads")
+        self.decay = torch.tensor(decay, dtype=torch.float32, device=rt.device)
+        self.norm = tensors["norm"].contiguous()
+
+    def from_rows(self, rows, ctx, binding):
+        """What the output product reads, from the stacked product's float32 rows (a column range of wider rows, or K
+        slices of them)."""
+        q, k, v, g = self._cut(rows)
+        o = ops.decay_scan(q, k, v, None, binding.state, ctx, self.heads, self.head_dim, self.v_dim, 0.0, torch.float32,
+                           decay=self.decay, chunks=self._chunks(ctx), act_in=True)
+        return ops.rownorm_gate(o, self.norm, self.eps, g, self.rt.act_dtype)
+
+
 @register_part("mixer", "gated_linear_attention")
 class GatedLinearAttention(_DecayMixer):
     def __init__(self, spec, tensors, parts, rt):
@@ -200,15 +233,18 @@ class GatedLinearAttention(_DecayMixer):
                               decay_from=(rows.narrow(-1, first, self.rank), self.decay_up, self.decay_bias, self.rate), weight=self.norm, q_scale=self.head_dim ** -0.5, chunks=self._chunks(ctx))
 
 
-def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float, left_norm: str, right_norm: str,
-                      weight: float = 0.5) -> PartSpec:
-    """``left``, ``right``: mixers made with ``given_input``; ``left_norm``, ``right_norm``: the names of their norms' weights."""
+def side_by_side_spec(left: PartSpec, right: PartSpec, width: int, eps: float = 0.0, left_norm: str = None, right_norm: str = None,
+                      weight=0.5) -> PartSpec:
+    """``left``, ``right``: mixers made with ``given_input``; ``left_norm``, ``right_norm``: the names of their norms' weights
+    (None: the result is not normed); ``weight``: one number for both, or a pair."""
     for p in (left, right):
         if not p.params.get("given_input"):
             raise ValueError("mixers side by side are handed their stacked product's rows (given_input)")
-    return PartSpec("mixer", "side_by_side", {"width": width, "eps": float(eps), "weight": float(weight)}, {
-        "left_norm": TensorSpec(left_norm, (width,), init=(1.0, 0.02)),
-        "right_norm": TensorSpec(right_norm, (width,), init=(1.0, 0.02))}, {"left": left, "right": right})
+    weight = tuple(float(w) for w in weight) if isinstance(weight, (tuple, list)) else float(weight)
+    norms = {role: TensorSpec(name, (width,), init=(1.0, 0.02)) for role, name in (("left_norm", left_norm), ("right_norm", right_norm))
+             if name is not None}
+    return PartSpec("mixer", "side_by_side", {"width": width, "eps": float(eps), "weight": weight}, norms,
+                    {"left": left, "right": right})
 
 
 @register_part("mixer", "side_by_side")
@@ -216,10 +252,11 @@ class SideBySide(Mixer):
     def __init__(self, spec, tensors, parts, rt):
         super().__init__(spec, tensors, parts, rt)
         p = spec.params
-        self.eps, self.weight = float(p["eps"]), float(p["weight"])
+        self.eps = float(p["eps"])
+        self.weights = p["weight"] if isinstance(p["weight"], tuple) else (p["weight"], p["weight"])
         self.left, self.right = parts["left"], parts["right"]
         self.sides = (("left", self.left), ("right", self.right))
-        self.norms = (tensors["left_norm"], tensors["right_norm"])
+        self.norms = (tensors.get("left_norm"), tensors.get("right_norm"))
         if sum(m.cache_spec() is not None for _, m in self.sides) > 1:
             raise ValueError("at most one of two mixers side by side keeps keys and values")
         ws = [m.input_weight for _, m in self.sides]
@@ -257,9 +294,9 @@ class SideBySide(Mixer):
             rows = self.inp(h, torch.float32)
         cut = (rows[..., :self.split], rows[..., self.split:])
         out = []
-        for (name, m), part, norm in zip(self.sides, cut, self.norms):
+        for (name, m), part, norm, weight in zip(self.sides, cut, self.norms, self.weights):
             y = m.out.raw(m.from_rows(part, ctx, self._binding(name, binding)))
-            out.append(Joined(y, self.weight, norm, self.eps))
+            out.append(Joined(y, weight, norm, self.eps))
         return out
 
     def forward(self, h, x, ctx, binding):

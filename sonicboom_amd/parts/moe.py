@@ -11,9 +11,11 @@
 
 With ``router_score`` "sigmoid" the scores are s = sigmoid(z), the ``top`` largest s are chosen and
 their weights are s times ``router_scale``, not renormalized; "softmax_all": the same with s the
-softmax of z over all experts.  With ``groups`` > 1 the experts lie in that many equal groups of
-neighbours, a group's score is its best expert's, and only experts of the ``keep_groups`` best groups
-can be chosen.  ``shared_gate`` false: the expert
+softmax of z over all experts; "sigmoid_corrected": the ``top`` largest s + c are chosen, s = sigmoid(z) and c a number
+an expert (``correction``), and their weights are ``router_scale`` s / (the sum of the chosen s + 1e-20).
+With ``groups`` > 1 the experts lie in that many equal groups of
+neighbours, a group's score is its best expert's (with "sigmoid_corrected" the sum of its two largest s + c), and
+only experts of the ``keep_groups`` best groups can be chosen.  ``shared_gate`` false: the expert
 that every row takes is added as it is (no sigmoid gate, no tensor for it).
 
 The router runs in float32 whatever the model's type (its matrix, with the shared expert's gate
@@ -39,19 +41,22 @@ from .spec import PartSpec, TensorSpec
 
 EXPERT_ACTIVATIONS = ("swish_clamp", "silu", "relu_sq")
 UNGATED = ("relu_sq",)            # experts of two matrices: W_down act(W_up f)
-ROUTER_SCORES = ("softmax_chosen", "sigmoid", "softmax_all")
+ROUTER_SCORES = ("softmax_chosen", "sigmoid", "softmax_all", "sigmoid_corrected")
 
 
 def moe_ffn_spec(prefix: str, width: int, experts: int, top: int, inner: int, limit: float, alpha: float = 1.702,
                  shared_inner: int = 0, shared_limit: float = 0.0, activation: str = "swish_clamp",
                  names=("gate", "up", "down"), expert_prefix: str = "e{}.", router_name: str = "router",
                  shared_prefix: str = "shared.", shared_gate_name: str = "shared.sg", router_score: str = "softmax_chosen",
-                 router_scale: float = 1.0, shared_gate: bool = True, groups: int = 1, keep_groups: int = 1) -> PartSpec:
+                 router_scale: float = 1.0, shared_gate: bool = True, groups: int = 1, keep_groups: int = 1,
+                 correction_name: str = "correction") -> PartSpec:
     """``shared_inner`` > 0: an expert of that inner width that every row takes, times the sigmoid of
     one more router row (``shared_gate_name``) unless ``shared_gate`` is false.  Experts without a gate
     (``activation`` one of ``UNGATED``) have no tensor of the first of ``names``."""
     gated = activation not in UNGATED
     tensors = {"router": TensorSpec(prefix + router_name, (experts, width))}
+    if router_score == "sigmoid_corrected":
+        tensors["correction"] = TensorSpec(prefix + correction_name, (experts,), init=(0.0, 0.1))
     for e in range(experts):
         ep = prefix + expert_prefix.format(e)
         if gated:
@@ -113,6 +118,7 @@ class MoEFFN(Part):
         rows = [tensors["router"].float()]
         if self.shared_gate:
             rows.append(tensors["shared.sg"].float().reshape(1, self.width))
+        self.correction = tensors["correction"].float().contiguous() if self.router_score == "sigmoid_corrected" else None
         self.router = torch.cat(rows, dim=0).contiguous()        # float32, the shared expert's gate row last
         if self.gated:
             self.w_in = ops.MoEWeight(_stack([torch.cat([tensors[f"e{e}.gate"], tensors[f"e{e}.up"]], dim=0)
@@ -141,7 +147,7 @@ class MoEFFN(Part):
         n = h.shape[0]
         ids, weights = ops.moe_router(h, self.router, self.experts, self.top, has_gate=self.shared_gate,
                                       score=self.router_score, score_scale=self.router_scale, groups=self.groups,
-                                      keep_groups=self.keep_groups)
+                                      keep_groups=self.keep_groups, correction=self.correction)
         plan = ops.moe_plan(ids, self.experts)
         if self.gated:
             mid = ops.moe_product(h, self.w_in, plan, self.top, act, self.limit, self.alpha, pair=self.activation)   # [n * top, inner]

@@ -1,4 +1,5 @@
-"""RMS norm (/root/reference/core/src/nn/norm.cpp:25-42), whole rows or in groups, and the layer norm."""
+"""RMS norm (/root/reference/core/src/nn/norm.cpp:25-42), whole rows or in groups, the layer norm, and the RMS norm of the
+sum of a residual's streams."""
 from __future__ import annotations
 
 from .. import ops
@@ -64,3 +65,23 @@ class LayerNorm(Part):
 
     def forward(self, x, out_dtype, rows=None):
         return ops.layernorm(x, self.weight, self.eps, out_dtype, rows)
+
+
+def streams_norm_spec(weight_name: str, width: int, streams: int, eps: float) -> PartSpec:
+    return PartSpec("norm", "streams_sum", {"width": width, "streams": int(streams), "eps": float(eps)},
+                    {"weight": TensorSpec(weight_name, (width,), init=(1.0, 0.02))})
+
+
+@register_part("norm", "streams_sum")
+class StreamsNorm(Part):
+    """The RMS norm of the sum of a residual's streams (x: [rows, streams * width])."""
+    category = "norm"
+    fusable = False
+
+    def __init__(self, spec, tensors, parts, rt):
+        super().__init__(spec, tensors, parts, rt)
+        self.streams, self.eps = int(spec.params["streams"]), float(spec.params["eps"])
+        self.weight = tensors.get("weight")
+
+    def forward(self, x, out_dtype, rows=None):
+        return ops.streams_read(x, self.streams, None, self.weight, self.eps, out_dtype, rows)
