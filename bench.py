@@ -267,9 +267,9 @@ def main() -> int:
     ap.add_argument("--prompt", type=int, default=PROMPT, help="cached prompt tokens per sequence")
     ap.add_argument("--context", type=int, default=CONTEXT, help="cache size per sequence")
     ap.add_argument("--workload", choices=("steady", "mixed", "forms", "designs"), default="steady")
-    ap.add_argument("--design", choices=("rasizen", "tatelorn", "nalasun", "fitatar", "dudatar"), default="rasizen",
+    ap.add_argument("--design", choices=("rasizen", "tatelorn", "nalasun", "fitatar", "dudatar", "nidasun"), default="rasizen",
                     help="--workload designs: the design that runs beside the Qwen2.5 design")
-    ap.add_argument("--beside", choices=("qwen2", "rasizen", "tatelorn", "nalasun", "fitatar", "dudatar"), default="qwen2",
+    ap.add_argument("--beside", choices=("qwen2", "rasizen", "tatelorn", "nalasun", "fitatar", "dudatar", "nidasun"), default="qwen2",
                     help="--workload designs: the design at the same sizes that the first one runs beside")
     ap.add_argument("--design-sizes", default="2048,4096",
                     help="--workload designs: the widths of the layer sizes to run, comma separated")
@@ -763,6 +763,29 @@ def dudatar_sizes(width, vocab=32768):
             "loop": {"start": 1, "stop": 3, "times": 3}, "layers": [both, both, linear, both]}
 
 
+def nidasun_sizes(width, vocab=32768, experts=8, top=2):
+    """Layer sizes in the manner of a real model of this width: four layers of which the middle two run three times (eight
+    layer runs) over four streams; attention over windows of 4,096 keys with heads of 128 (a quarter of them kv heads) beside
+    a gated recurrence of half a width in blocks of 128 channels behind four taps; lightning attention with half as many
+    heads of 128 x 128 as the Qwen2.5 layer has; attention over chunks of 8,192 keys.  Dense feed-forwards of 4 widths
+    (the weights of the Qwen2.5 layer's) and, in one of the two repeated layers and in the last, `experts` gated experts
+    of one width of which a row takes `top`."""
+    heads = width // 128
+    att = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    routed = {"kind": "moe", "expert": {"ff": width},
+              "router": {"experts": experts, "top": top, "scale": 1.5, "groups": {"count": 4, "keep": 2}}}
+    dense = {"kind": "dense", "ff": 4 * width}
+    both = {"left": dict(att, mask={"size": 4096}, rot={"base": 1e6, "dims": 128, "scaling": {"factor": 8.0}}),
+            "right": {"width": width // 2, "blocks": width // 256, "conv": 4}, "left_scale": 0.7, "right_scale": 0.7}
+    half = max(1, heads // 2)
+    light = {"heads": half, "dim": 128, "vdim": 128, "decay": [1.0 - 2.0 ** (-5 - 5.0 * i / half) for i in range(half)]}
+    chunked = dict(att, mask={"size": 8192}, rot={"base": 1e6, "dims": 64})
+    return {"architecture": "Nidasun", "vocab": vocab, "width": width, "streams": 4, "norm": {"eps": 1e-6},
+            "loop": {"start": 1, "stop": 3, "times": 3},
+            "layers": [{"type": "parallel", "mixer": both, "mlp": dense}, {"type": "parallel", "mixer": both, "mlp": routed},
+                       {"type": "lightning", "mixer": light, "mlp": dense}, {"type": "attention", "mixer": chunked, "mlp": routed}]}
+
+
 VECTOR_F32_FLOPS = 157.3e12      # the vector units' float32 peak, against which the recurrences' scans are priced
 
 
@@ -774,7 +797,8 @@ class AllOpsTimer:
             "attention_tall_ok", "attention_mfma_ok", "attention_decode_rope_ok", "gate_code", "reduce_resid_norm_ok",
             "attention_decode_pages_per_wave", "gemm_tile_shape", "gemm_few_rows_kernel", "mingru_chunk_rows",
             "loaded_paths", "check", "latent_attention_mfma_ok", "capped_attention_mfma_ok", "moe_max_top", "moe_plan",
-            "time_conv_max_taps", "state_scan_limits", "state_scan_chunk_rows", "shared_attention_mfma_ok", "decay_scan_max_side", "decay_scan_max_rank", "decay_chunk_rows")
+            "time_conv_max_taps", "state_scan_limits", "state_scan_chunk_rows", "shared_attention_mfma_ok", "decay_scan_max_side", "decay_scan_max_rank", "decay_chunk_rows",
+            "streams_max", "gated_lru_chunk_rows", "gated_lru_limits", "gated_lru_chunked_ok")
     INNER = ("attention_plain", "attention_decode_mfma", "attention_prefill_mfma", "latent_attention_plain",
              "latent_attention_mfma", "attention_capped_plain", "attention_capped_mfma",
              "moe_product_plain", "attention_shared_plain", "attention_shared_mfma",
@@ -811,6 +835,13 @@ class AllOpsTimer:
                         label = f"{_name} {len(args[2])} branches"
                     elif _name == "decay_scan":
                         label = f"{_name} {'head' if kw.get('decay') is not None else 'channel'} {args[6]}x{args[7]}x{args[8]}"
+                    elif _name == "streams_join":
+                        parts = sum(1 if t[0].dim() == 2 else t[0].shape[1 if t[2] else 0] for t in args[2])
+                        label = f"{_name} {args[1]} streams {parts} parts"
+                    elif _name == "gated_lru":
+                        label = f"{_name} {args[6].shape[0]}x{args[6].shape[1]}"
+                    elif _name == "rownorm_gate":
+                        label = f"{_name} {args[0].shape[1]}"
                     elif _name == "time_conv":
                         label = f"{_name} {args[1].shape[0]}"
                     elif _name in ("activate", "sigmoid_mul_", "rmsnorm_pair"):
@@ -914,6 +945,22 @@ def design_roofline(label, us, calls, rows, depth, batch, width, cfgs):
         own = 1 if "channel" in label else 0
         nbytes = rows * (4 * h * ((2 + own) * d + 2 * e) + 2 * h * e) + (2 * batch * 4 * h * d * e if decode else 0)
         flops, peak_f = rows * h * d * e * 4, VECTOR_F32_FLOPS
+    elif label.startswith("streams_join"):
+        streams, parts = int(label.split()[1]), int(label.split()[3])
+        nbytes = rows * width * (8 * streams + 4 * parts + 2)
+    elif label == "streams_read":
+        nbytes = (rows if calls > 1 or decode else 1) * width * (16 + 2)
+    elif label == "streams_embed":
+        nbytes = rows * width * (2 + 16)
+    elif label.startswith("gated_lru"):
+        blocks, m = (int(v) for v in label.split()[1].split("x"))
+        w = blocks * m      # x and y in, the result out; the gates' matrices; decoding: the state and its inputs both ways
+        nbytes = rows * w * (8 + 2) + 4 * blocks * m * m + (2 * batch * w * 4 * 3 if decode else 0)
+        flops = 2 * rows * w * 2 * m
+    elif label.startswith("rownorm_gate"):
+        nbytes = rows * int(label.split()[1]) * (8 + 2)
+    elif label == "rownorm_kv_store":
+        nbytes = rows * (H * 128 + 2 * cfgs["kvw"]) * (4 + 2)
     elif label == "log_decay":
         nbytes = rows * H * 128 * 4
     elif label == "layernorm":
@@ -943,7 +990,7 @@ def design_comparison(a) -> int:
     out, table = {}, []
     for width in (int(v) for v in a.design_sizes.split(",")):
         sizes = {"rasizen": rasizen_sizes, "tatelorn": tatelorn_sizes, "nalasun": nalasun_sizes, "fitatar": fitatar_sizes,
-                 "dudatar": dudatar_sizes, "qwen2": qwen_sizes}
+                 "dudatar": dudatar_sizes, "nidasun": nidasun_sizes, "qwen2": qwen_sizes}
         for design, cfg in ((a.design, sizes[a.design](width)), (a.beside, sizes[a.beside](width))):
             model = DecoderModel.from_random(cfg, seed=0, dtype="bfloat16", device="cuda:0")
             heads = width // 128
