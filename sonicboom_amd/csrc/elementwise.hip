@@ -141,7 +141,57 @@ __global__ void activate_kernel(TO *__restrict__ out, const TI *__restrict__ in,
   }
 }
 
+// out = act(the sum of K slices + bias), numbers of a row of `width` in fours: every slice asked for before any is added.
+template <typename TO>
+__global__ void __launch_bounds__(256)
+activate_slices_kernel(TO *__restrict__ out, const float *__restrict__ in, int n_slices, size_t slice_stride, const float *__restrict__ bias,
+                       int width, size_t n4, int kind, const void *__restrict__ params, int params_dtype) {
+  const size_t idx = size_t(blockIdx.x) * 256 + threadIdx.x;
+  if (idx >= n4) return;
+  float ap = 0.0f, an = 0.0f;
+  if (kind == SB_ACT_XIELU) {
+    ap = softplus_f(ld_dyn(params, params_dtype, 0));
+    an = 0.5f + softplus_f(ld_dyn(params, params_dtype, 1));
+  }
+  float4 part[kSliceLoads];
+#pragma unroll
+  for (int s = 0; s < kSliceLoads; ++s) part[s] = *reinterpret_cast<const float4 *>(in + min(s, n_slices - 1) * slice_stride + 4 * idx);
+  float z[4] = {part[0].x, part[0].y, part[0].z, part[0].w};
+#pragma unroll
+  for (int s = 1; s < kSliceLoads; ++s)
+    if (s < n_slices) { z[0] += part[s].x; z[1] += part[s].y; z[2] += part[s].z; z[3] += part[s].w; }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    if (bias) z[e] += bias[(4 * idx) % width + e];
+    z[e] = activate_one(z[e], kind, ap, an);
+  }
+  if constexpr (sizeof(TO) == 4)
+    reinterpret_cast<float4 *>(out)[idx] = make_float4(z[0], z[1], z[2], z[3]);
+  else
+    reinterpret_cast<uint2 *>(out)[idx] = make_uint2(uint32_t(f32_to_bf16(z[0])) | uint32_t(f32_to_bf16(z[1])) << 16,
+                                                     uint32_t(f32_to_bf16(z[2])) | uint32_t(f32_to_bf16(z[3])) << 16);
+}
+
 }  // namespace
+
+// in f32 [n_slices][n_rows * width], width a multiple of 4, up to 8 slices; bias f32 [width] or NULL.
+extern "C" int sb_activate_slices(void *out, int out_dtype, const float *in, int n_slices, const float *bias, int n_rows, int width, int kind,
+                                  const void *params, int params_dtype, void *stream) {
+  SB_REQUIRE(out && in && n_rows >= 0 && width > 0 && n_slices > 0, "sb_activate_slices: bad sizes rows=%d width=%d slices=%d", n_rows, width,
+             n_slices);
+  SB_REQUIRE(sb::valid_dtype(out_dtype) && kind >= SB_ACT_SILU && kind <= SB_ACT_RELU_SQ, "sb_activate_slices: unknown type or activation");
+  SB_REQUIRE(kind != SB_ACT_XIELU || (params && sb::valid_dtype(params_dtype)), "sb_activate_slices: xIELU takes two numbers");
+  SB_SUPPORT(width % 4 == 0 && n_slices <= kSliceLoads && ((reinterpret_cast<uintptr_t>(in) | reinterpret_cast<uintptr_t>(out)) & 15) == 0,
+             "sb_activate_slices: rows of %d in %d slices", width, n_slices);
+  const size_t n4 = size_t(n_rows) * width / 4;
+  if (n4 == 0) return SB_OK;
+  hipStream_t s = (hipStream_t)stream;
+  const unsigned nb = blocks_for(n4, 256);
+  if (out_dtype == SB_F32)
+    activate_slices_kernel<float><<<nb, 256, 0, s>>>((float *)out, in, n_slices, 4 * n4, bias, width, n4, kind, params, params_dtype);
+  else activate_slices_kernel<bf16_t><<<nb, 256, 0, s>>>((bf16_t *)out, in, n_slices, 4 * n4, bias, width, n4, kind, params, params_dtype);
+  return sb::check_launch("sb_activate_slices");
+}
 
 extern "C" int sb_add_scaled(float *resid, const void *y, int y_dtype, float scale, size_t n, void *stream) {
   SB_REQUIRE(resid && y, "sb_add_scaled: null pointer");

@@ -39,9 +39,27 @@ struct LruArgs {
   const int32_t *chunks; int n_chunks; float2 *folded;           // [n_chunks, width]
 };
 
-__device__ __forceinline__ float sigmoid_f(float v) { return 1.0f / (1.0f + expf(-v)); }
+constexpr float kLog2e = 1.4426950408889634f;
 
-__device__ __forceinline__ float gelu_f(float g) { return gate_act(g, SB_GATE_GELU_TANH); }
+// By the hardware's exponential, reciprocal and root (a unit or two of the last digit each); an exponential's argument is
+// rounded once more on its way to base two, which counts as much as the rounding of the argument itself.
+__device__ __forceinline__ float exp_f(float v) { return __builtin_amdgcn_exp2f(v * kLog2e); }
+__device__ __forceinline__ float sigmoid_f(float v) { return __builtin_amdgcn_rcpf(1.0f + exp_f(-v)); }
+
+// (1 + tanh x) / 2 = sigmoid(2 x)
+__device__ __forceinline__ float gelu_f(float g) { return g * sigmoid_f(1.5957691216057308f * g * fmaf(0.044715f * g, g, 1.0f)); }
+
+// 1 - exp(-y) for y >= 0 with e = exp(-y) at hand: the series below y = 1/2 (its next term is below the last digit there)
+__device__ __forceinline__ float one_minus_exp(float y, float e) {
+  float p = fmaf(y, -1.0f / 8.0f, 1.0f);
+  p = fmaf(y * (-1.0f / 7.0f), p, 1.0f);
+  p = fmaf(y * (-1.0f / 6.0f), p, 1.0f);
+  p = fmaf(y * (-1.0f / 5.0f), p, 1.0f);
+  p = fmaf(y * (-1.0f / 4.0f), p, 1.0f);
+  p = fmaf(y * (-1.0f / 3.0f), p, 1.0f);
+  p = fmaf(y * (-1.0f / 2.0f), p, 1.0f);
+  return y < 0.5f ? y * p : 1.0f - e;
+}
 
 __device__ __forceinline__ float input_at(const LruArgs &a, int row, int c) {
   return sum_slices(a.x + size_t(row) * a.row_stride + c, a.n_slices, a.slice_stride) + a.x_bias[c];
@@ -50,8 +68,8 @@ __device__ __forceinline__ float input_at(const LruArgs &a, int row, int c) {
 // The convolution's input `back` rows before row r of the sequence (its row `row` of the step, at position pos).
 __device__ __forceinline__ float input_back(const LruArgs &a, int row, int r, int pos, int slot, int back, int c) {
   if (back <= r) return input_at(a, row - back, c);
-  if (pos < back) return 0.0f;
-  return a.ring[(size_t(slot) * a.taps + (pos - back) % a.taps) * a.width + c];
+  const float kept = a.ring[(size_t(slot) * a.taps + max(pos - back, 0) % a.taps) * a.width + c];
+  return pos < back ? 0.0f : kept;
 }
 
 // u of a row.  T: the taps where the kernel is compiled for their number, or 0.
@@ -75,8 +93,8 @@ __device__ __forceinline__ float conv_at(const LruArgs &a, int row, int r, int p
 }
 
 __device__ __forceinline__ float2 decay_and_input(float zr, float zi, float u, float rate) {
-  const float r = sigmoid_f(zr), i = sigmoid_f(zi), la = -rate * r;
-  return make_float2(expf(la), sqrtf(-expm1f(2.0f * la)) * (i * u));
+  const float r = sigmoid_f(zr), i = sigmoid_f(zi), y = rate * r, a = exp_f(-y);
+  return make_float2(a, __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * y, a * a)) * (i * u));
 }
 
 __device__ __forceinline__ void store_out(const LruArgs &a, int row, int c, float S, float y) {
@@ -89,52 +107,127 @@ __device__ __forceinline__ void load8(const float *p, float (&v)[8]) {
   const float4 a = reinterpret_cast<const float4 *>(p)[0], b = reinterpret_cast<const float4 *>(p)[1];
   v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
 }
-__device__ __forceinline__ void load8(const bf16_t *p, float (&v)[8]) {
-  const uint4 a = *reinterpret_cast<const uint4 *>(p);
-  const uint32_t u[4] = {a.x, a.y, a.z, a.w};
+
+// Eight neighbouring weights as they lie in memory.
+struct Eight16 { uint4 v; };
+struct Eight32 { float4 a, b; };
+template <typename TW> struct RawOf;
+template <> struct RawOf<bf16_t> { typedef Eight16 type; };
+template <> struct RawOf<float> { typedef Eight32 type; };
+__device__ __forceinline__ void raw8(Eight16 &r, const bf16_t *p) { r.v = *reinterpret_cast<const uint4 *>(p); }
+__device__ __forceinline__ void raw8(Eight32 &r, const float *p) {
+  r.a = reinterpret_cast<const float4 *>(p)[0];
+  r.b = reinterpret_cast<const float4 *>(p)[1];
+}
+__device__ __forceinline__ void unpack8(const Eight16 &r, float (&v)[8]) {
+  const uint32_t u[4] = {r.v.x, r.v.y, r.v.z, r.v.w};
 #pragma unroll
   for (int i = 0; i < 4; ++i) { v[2 * i] = __uint_as_float(u[i] << 16); v[2 * i + 1] = __uint_as_float(u[i] & 0xffff0000u); }
 }
+__device__ __forceinline__ void unpack8(const Eight32 &r, float (&v)[8]) {
+  v[0] = r.a.x; v[1] = r.a.y; v[2] = r.a.z; v[3] = r.a.w; v[4] = r.b.x; v[5] = r.b.y; v[6] = r.b.z; v[7] = r.b.w;
+}
 
-// grid (blocks of channels * sixteens of a block, rows / kRows).
-template <typename TW, int T, bool STEP>
+// grid (blocks of channels * sixteens of a block, rows / kRows).  In a step row i is sequence i's only one: what the kernel
+// needs from memory is asked for in two rounds (the rows' positions and slots with the weights, then everything that hangs
+// on them).  SL: 1 for whole rows, 8 for rows in up to eight K slices, 0 for any number.
+template <typename TW, int T, bool STEP, int SL>
 __global__ void __launch_bounds__(256) lru_gates_kernel(LruArgs a, int vec) {
   extern __shared__ __attribute__((aligned(16))) float us[];         // [kRows][padded]
+  __shared__ int pos_of[kRows], slot_of[kRows];
   const int padded = (a.m + 7) & ~7, per_block = (a.m + 15) / 16;
   const int blk = blockIdx.x / per_block, o0 = (blockIdx.x % per_block) * 16, c0 = blk * a.m;
   const int row0 = blockIdx.y * kRows, nr = min(kRows, a.n_rows - row0), tid = threadIdx.x;
   const int lane16 = tid & 15, o = o0 + (tid >> 4);
   const bool live = o < a.m;
   const int c = c0 + min(o, a.m - 1);
-  // what the end of the kernel needs is asked for first
   const int my_row = row0 + min(lane16, nr - 1);
-  const int my_slot = a.slots[a.row_seq[my_row]];
-  float S = 0.0f, y = 0.0f;
-  if (STEP && lane16 < nr) {
-    S = a.state[size_t(my_slot) * a.width + c];
-    y = sum_slices(a.y + size_t(my_row) * a.row_stride + c, a.n_slices, a.slice_stride) + a.y_bias[c];
+  const TW *wr = (const TW *)a.ra + size_t(c) * a.m, *wi = (const TW *)a.ri + size_t(c) * a.m;
+  if (tid < kRows) {
+    const int row = row0 + min(tid, nr - 1);
+    pos_of[tid] = a.row_pos[row];
+    slot_of[tid] = a.slots[STEP ? row : a.row_seq[row]];
   }
-  for (int idx = tid; idx < kRows * padded; idx += 256) {
-    const int i = idx / padded, k = idx - i * padded;
-    float u = 0.0f;
-    if (i < nr && k < a.m) {
-      const int row = row0 + i, seq = a.row_seq[row], pos = a.row_pos[row], slot = a.slots[seq];
-      float current;
-      u = conv_at<T>(a, row, row - a.cu_rows[seq], pos, slot, c0 + k, current);
-      if (STEP && k >= o0 && k < o0 + 16) a.ring[(size_t(slot) * a.taps + pos % a.taps) * a.width + c0 + k] = current;
+  typename RawOf<TW>::type raw_r, raw_i;
+  if (vec) {
+    const int k = min(8 * lane16, a.m - 8);        // (lanes past the block's end do not use them)
+    raw8(raw_r, wr + k);
+    raw8(raw_i, wi + k);
+  }
+  const float br = a.ra_b[c], bi = a.ri_b[c], rate = a.rate[c];
+  __syncthreads();
+  float S = 0.0f, y_in[SL > 0 ? SL : 1];
+  const int my_slot = slot_of[lane16 & (kRows - 1)];
+  if (STEP) {
+    S = a.state[size_t(my_slot) * a.width + c];
+    if (SL > 0)
+#pragma unroll
+      for (int s = 0; s < SL; ++s) y_in[s] = a.y[min(s, a.n_slices - 1) * a.slice_stride + size_t(my_row) * a.row_stride + c];
+  }
+  if constexpr (STEP && T > 0 && SL > 0) {
+    constexpr int U = 4;                            // numbers of u that a thread works on at once
+    for (int base = tid; base < kRows * padded; base += 256 * U) {
+      float x_in[U][SL], kept[U][T];                // kept[j][t]: the input T - 1 - t rows back
+      float w[U][T], bx[U], bw[U];
+#pragma unroll
+      for (int j = 0; j < U; ++j) {
+        const int idx = min(base + 256 * j, kRows * padded - 1), i = idx / padded, k = min(idx - i * padded, a.m - 1);
+        const int row = row0 + min(i, nr - 1), pos = pos_of[i];
+        const float *ring = a.ring + size_t(slot_of[i]) * T * a.width + c0 + k;
+#pragma unroll
+        for (int s = 0; s < SL; ++s) x_in[j][s] = a.x[min(s, a.n_slices - 1) * a.slice_stride + size_t(row) * a.row_stride + c0 + k];
+#pragma unroll
+        for (int t = 0; t < T - 1; ++t) kept[j][t] = ring[size_t(max(pos - (T - 1 - t), 0) % T) * a.width];
+#pragma unroll
+        for (int t = 0; t < T; ++t) w[j][t] = a.taps_w[size_t(c0 + k) * T + t];
+        bx[j] = a.x_bias[c0 + k];
+        bw[j] = a.taps_b[c0 + k];
+      }
+#pragma unroll
+      for (int j = 0; j < U; ++j) {
+        const int idx = base + 256 * j, i = idx / padded, k = idx - i * padded;
+        if (idx >= kRows * padded) continue;
+        const bool on = i < nr && k < a.m;
+        const int pos = pos_of[min(i, kRows - 1)];
+        float cur = x_in[j][0];
+#pragma unroll
+        for (int s = 1; s < SL; ++s)
+          if (s < a.n_slices) cur += x_in[j][s];
+        cur += bx[j];
+        float acc = 0.0f;
+#pragma unroll
+        for (int t = 0; t < T - 1; ++t) acc = fmaf(w[j][t], pos < T - 1 - t ? 0.0f : kept[j][t], acc);
+        acc = fmaf(w[j][T - 1], cur, acc) + bw[j];
+        if (on && k >= o0 && k < o0 + 16) a.ring[(size_t(slot_of[i]) * T + pos % T) * a.width + c0 + k] = cur;
+        us[idx] = on ? acc : 0.0f;
+      }
     }
-    us[idx] = u;
+  } else {
+    for (int idx = tid; idx < kRows * padded; idx += 256) {
+      const int i = idx / padded, k = idx - i * padded;
+      float u = 0.0f;
+      if (i < nr && k < a.m) {
+        const int row = row0 + i, pos = pos_of[i], slot = slot_of[i];
+        float current;
+        u = conv_at<T>(a, row, STEP ? 0 : row - a.cu_rows[a.row_seq[row]], pos, slot, c0 + k, current);
+        if (STEP && k >= o0 && k < o0 + 16) a.ring[(size_t(slot) * a.taps + pos % a.taps) * a.width + c0 + k] = current;
+      }
+      us[idx] = u;
+    }
   }
   __syncthreads();
   float zr[kRows], zi[kRows];
 #pragma unroll
   for (int i = 0; i < kRows; ++i) zr[i] = zi[i] = 0.0f;
-  const TW *wr = (const TW *)a.ra + size_t(c) * a.m, *wi = (const TW *)a.ri + size_t(c) * a.m;
   for (int k = 8 * lane16; k < a.m; k += 128) {
     float r8[8], i8[8];
     if (vec) {
-      load8(wr + k, r8);
-      load8(wi + k, i8);
+      if (k >= 128) {
+        raw8(raw_r, wr + k);
+        raw8(raw_i, wi + k);
+      }
+      unpack8(raw_r, r8);
+      unpack8(raw_i, i8);
     } else {
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
@@ -153,23 +246,35 @@ __global__ void __launch_bounds__(256) lru_gates_kernel(LruArgs a, int vec) {
       }
     }
   }
+  // sums over the sixteen lanes: at every step a lane hands half of its numbers over and keeps the sums of the other half,
+  // until lane l has row l % 8 of one of the two products (lanes 0 .. 7 the first)
+  static_assert(kRows == 8, "sixteen lanes share the sums of eight rows of two products");
+  float z[2 * kRows];
+#pragma unroll
+  for (int i = 0; i < kRows; ++i) { z[i] = zr[i]; z[kRows + i] = zi[i]; }
 #pragma unroll
   for (int off = 8; off > 0; off >>= 1)
 #pragma unroll
-    for (int i = 0; i < kRows; ++i) {
-      zr[i] += __shfl_xor(zr[i], off, 64);
-      zi[i] += __shfl_xor(zi[i], off, 64);
+    for (int i = 0; i < off; ++i) {
+      const bool up = lane16 & off;
+      z[i] = (up ? z[off + i] : z[i]) + __shfl_xor(up ? z[i] : z[off + i], off, 64);
     }
-  float r = 0.0f, g = 0.0f;
-#pragma unroll
-  for (int i = 0; i < kRows; ++i)
-    if (lane16 == i) { r = zr[i]; g = zi[i]; }
+  const float g = __shfl_xor(z[0], 8, 64);           // (of lanes 0 .. 7)
   if (!live || lane16 >= nr) return;
-  const float2 ab = decay_and_input(r + a.ra_b[c], g + a.ri_b[c], us[lane16 * padded + o], a.rate[c]);
+  const float2 ab = decay_and_input(z[0] + br, g + bi, us[lane16 * padded + o], rate);
   if (STEP) {
     S = fmaf(ab.x, S, ab.y);
     a.state[size_t(my_slot) * a.width + c] = S;
-    store_out(a, my_row, c, S, y);
+    float y;
+    if (SL > 0) {
+      y = y_in[0];
+#pragma unroll
+      for (int s = 1; s < SL; ++s)
+        if (s < a.n_slices) y += y_in[s];
+    } else {
+      y = sum_slices(a.y + size_t(my_row) * a.row_stride + c, a.n_slices, a.slice_stride);
+    }
+    store_out(a, my_row, c, S, y + a.y_bias[c]);
   } else {
     a.ab[size_t(my_row) * a.width + c] = ab;
   }
@@ -210,6 +315,20 @@ __global__ void __launch_bounds__(512) lru_chunk_gates_kernel(LruArgs a) {
   const int32_t *ch = a.chunks + 4 * size_t(blockIdx.x);
   const int r0 = ch[0], nr = ch[1], seq = ch[2];
   const int c0 = blockIdx.y * a.m, tid = threadIdx.x, threads = blockDim.x, lane = tid & 63, col = lane & 15, g = lane >> 4;
+  const bf16_t *wr = (const bf16_t *)a.ra, *wi = (const bf16_t *)a.ri;
+  const int n_ot = (a.m + 15) / 16, first_ot = min(tid >> 6, n_ot - 1);
+  // what the wave's first sixteen channels need is asked for first
+  constexpr int AHEAD = 4;               // steps of 32 of the products
+  uint4 ahead[AHEAD][2];
+  {
+    const int o = 16 * first_ot + col, c = c0 + min(o, a.m - 1);
+#pragma unroll
+    for (int s = 0; s < AHEAD; ++s) {
+      const int k = 32 * s + 8 * g;
+      ahead[s][0] = ld16(wr + size_t(c) * a.m + k, k < a.m && o < a.m);
+      ahead[s][1] = ld16(wi + size_t(c) * a.m + k, k < a.m && o < a.m);
+    }
+  }
   const int first = a.cu_rows[seq], slot = a.slots[seq], p0 = a.row_pos[r0];
   // a thread a channel and a part of sixteen rows: every input is read once and stays for the taps after it
   for (int item = tid; item < (kChunk / kPart) * m32; item += threads) {
@@ -226,8 +345,21 @@ __global__ void __launch_bounds__(512) lru_chunk_gates_kernel(LruArgs a) {
       for (int j = 0; j < N; ++j) {
         // input i0 - (T - 1) + j of the chunk; rows past the chunk's last read the last again
         const int i = i0 - (T - 1) + j, row = r0 + min(i, nr - 1);
-        if (row >= first) in[j] = input_at(a, row, c0 + k);
-        else in[j] = p0 + i >= 0 ? a.ring[(size_t(slot) * T + (p0 + i) % T) * a.width + c0 + k] : 0.0f;
+        in[j] = a.x[size_t(max(row, first)) * a.row_stride + c0 + k];
+      }
+      for (int s = 1; s < a.n_slices; ++s)
+#pragma unroll
+        for (int j = 0; j < N; ++j)
+          in[j] += a.x[s * a.slice_stride + size_t(max(r0 + min(i0 - (T - 1) + j, nr - 1), first)) * a.row_stride + c0 + k];
+      const float bx = a.x_bias[c0 + k];
+#pragma unroll
+      for (int j = 0; j < N; ++j) in[j] += bx;
+      if (r0 + i0 - (T - 1) < first) {      // the sequence's first part of the step: inputs of earlier steps
+#pragma unroll
+        for (int j = 0; j < T - 1; ++j) {
+          const int i = i0 - (T - 1) + j, p = p0 + i;
+          if (r0 + i < first) in[j] = p >= 0 ? a.ring[(size_t(slot) * T + p % (T > 0 ? T : 1)) * a.width + c0 + k] : 0.0f;
+        }
       }
       float w[T > 0 ? T : 1];
 #pragma unroll
@@ -248,27 +380,26 @@ __global__ void __launch_bounds__(512) lru_chunk_gates_kernel(LruArgs a) {
       }
     }
 #pragma unroll
-    for (int i = 0; i < kPart; ++i) {
-      const bf16_t hi = f32_to_bf16(u[i]);
-      const float rest = u[i] - bf16_to_f32(hi);
-      const bf16_t mid = f32_to_bf16(rest);
-      dst[i * stride] = hi;
-      dst[plane + i * stride] = mid;
-      dst[2 * plane + i * stride] = f32_to_bf16(rest - bf16_to_f32(mid));
+    for (int i = 0; i < kPart; i += 2) {         // two rows a conversion
+      float f0 = u[i], f1 = u[i + 1];
+#pragma unroll
+      for (int p = 0; p < 3; ++p) {
+        const uint32_t w = pack_bf16(f0, f1);
+        dst[p * plane + i * stride] = bf16_t(w & 0xffffu);
+        dst[p * plane + (i + 1) * stride] = bf16_t(w >> 16);
+        f0 -= __uint_as_float(w << 16);
+        f1 -= __uint_as_float(w & 0xffff0000u);
+      }
     }
   }
   __syncthreads();
-  const bf16_t *wr = (const bf16_t *)a.ra, *wi = (const bf16_t *)a.ri;
-  const int n_ot = (a.m + 15) / 16;
   for (int ot = tid >> 6; ot < n_ot; ot += threads >> 6) {
     const int o = 16 * ot + col, c = c0 + min(o, a.m - 1);
     floatx4_t zr[kChunk / 16], zi[kChunk / 16];
 #pragma unroll
     for (int t = 0; t < kChunk / 16; ++t) zr[t] = zi[t] = floatx4_t{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-    for (int k = 8 * g; k < m32; k += 32) {
-      const bool in = k < a.m && o < a.m;
-      const bf16x8_t fr = as_bf16x8(ld16(wr + size_t(c) * a.m + k, in)), fi = as_bf16x8(ld16(wi + size_t(c) * a.m + k, in));
+    auto product = [&](int k, uint4 w0, uint4 w1) {
+      const bf16x8_t fr = as_bf16x8(w0), fi = as_bf16x8(w1);
 #pragma unroll
       for (int p = 2; p >= 0; --p)
 #pragma unroll
@@ -277,9 +408,20 @@ __global__ void __launch_bounds__(512) lru_chunk_gates_kernel(LruArgs a) {
           zr[t] = mfma16(fu, fr, zr[t]);
           zi[t] = mfma16(fu, fi, zi[t]);
         }
+    };
+    const float br = a.ra_b[c], bi = a.ri_b[c], rate = a.rate[c];
+    int s0 = 0;
+    if (ot == first_ot) {
+#pragma unroll
+      for (int s = 0; s < AHEAD; ++s)
+        if (32 * s < m32) product(32 * s + 8 * g, ahead[s][0], ahead[s][1]);
+      s0 = AHEAD;
+    }
+    for (int k = 32 * s0 + 8 * g; k < m32; k += 32) {
+      const bool in = k < a.m && o < a.m;
+      product(k, ld16(wr + size_t(c) * a.m + k, in), ld16(wi + size_t(c) * a.m + k, in));
     }
     // a lane has rows 16 t + 4 g .. + 3 of channel o
-    const float br = a.ra_b[c], bi = a.ri_b[c], rate = a.rate[c];
     float2 total = make_float2(1.0f, 0.0f);
 #pragma unroll
     for (int t = 0; t < kChunk / 16; ++t) {
@@ -373,15 +515,26 @@ __global__ void __launch_bounds__(256) lru_chunk_walk_kernel(LruArgs a) {
     }
 }
 
+template <typename TW, int SL>
+void launch_step(const LruArgs &a, dim3 grid, size_t lds, int vec, hipStream_t s) {
+  if (a.taps == 2) lru_gates_kernel<TW, 2, true, SL><<<grid, 256, lds, s>>>(a, vec);
+  else if (a.taps == 3) lru_gates_kernel<TW, 3, true, SL><<<grid, 256, lds, s>>>(a, vec);
+  else if (a.taps == 4) lru_gates_kernel<TW, 4, true, SL><<<grid, 256, lds, s>>>(a, vec);
+  else lru_gates_kernel<TW, 0, true, SL><<<grid, 256, lds, s>>>(a, vec);
+}
+
 template <typename TW, bool STEP>
 void launch_gates(const LruArgs &a, hipStream_t s) {
   const dim3 grid((a.width / a.m) * ((a.m + 15) / 16), (a.n_rows + kRows - 1) / kRows);
   const size_t lds = size_t(kRows) * ((a.m + 7) & ~7) * sizeof(float);
   const int vec = a.m % 8 == 0 && (reinterpret_cast<uintptr_t>(a.ra) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.ri) & 15) == 0;
-  if (a.taps == 2) lru_gates_kernel<TW, 2, STEP><<<grid, 256, lds, s>>>(a, vec);
-  else if (a.taps == 3) lru_gates_kernel<TW, 3, STEP><<<grid, 256, lds, s>>>(a, vec);
-  else if (a.taps == 4) lru_gates_kernel<TW, 4, STEP><<<grid, 256, lds, s>>>(a, vec);
-  else lru_gates_kernel<TW, 0, STEP><<<grid, 256, lds, s>>>(a, vec);
+  if constexpr (STEP) {
+    if (a.n_slices == 1) launch_step<TW, 1>(a, grid, lds, vec, s);
+    else if (a.n_slices <= 8) launch_step<TW, 8>(a, grid, lds, vec, s);
+    else lru_gates_kernel<TW, 0, true, 0><<<grid, 256, lds, s>>>(a, vec);
+  } else {
+    lru_gates_kernel<TW, 0, false, 0><<<grid, 256, lds, s>>>(a, vec);
+  }
 }
 
 template <int T>

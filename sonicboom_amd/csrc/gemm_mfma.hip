@@ -34,6 +34,7 @@ struct Args {
   const float *resid;
   float resid_scale;   // Y = resid_scale * (X W^T + bias) + resid  (1 unless a branch has a multiplier)
   int n_rows, n_out, n_in;
+  int relu_sq;     // 1: Y = max(X W^T + bias, 0)^2 (no residual, whole products)
   int gated;       // an sb_gate; not 0: W is [2*n_out, n_in], rows n (gate) and n_out + n (up)
   int tiles_m, tiles_n;
   int w_tiles;     // packed W: 16-row tiles of one half (ceil(n_out / 16))
@@ -122,6 +123,10 @@ __device__ __forceinline__ void store_tile(const Args &a, float *lds_f, int t0, 
 #pragma unroll
           for (int q = 0; q < 4; ++q) v[q] = v[q] + ld_dyn(bias, a.bias_dtype, n_first + q);
         }
+        if (a.relu_sq) {
+#pragma unroll
+          for (int q = 0; q < 4; ++q) { const float z = fmaxf(v[q], 0.0f); v[q] = z * z; }
+        }
         if (resid) {
           const floatx4_t rv = *reinterpret_cast<const floatx4_t *>(resid + idx);
 #pragma unroll
@@ -141,6 +146,7 @@ __device__ __forceinline__ void store_tile(const Args &a, float *lds_f, int t0, 
           if (n_first + q >= a.n_out) continue;
           float u = v[q];
           if (bias) u = u + ld_dyn(bias, a.bias_dtype, n_first + q);
+          if (a.relu_sq) { const float z = fmaxf(u, 0.0f); u = z * z; }
           if (resid) u = u * a.resid_scale + resid[idx + q];
           if (f32_out) y_f[idx + q] = u;
           else y_h[idx + q] = f32_to_bf16(u);
@@ -770,6 +776,18 @@ extern "C" int sb_gemm_mfma_scaled_bf16(void *y, int y_dtype, const void *x, con
                                         int bias_dtype, const float *resid, float resid_scale, int n_rows, int n_out,
                                         int n_in, int gated, int packed, int tile_shape, void *stream);
 
+namespace {
+int gemm_whole(void *y, int y_dtype, const void *x, const void *w, const void *bias, int bias_dtype, const float *resid, float resid_scale,
+               int n_rows, int n_out, int n_in, int gated, int relu_sq, int packed, int tile_shape, void *stream);
+}
+
+// The product with an activation of an ungated feed-forward on its way out: SB_ACT_RELU_SQ, max(z, 0)^2 of z = X W^T + bias.
+extern "C" int sb_gemm_mfma_act_bf16(void *y, int y_dtype, const void *x, const void *w, const void *bias, int bias_dtype, int n_rows,
+                                     int n_out, int n_in, int act, int packed, int tile_shape, void *stream) {
+  SB_SUPPORT(act == SB_ACT_RELU_SQ, "sb_gemm_mfma_act_bf16: activation %d is not the square of max(z, 0)", act);
+  return gemm_whole(y, y_dtype, x, w, bias, bias_dtype, nullptr, 1.0f, n_rows, n_out, n_in, 0, 1, packed, tile_shape, stream);
+}
+
 extern "C" int sb_gemm_mfma_bf16(void *y, int y_dtype, const void *x, const void *w, const void *bias,
                                  int bias_dtype, const float *resid, int n_rows, int n_out, int n_in,
                                  int gated, int packed, int tile_shape, void *stream) {
@@ -782,6 +800,12 @@ extern "C" int sb_gemm_mfma_bf16(void *y, int y_dtype, const void *x, const void
 extern "C" int sb_gemm_mfma_scaled_bf16(void *y, int y_dtype, const void *x, const void *w, const void *bias,
                                         int bias_dtype, const float *resid, float resid_scale, int n_rows, int n_out,
                                         int n_in, int gated, int packed, int tile_shape, void *stream) {
+  return gemm_whole(y, y_dtype, x, w, bias, bias_dtype, resid, resid_scale, n_rows, n_out, n_in, gated, 0, packed, tile_shape, stream);
+}
+
+namespace {
+int gemm_whole(void *y, int y_dtype, const void *x, const void *w, const void *bias, int bias_dtype, const float *resid, float resid_scale,
+               int n_rows, int n_out, int n_in, int gated, int relu_sq, int packed, int tile_shape, void *stream) {
   SB_REQUIRE(y && x && w, "sb_gemm_mfma_bf16: null pointer");
   SB_REQUIRE(n_rows >= 0 && n_out > 0 && n_in > 0, "sb_gemm_mfma_bf16: bad sizes rows=%d out=%d in=%d",
              n_rows, n_out, n_in);
@@ -796,7 +820,7 @@ extern "C" int sb_gemm_mfma_scaled_bf16(void *y, int y_dtype, const void *x, con
   Args a;
   a.y = y; a.y_dtype = y_dtype; a.x = (const bf16_t *)x; a.w = (const bf16_t *)w;
   a.bias = bias; a.bias_dtype = bias_dtype; a.resid = resid; a.resid_scale = resid_scale;
-  a.n_rows = n_rows; a.n_out = n_out; a.n_in = n_in; a.gated = gated;
+  a.n_rows = n_rows; a.n_out = n_out; a.n_in = n_in; a.gated = gated; a.relu_sq = relu_sq;
   a.partial = nullptr; a.stages_per_slice = 0;
   a.vec4 = n_out % 4 == 0 && (reinterpret_cast<uintptr_t>(y) | reinterpret_cast<uintptr_t>(resid)) % 16 == 0;
   const bool direct_ok = packed && n_in % 64 == 0;
@@ -849,6 +873,7 @@ extern "C" int sb_gemm_mfma_scaled_bf16(void *y, int y_dtype, const void *x, con
   if (rc != SB_OK) return rc;
   return sb::check_launch("sb_gemm_mfma_bf16");
 }
+}  // namespace
 
 namespace {
 // K slices of the partial form, and the tiles that multiply them.  Few rows: enough blocks for
@@ -928,7 +953,7 @@ extern "C" int sb_gemm_mfma_partial_bf16(float *partial, const void *x, const vo
   Args a;
   a.y = nullptr; a.y_dtype = SB_F32; a.x = (const bf16_t *)x; a.w = (const bf16_t *)w;
   a.bias = nullptr; a.bias_dtype = 0; a.resid = nullptr; a.resid_scale = 1.0f;
-  a.n_rows = n_rows; a.n_out = n_out; a.n_in = n_in; a.gated = 0;
+  a.n_rows = n_rows; a.n_out = n_out; a.n_in = n_in; a.gated = 0; a.relu_sq = 0;
   const PartialPlan plan = partial_plan(n_rows, n_out, n_in, packed && n_in % 64 == 0);
   const int tile = plan.big ? 256 : 128;
   a.tiles_m = (n_rows + tile - 1) / tile;

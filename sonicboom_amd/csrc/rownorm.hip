@@ -24,6 +24,7 @@ struct KVArgs {
   const int32_t *row_pos, *row_seq, *page_table; int max_pages, n_pages;
   void *k_cache, *v_cache;
   int heads_q, heads_kv, dk, dv;
+  int w_eights;                        // bfloat16 weights that are read eight at a time, pairs in eights
 };
 
 template <int THREADS, int N>
@@ -62,11 +63,30 @@ __device__ __forceinline__ float turned(const KVArgs &a, const float *row, int q
   return lo ? y0 : y1;
 }
 
+__device__ __forceinline__ void lds8(const float *p, float (&v)[8]) {
+  const float4 a = reinterpret_cast<const float4 *>(p)[0], b = reinterpret_cast<const float4 *>(p)[1];
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+}
+
+// numbers i .. i + 7 of the row of q and k after their norm (bfloat16 weights in eights), as normed() gives them one by one
+__device__ __forceinline__ void normed8(const KVArgs &a, const float *row, int qw, int i, float q_inv, float k_inv, float (&v)[8]) {
+  const bool is_q = i < qw;
+  const uint4 w = *reinterpret_cast<const uint4 *>(is_q ? (const bf16_t *)a.q_w + i : (const bf16_t *)a.k_w + (i - qw));
+  const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+  const float inv = is_q ? q_inv : k_inv;
+  lds8(row + i, v);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    v[2 * e] = (v[2 * e] * inv) * __uint_as_float(u[e] << 16);
+    v[2 * e + 1] = (v[2 * e + 1] * inv) * __uint_as_float(u[e] & 0xffff0000u);
+  }
+}
+
 // EIGHTS: bfloat16 queries and cache, head sizes in eights: eight numbers a store; FOURS: the row is read four at a time
 template <typename TQ, typename TC, int THREADS, bool EIGHTS, bool FOURS>
 __global__ void __launch_bounds__(THREADS) rownorm_kv_store_kernel(KVArgs a) {
   extern __shared__ __attribute__((aligned(16))) float row[];
-  __shared__ float cs[kMaxHalf], sn[kMaxHalf];
+  __shared__ __attribute__((aligned(16))) float cs[kMaxHalf], sn[kMaxHalf];
   const int r = blockIdx.x, tid = threadIdx.x;
   const float *src = a.qkv + size_t(r) * a.row_stride;
   const int qw = a.heads_q * a.dk, kw = a.heads_kv * a.dk, n = qw + kw;
@@ -106,11 +126,29 @@ __global__ void __launch_bounds__(THREADS) rownorm_kv_store_kernel(KVArgs a) {
   if (EIGHTS) {
     for (int g = tid; g < n / 8; g += THREADS) {
       const int i0 = 8 * g, head = i0 / a.dk, d0 = i0 - head * a.dk;
+      float v[8];
+      if (a.w_eights) {                  // (the pairs in eights too: eight numbers turn together, or none does)
+        normed8(a, row, qw, i0, q_inv, k_inv, v);
+        if (d0 < 2 * a.half) {
+          const bool lo = d0 < a.half;
+          float o[8], c8[8], s8[8];
+          normed8(a, row, qw, lo ? i0 + a.half : i0 - a.half, q_inv, k_inv, o);
+          lds8(cs + (lo ? d0 : d0 - a.half), c8);
+          lds8(sn + (lo ? d0 : d0 - a.half), s8);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            float y0, y1;
+            rotate_pair(lo ? v[e] : o[e], lo ? o[e] : v[e], c8[e], s8[e], y0, y1);
+            v[e] = lo ? y0 : y1;
+          }
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = turned(a, row, qw, i0 + e, d0 + e, q_inv, k_inv, cs, sn);
+      }
       uint32_t packed[4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e)
-        packed[e] = uint32_t(f32_to_bf16(turned(a, row, qw, i0 + 2 * e, d0 + 2 * e, q_inv, k_inv, cs, sn))) |
-                    uint32_t(f32_to_bf16(turned(a, row, qw, i0 + 2 * e + 1, d0 + 2 * e + 1, q_inv, k_inv, cs, sn))) << 16;
+      for (int e = 0; e < 4; ++e) packed[e] = uint32_t(f32_to_bf16(v[2 * e])) | uint32_t(f32_to_bf16(v[2 * e + 1])) << 16;
       const uint4 o = make_uint4(packed[0], packed[1], packed[2], packed[3]);
       if (i0 < qw) *reinterpret_cast<uint4 *>((bf16_t *)a.q_out + size_t(r) * qw + i0) = o;
       else if (page >= 0)      // eight neighbouring numbers of a key stay neighbours in the cache's order
@@ -227,7 +265,8 @@ extern "C" int sb_rownorm_kv_store(void *q_out, int q_dtype, const float *qkv, i
              n, half, kMaxRow, kMaxHalf);
   if (n_rows == 0) return SB_OK;
   const KVArgs a{q_out, qkv, row_stride, n_slices, slice_stride, q_w, k_w, w_dtype, eps, inv_freq, half, row_pos, row_seq, page_table,
-                 max_pages, n_pages, k_cache, v_cache, heads_q, heads_kv, dk, dv};
+                 max_pages, n_pages, k_cache, v_cache, heads_q, heads_kv, dk, dv,
+                 w_dtype == SB_BF16 && half % 8 == 0 && ((reinterpret_cast<uintptr_t>(q_w) | reinterpret_cast<uintptr_t>(k_w)) & 15) == 0};
   hipStream_t s = (hipStream_t)stream;
   const auto aligned = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   const bool fours = dk % 4 == 0 && row_stride % 4 == 0 && slice_stride % 4 == 0 && aligned(qkv);

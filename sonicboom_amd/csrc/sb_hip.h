@@ -584,6 +584,14 @@ int sb_decay_chunks(void *out, int out_dtype, int out_stride, const float *q, co
 int sb_log_decay(float *out, int out_stride, const float *a, int a_stride, const float *w, const float *bias, int n_rows,
                  int rank, int width, float rate, void *stream);
 
+/* ---- activations where a product ends (csrc/gemm_mfma.hip, csrc/elementwise.hip) ----------------------------
+ * sb_gemm_mfma_act_bf16: sb_gemm_mfma_bf16 with Y = act(X W^T + bias); SB_ACT_RELU_SQ only.
+ * sb_activate_slices: act(the sum of K slices + bias), rows of a width in fours, up to eight slices. */
+int sb_gemm_mfma_act_bf16(void *y, int y_dtype, const void *x, const void *w, const void *bias, int bias_dtype, int n_rows, int n_out,
+                          int n_in, int act, int packed, int tile_shape, void *stream);
+int sb_activate_slices(void *out, int out_dtype, const float *in, int n_slices, const float *bias, int n_rows, int width, int kind,
+                       const void *params, int params_dtype, void *stream);
+
 /* ---- a residual of several streams that mix (csrc/streams.hip) -----------------------------------------
  * A row of x is `streams` rows of `width` float32 numbers X_1 .. X_S side by side.
  * sb_streams_embed: all of them table[id].

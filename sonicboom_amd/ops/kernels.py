@@ -217,6 +217,26 @@ def activate(x: torch.Tensor, out_dtype: torch.dtype, activation: str, params: O
     return out
 
 
+def activate_slices(part: torch.Tensor, out_dtype: torch.dtype, activation: str, bias: Optional[torch.Tensor] = None,
+                    params: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """act(the sum of ``part``'s slices + bias) for float32 ``part`` [slices, rows, width], ``bias`` float32 [width]."""
+    _dev(part, bias, params)
+    if part.dtype != torch.float32 or part.dim() != 3 or activation not in ACTIVATIONS:
+        raise KernelLibraryError(f"slices must be float32 [slices, rows, width] and the activation one of {sorted(ACTIVATIONS)}")
+    slices, n, width = part.shape
+    if bias is not None:
+        _f32_vec(bias, width, "biases")
+    if activation == "xielu" and (params is None or params.numel() != 2):
+        raise KernelLibraryError("xIELU takes two numbers")
+    if width % 4 or slices > 8:
+        whole = part.sum(0) if bias is None else part.sum(0) + bias
+        return activate(whole, out_dtype, activation, params)
+    out = torch.empty((n, width), dtype=out_dtype, device=part.device)
+    check(library.core().sb_activate_slices(_p(out), _dt(out), _p(part), slices, _p(bias), n, width, ACTIVATIONS[activation], _p(params),
+                                            _dt(params) if params is not None else 0, _stream()))
+    return out
+
+
 def cast(x: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     _dev(x)
     if x.dtype == dtype:
@@ -674,6 +694,25 @@ def gemm_bf16_add_scaled(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.
     check(library.core().sb_gemm_mfma_scaled_bf16(_p(resid), 0, _p(x), _p(w), _p(bias), _dt(bias) if bias is not None else 0,
                                                   _p(resid), float(scale), t, n, k, 0, 1, _hints.tile_shape, _stream()))
     return True
+
+
+def gemm_bf16_activated(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out_dtype: torch.dtype, activation: str,
+                        packed_shape) -> Optional[torch.Tensor]:
+    """act(x w^T (+ bias)) in the tiled product's own epilogue; None when the activation or the sizes are not its own (few
+    rows go to the weight-streaming kernels): the caller then activates in a pass of its own."""
+    _dev(x, w, bias)
+    if activation != "relu_sq" or x.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or packed_shape is None or x.dim() != 2:
+        return None
+    n, k = packed_shape
+    t = x.shape[0]
+    if t <= STREAM_MAX_ROWS or x.shape[1] != k or k % 8 or x.data_ptr() % 16 or w.data_ptr() % 16:
+        return None
+    if bias is not None and bias.numel() != n:
+        raise KernelLibraryError(f"bias has {bias.numel()} elements, the product has {n} columns")
+    y = torch.empty((t, n), dtype=out_dtype, device=x.device)
+    check(library.core().sb_gemm_mfma_act_bf16(_p(y), _dt(y), _p(x), _p(w), _p(bias), _dt(bias) if bias is not None else 0, t, n, k,
+                                               ACTIVATIONS[activation], 1, _hints.tile_shape, _stream()))
+    return y
 
 
 @contextlib.contextmanager

@@ -109,6 +109,8 @@ _CORE_SIGNATURES = {
     "sb_log_decay": [_P, _I, _P, _I, _P, _P, _I, _I, _I, _F, _P],
     "sb_moe_router_corrected": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P],
     "sb_attention_chunked": [_P, _P, _I, _I, _P, _P, _I, _P, _I, _I, _P, _P, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _P, _I, _I, _I, _P],
+    "sb_gemm_mfma_act_bf16": [_P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
+    "sb_activate_slices": [_P, _I, _P, _I, _P, _I, _I, _I, _P, _I, _P],
     "sb_streams_max": [],
     "sb_streams_max_parts": [],
     "sb_streams_embed": [_P, _P, _I, _P, _I, _I, _I, _I, _P],

@@ -13,8 +13,8 @@ kernel, whose output is rounded once to the activation type.
 ``dense``: y = W_down act(W_up f + b_up) + b_down (biases when the spec names them), the activation one
 of ``ops.ACTIVATIONS`` ("gelu_erf": z Phi(z) by the error function; "relu_sq": max(z, 0)^2); "xielu" reads its two
 numbers (p, q) from a tensor of the layer: softplus(p) z^2 + z/2 for z > 0 and
-(1/2 + softplus(q)) (exp(z) - 1 - z) + z/2 else.  The up product leaves in float32, the activation
-kernel rounds once to the activation type.
+(1/2 + softplus(q)) (exp(z) - 1 - z) + z/2 else.  The activation is applied to the product in float32
+(``Linear.activated``) and rounded once to the activation type.
 
 Both add ``out_scale`` times their result into the stream (1 unless the spec says otherwise), or hand it over to a block
 that adds it up itself (``produce``).
@@ -118,13 +118,13 @@ class DenseFFN(Part):
     def forward(self, h, x, ctx, then_norm=None):
         """x += out_scale * (W_down act(W_up h + b_up) + b_down).  Returns then_norm(x) when the down projection could
         apply the norm in its last pass, else None."""
-        mid = ops.activate(self.up(h, torch.float32), self.rt.act_dtype, self.activation, self.act_params)
+        mid = self.up.activated(h, self.rt.act_dtype, self.activation, self.act_params)
         return self.down.add_into(mid, x, then_norm, self.rt.act_dtype, scale=self.out_scale)
 
     def produce(self, h, ctx):
         """ffn(h) in float32 (whole, or in K slices), for a block that adds it up itself."""
         if self.out_scale != 1.0:
             raise ValueError("a feed-forward that hands its result over has no multiplier of its own")
-        mid = ops.activate(self.up(h, torch.float32), self.rt.act_dtype, self.activation, self.act_params)
+        mid = self.up.activated(h, self.rt.act_dtype, self.activation, self.act_params)
         part = self.down.partial(mid) if self.down.bias is not None else None
         return self.down.raw(mid) if part is None else Joined(part, bias=self.down.bias)

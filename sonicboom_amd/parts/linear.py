@@ -96,6 +96,18 @@ class Linear:
             ops.add_scaled(resid, self(x, torch.float32), scale)      # a pass of its own over the stream
         return None
 
+    def activated(self, x: torch.Tensor, out_dtype: torch.dtype, activation: str, params: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """act(x W^T (+ b)): in the tiled product's epilogue where it knows the activation; in the pass that adds a product's K
+        slices where there are any; else in a pass of its own over the float32 product."""
+        if self.packed is not None and x.dtype == torch.bfloat16:
+            y = ops.gemm_bf16_activated(x, self.packed, self.bias, out_dtype, activation, (self.rows, self.n_in))
+            if y is not None:
+                return y
+            part = self.partial(x) if self.n_out % 4 == 0 else None
+            if part is not None and part.shape[0] <= 8 and (self.bias is None or self.bias.dtype == torch.float32):
+                return ops.activate_slices(part, out_dtype, activation, self.bias, params)
+        return ops.activate(self(x, torch.float32), out_dtype, activation, params)
+
     def gated_product(self, x: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
         """act(x Wg^T) * (x Wu^T): one fused kernel on the matrix cores, or the product in
         float32 followed by the activation kernel."""
