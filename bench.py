@@ -838,6 +838,8 @@ class AllOpsTimer:
                     elif _name == "streams_join":
                         parts = sum(1 if t[0].dim() == 2 else t[0].shape[1 if t[2] else 0] for t in args[2])
                         label = f"{_name} {args[1]} streams {parts} parts"
+                    elif _name == "activate_slices":
+                        label = f"{_name} {args[0].shape[0]}x{args[0].shape[-1]}"
                     elif _name == "gated_lru":
                         label = f"{_name} {args[6].shape[0]}x{args[6].shape[1]}"
                     elif _name == "rownorm_gate":
@@ -891,6 +893,9 @@ def design_roofline(label, us, calls, rows, depth, batch, width, cfgs):
         nbytes = rows * cfgs["gru"] * (12 + 2)
     elif label == "activate":
         nbytes = rows * cfgs["ff"] * (4 + 2)
+    elif label.startswith("activate_slices "):
+        slices, n = (int(v) for v in label.split()[1].split("x"))
+        nbytes = rows * n * (4 * slices + 2)
     elif label.startswith("activate "):
         nbytes = rows * int(label.split()[1]) * (4 + 2)
     elif label.startswith("sigmoid_mul_ "):
@@ -956,7 +961,7 @@ def design_roofline(label, us, calls, rows, depth, batch, width, cfgs):
         blocks, m = (int(v) for v in label.split()[1].split("x"))
         w = blocks * m      # x and y in, the result out; the gates' matrices; decoding: the state and its inputs both ways
         nbytes = rows * w * (8 + 2) + 4 * blocks * m * m + (2 * batch * w * 4 * 3 if decode else 0)
-        flops = 2 * rows * w * 2 * m
+        flops, peak_f = 2 * rows * w * 2 * m, VECTOR_F32_FLOPS      # (the gates' products are float32)
     elif label.startswith("rownorm_gate"):
         nbytes = rows * int(label.split()[1]) * (8 + 2)
     elif label == "rownorm_kv_store":

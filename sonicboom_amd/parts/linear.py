@@ -100,7 +100,8 @@ class Linear:
         """act(x W^T (+ b)): in the tiled product's epilogue where it knows the activation; in the pass that adds a product's K
         slices where there are any; else in a pass of its own over the float32 product."""
         if self.packed is not None and x.dtype == torch.bfloat16:
-            y = ops.gemm_bf16_activated(x, self.packed, self.bias, out_dtype, activation, (self.rows, self.n_in))
+            y = ops.gemm_bf16_activated(x, self.packed, self.bias, out_dtype, activation,
+                                        packed_shape=(self.rows, self.n_in))
             if y is not None:
                 return y
             part = self.partial(x) if self.n_out % 4 == 0 else None

@@ -657,7 +657,7 @@ def test_the_gated_recurrence_gives_the_same_bits_however_the_rows_are_cut():
 
 
 @pytest.mark.parametrize("h_dtype", [F32, BF16])
-@pytest.mark.parametrize("experts, top, groups, keep", [(8, 3, 2, 1), (6, 2, 3, 2), (64, 8, 8, 4), (200, 16, 1, 1), (12, 4, 12, 5), (130, 5, 65 // 13, 3), (4, 4, 2, 2)])
+@pytest.mark.parametrize("experts, top, groups, keep", [(10, 3, 2, 1), (6, 2, 3, 2), (64, 8, 8, 4), (200, 16, 1, 1), (12, 4, 12, 5), (130, 5, 65 // 13, 3), (4, 4, 2, 2)])
 def test_the_router_by_corrected_scores(h_dtype, experts, top, groups, keep):
     from sonicboom_amd import ops
     width, rows = 96, 300
@@ -750,7 +750,7 @@ def mixer_harness(mixer, rt_dtype, width, n_tokens_cap=64 * 20):
 
 
 LAYERS = [
-    att((6, 2, 32, 48), 90, (1e4, 16)), att((3, 3, 10, 14), 33, (77.0, 6)), att((8, 1, 64, 64), 64, (5e5, 64)), att((1, 1, 128, 128), 1, (1e4, 0)),
+    att((6, 2, 32, 48), 90, (1e4, 16)), att((3, 3, 10, 14), 33, (77.0, 6)), att((10, 2, 64, 64), 64, (5e5, 64)), att((1, 1, 128, 128), 1, (1e4, 0)),
     lin(4, 48, 32, (0.75, 0.96875, 0.998, 1.0)), lin(1, 10, 14, (0.5,)), lin(2, 200, 132, (0.9375, 0.99)), lin(2, 128, 128, (0.9, 0.9995)),
     par((4, 4, 32, 32), 40, (5e3, 32, 4.0), (96, 3, 4)), par((3, 3, 10, 14), 67, (77.0, 6, 3.0), (42, 2, 5)),
     par((8, 2, 64, 64), 128, (1e4, 32, 8.0), (256, 2, 3), scales=(1.1, -0.4)), par((2, 1, 16, 48), 130, (1e4, 8), (272, 2, 2)),

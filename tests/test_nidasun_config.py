@@ -311,7 +311,7 @@ def test_the_plain_pieces():
 
 
 def test_coded_routers_make_no_close_calls():
-    cfg = config(40, 40, 2, [lin(2, 4, 4, (0.5, 0.9), ff=(8, 12, 4, 1.0, 4, 2)), att((2, 1, 4, 4), 6, (100.0, 4), ff=(8, 8, 3, 2.0, 2, 1))],
+    cfg = config(40, 40, 2, [lin(2, 4, 4, (0.5, 0.9), ff=(8, 12, 4, 1.0, 4, 2)), att((2, 1, 4, 4), 6, (100.0, 4), ff=(8, 10, 3, 2.0, 2, 1))],
                  loop=(0, 2, 3))
     w = random_weights(cfg, seed=4, coded=True)
     gaps, chosen = [], set()
